@@ -96,14 +96,14 @@ def _free_port() -> int:
 # start FRESH children with the next rung's knobs:
 #   1. the defaults (two staggered SP halves on two streams, RCCL channel cap 16, SP chunking);
 #   2. one stream (NXD_SP_STREAMS=1: the one-pass TP + SP step);
-#   3. additionally one SP chunk, RCCL's own channel choice and normal-priority comm streams.
+#   3. additionally one SP chunk, RCCL's own channel choice.
 # The JSON line records the rung that produced it and each failed rung's exit code, reason and
 # stderr tail (the watchdog's stack / flight-recorder dump).
 LADDER = [
     ("defaults", {}),
     ("one_stream", {"NXD_SP_STREAMS": "1", "NXD_SP_STREAMS_NO_SP": "0"}),
     ("conservative", {"NXD_SP_STREAMS": "1", "NXD_SP_STREAMS_NO_SP": "0", "NXD_SP_CHUNKS": "1",
-                      "NXD_RCCL_CHANNELS": "auto", "NXD_COMM_HIGH_PRIORITY": "0"}),
+                      "NXD_RCCL_CHANNELS": "auto"}),
 ]
 if os.environ.get("NXD_BENCH_LADDER", "1") == "0":
     LADDER = LADDER[:1]   # no fallback: the defaults only

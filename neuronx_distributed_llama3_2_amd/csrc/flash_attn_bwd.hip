@@ -911,6 +911,11 @@ int64_t flash_attn_bwd_workspace(int B, int Sq, int Sk, int Hq, int Hkv, int D, 
   return n;
 }
 
+__global__ void __launch_bounds__(256) zero_fill_kernel(f32x4_t* p, int64_t n4) {
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n4; i += (int64_t)gridDim.x * 256)
+    p[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+}
+
 int flash_attn_bwd_launch(const void* q, const void* k, const void* v, const void* o, const void* dout,
                           const float* lse, float* ws, void* dq, void* dk, void* dv,
                           const int64_t* qs, const int64_t* ks, const int64_t* vs, const int64_t* os,
@@ -934,10 +939,10 @@ int flash_attn_bwd_launch(const void* q, const void* k, const void* v, const voi
   const bool slabs = slab_mode() != 0;
   float* dk_slab = slabs ? ndelta + (int64_t)B * Hq * Sq : nullptr;
   float* dv_slab = slabs ? dk_slab + (int64_t)B * Hkv * per_bh * kBlockK * D : nullptr;
-  // zeroing: one memset for the accumulators (the slabs are written whole by the kernel), or, opt-in,
+  // zeroing: one fill launch for the accumulators (the slabs are written whole by the kernel), or, opt-in,
   // the dQ rows zeroed by the prep kernel, which visits every (row, head) anyway
-  // NXD_FAB_PREP_ZERO=1 zeroes in the prep kernel instead of the memset launch: bench 3,006 / 3,016
-  // vs 2,999 / 3,007 ms per step with the memset (profiles/r4_fab_prep_zero_ab.txt), so off
+  // NXD_FAB_PREP_ZERO=1 zeroes in the prep kernel instead of a separate launch: bench 3,006 / 3,016
+  // vs 2,999 / 3,007 ms per step separately (profiles/r4_fab_prep_zero_ab.txt), so off
   static int prep_zero = -1;
   if (prep_zero < 0) {
     const char* e = getenv("NXD_FAB_PREP_ZERO");
@@ -945,7 +950,10 @@ int flash_attn_bwd_launch(const void* q, const void* k, const void* v, const voi
   }
   const bool pz = slabs && prep_zero;
   if (!pz)
-    (void)hipMemsetAsync(ws, 0, (size_t)((int64_t)B * Hq * Sq_pad * D + (slabs ? 0 : 2 * (int64_t)B * Hkv * Sk_pad * D)) * sizeof(float), stream);
+    // a kernel, not hipMemsetAsync: a training step is captured into hipGraphs, whose memset nodes
+    // have left wrong values on replays after the first (D is a multiple of 8: whole float4s)
+    hipLaunchKernelGGL(zero_fill_kernel, dim3(4096), dim3(256), 0, stream, reinterpret_cast<f32x4_t*>(ws),
+                       ((int64_t)B * Hq * Sq_pad * D + (slabs ? 0 : 2 * (int64_t)B * Hkv * Sk_pad * D)) / 4);
   float* dq_zero = pz ? dq_acc : nullptr;
 
   const int64_t nrows = (int64_t)B * Hq * Sq;

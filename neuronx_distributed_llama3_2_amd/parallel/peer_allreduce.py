@@ -269,7 +269,7 @@ class PeerCollectives:
             self.par = PeerAllReduce(self.group, nmax=cap // 4)
             self.cap = cap
             if self.stream is None:
-                self.stream = torch.cuda.Stream(priority=-1)
+                self.stream = torch.cuda.Stream()
         return self.par
 
     def _launch(self, inp, out, mode, nbytes, async_op):

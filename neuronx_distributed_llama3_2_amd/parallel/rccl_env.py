@@ -7,8 +7,6 @@ collective uses.  The chunked SP overlap (parallel_layers/sp.py) wants collectiv
 most CUs to the concurrent GEMM; a pure comm benchmark wants many channels.  Both are settable:
 
     NXD_RCCL_CHANNELS=<n>   -> NCCL_MAX_NCHANNELS = n (default 16; 0 / "auto": RCCL picks)
-    NXD_COMM_HIGH_PRIORITY  -> TP / EP groups get high-priority RCCL streams (default 1;
-                               parallel_layers/parallel_state.py)
 
 Default channel cap, from profiles/r3_cu_interference.jsonl (one MI355X: TP=8-shape GEMMs and the
 FA forward on the compute stream while a copy kernel of K workgroups -- RCCL runs one per channel --

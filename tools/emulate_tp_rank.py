@@ -39,7 +39,7 @@ class _Done:
 
 
 class _Link:
-    """Optional link-time model (--link-gbps B): every collective runs on one high-priority side
+    """Optional link-time model (--link-gbps B): every collective runs on one side
     stream (RCCL's per-communicator stream) after the producer's work, as a spin of
     bytes-on-the-wire / B followed by its receiving-side write; the consumer waits on it.  Ring
     bytes per rank: all-gather / reduce-scatter (n-1)/n of the full tensor, all-reduce twice that.
@@ -72,8 +72,8 @@ class _Link:
             self.cycles_per_s = 10_000_000 / (e0.elapsed_time(e1) / 1e3)
         self.bps = gbps * 1e9
         self.cus = max(1, int(cus))
-        self.stream = torch.cuda.Stream(priority=-1)
-        self.copy_stream = torch.cuda.Stream(priority=-1)
+        self.stream = torch.cuda.Stream()
+        self.copy_stream = torch.cuda.Stream()
         self.src = torch.zeros(self.cus * 4096, dtype=torch.uint8, device="cuda")
         self.dst = torch.empty_like(self.src)
         self.busy_s = 0.0
