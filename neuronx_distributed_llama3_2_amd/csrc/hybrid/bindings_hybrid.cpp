@@ -1,0 +1,296 @@
+// Python bindings of the hybrid-decoder kernels (module `neuronx_distributed_llama3_2_amd._hybrid`).
+// Every entry point checks shapes, types and the kernels' size limits on the host before it launches
+// on the caller's current stream.
+#include <torch/extension.h>
+#include <ATen/hip/HIPContext.h>
+#include <hip/hip_runtime.h>
+
+#include "delta_rule.h"
+#include "window_attn.h"
+
+void register_gemm(pybind11::module& m);  // ../gemm.cpp
+
+namespace nxd {
+int hyper_step_launch(bool, float*, const void*, const int64_t*, int64_t, const void*, int64_t, const float*, const float*,
+                      const float*, const float*, const float*, float, void*, int64_t, const int64_t*, bool, int64_t, int,
+                      int, hipStream_t);
+int relu_squared_launch(bool, const void*, void*, int64_t, hipStream_t);
+int softcap_launch(float*, int64_t, float, hipStream_t);
+int delta_prep_launch(bool, const DeltaParams&, hipStream_t);
+int delta_scan_launch(bool, const DeltaParams&, hipStream_t);
+int delta_out_launch(bool, const DeltaParams&, hipStream_t);
+int delta_decode_launch(bool, const DeltaParams&, hipStream_t);
+int attn_prep_launch(bool, const WindowAttnParams&, hipStream_t);
+int attn_row_launch(bool, const WindowAttnParams&, hipStream_t);
+}  // namespace nxd
+
+namespace {
+
+using at::Tensor;
+using Opt = c10::optional<Tensor>;
+
+hipStream_t cur_stream() { return at::hip::getCurrentHIPStream().stream(); }
+void check_rc(int rc, const char* what) { TORCH_CHECK(rc == 0, what, " failed with code ", rc); }
+
+// activation tensors: bf16 or fp32, unit inner stride
+bool act_f32(const Tensor& t, const char* n) {
+  TORCH_CHECK(t.is_cuda() && t.dim() >= 2 && t.stride(-1) == 1, n, ": GPU tensor with a unit inner stride");
+  TORCH_CHECK(t.scalar_type() == at::kBFloat16 || t.scalar_type() == at::kFloat, n, ": bf16 or fp32");
+  return t.scalar_type() == at::kFloat;
+}
+void same_act(const Tensor& t, const Tensor& like, const char* n) {
+  act_f32(t, n);
+  TORCH_CHECK(t.scalar_type() == like.scalar_type(), n, ": activation type differs");
+}
+float* f32_ptr(const Tensor& t, int64_t numel, const char* n) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kFloat && t.is_contiguous() && t.numel() == numel, n,
+              ": contiguous fp32 of ", numel, " elements");
+  return t.data_ptr<float>();
+}
+float* f32_opt(const Opt& t, int64_t numel, const char* n) { return t.has_value() ? f32_ptr(*t, numel, n) : nullptr; }
+const int* i32_opt(const Opt& t, int64_t numel, const char* n) {
+  if (!t.has_value()) return nullptr;
+  TORCH_CHECK(t->is_cuda() && t->scalar_type() == at::kInt && t->is_contiguous() && t->numel() == numel, n,
+              ": contiguous int32 of ", numel, " elements");
+  return t->data_ptr<int>();
+}
+// first position of every sequence: int64 [B] or [B, T'] (column 0)
+const int64_t* pos_ptr(const Tensor& t, int64_t B, int64_t* stride) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kLong && t.dim() >= 1 && t.dim() <= 2 && t.size(0) == B,
+              "positions: int64 [B] or [B, T]");
+  *stride = B > 1 ? t.stride(0) : 0;
+  return t.data_ptr<int64_t>();
+}
+void check_align(const Tensor& t, const char* n) {
+  TORCH_CHECK(reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0, n, ": 16-byte alignment");
+}
+
+void hyper_step(Tensor x, Opt embed, Opt ids, Opt y, Opt bias, Opt mix, Opt write, Opt read, Opt norm_w, double eps, Opt h,
+                Opt rows, bool store) {
+  TORCH_CHECK(x.dim() == 3 && x.is_cuda() && x.scalar_type() == at::kFloat && x.is_contiguous(), "hyper_step: x fp32 [M, S, W]");
+  const int64_t M = x.size(0), S = x.size(1), W = x.size(2);
+  TORCH_CHECK(S >= 1 && S <= 8, "hyper_step: 1..8 streams");
+  TORCH_CHECK(W >= 1 && W <= 16384, "hyper_step: width up to 16384");
+  TORCH_CHECK(h.has_value() == read.has_value() && h.has_value() == norm_w.has_value(), "hyper_step: read, norm and h together");
+  TORCH_CHECK(h.has_value() || y.has_value(), "hyper_step: nothing to do");
+  check_align(x, "x");
+  bool f32 = false, have = false;
+  auto act = [&](const Tensor& t, const char* n) {
+    const bool f = act_f32(t, n);
+    TORCH_CHECK(!have || f == f32, "hyper_step: activation types differ");
+    f32 = f;
+    have = true;
+    check_align(t, n);
+  };
+  const int64_t R = rows.has_value() ? rows->numel() : M;
+  if (rows.has_value()) {
+    TORCH_CHECK(rows->is_cuda() && rows->scalar_type() == at::kLong && rows->is_contiguous(), "hyper_step: int64 rows");
+    TORCH_CHECK(!store, "hyper_step: selected rows are only read");
+  }
+  if (embed.has_value()) {
+    act(*embed, "embed");
+    TORCH_CHECK(embed->is_contiguous() && embed->dim() == 2 && embed->size(1) == W, "hyper_step: embed [V, W]");
+    TORCH_CHECK(ids.has_value() && ids->is_cuda() && ids->scalar_type() == at::kLong && ids->is_contiguous() && ids->numel() == M,
+                "hyper_step: int64 ids [M]");
+  }
+  int64_t ldy = 0, ldh = 0;
+  if (y.has_value()) {
+    act(*y, "y");
+    TORCH_CHECK(y->dim() == 2 && y->size(0) == M && y->size(1) == W, "hyper_step: y [M, W]");
+    TORCH_CHECK(mix.has_value() && write.has_value(), "hyper_step: mix and write with y");
+    ldy = y->stride(0);
+  }
+  if (h.has_value()) {
+    act(*h, "h");
+    TORCH_CHECK(h->dim() == 2 && h->size(0) == R && h->size(1) == W, "hyper_step: h [R, W]");
+    ldh = h->stride(0);
+  }
+  check_rc(nxd::hyper_step_launch(f32, x.data_ptr<float>(), embed.has_value() ? embed->data_ptr() : nullptr,
+                                  embed.has_value() ? ids->data_ptr<int64_t>() : nullptr,
+                                  embed.has_value() ? embed->size(0) : 0, y.has_value() ? y->data_ptr() : nullptr, ldy,
+                                  f32_opt(bias, W, "bias"), f32_opt(mix, S * S, "mix"), f32_opt(write, S, "write"),
+                                  f32_opt(read, S, "read"), f32_opt(norm_w, W, "norm_w"), (float)eps,
+                                  h.has_value() ? h->data_ptr() : nullptr, ldh,
+                                  rows.has_value() ? rows->data_ptr<int64_t>() : nullptr, store, R, (int)S, (int)W,
+                                  cur_stream()),
+           "hyper_step");
+}
+
+void relu_squared(Tensor x, Tensor y) {
+  const bool f32 = act_f32(x, "x");
+  same_act(y, x, "y");
+  TORCH_CHECK(x.is_contiguous() && y.is_contiguous() && x.numel() == y.numel(), "relu_squared: contiguous, equal sizes");
+  check_align(x, "x");
+  check_align(y, "y");
+  check_rc(nxd::relu_squared_launch(f32, x.data_ptr(), y.data_ptr(), x.numel(), cur_stream()), "relu_squared");
+}
+
+void softcap_(Tensor x, double cap) {
+  TORCH_CHECK(x.is_cuda() && x.scalar_type() == at::kFloat && x.is_contiguous() && cap > 0, "softcap_: contiguous fp32, cap > 0");
+  check_rc(nxd::softcap_launch(x.data_ptr<float>(), x.numel(), (float)cap, cur_stream()), "softcap_");
+}
+
+// The recurrence over T new tokens of B sequences.  one launch (T == 1 and `fused`) or three with the
+// fp32 intermediates; sizes (H, G, D, V).
+void delta_rule(Tensor proj, int64_t B, int64_t T, std::vector<int64_t> sizes, Tensor conv, Tensor a_log, Tensor dt_bias,
+                Tensor norm_w, double eps, Tensor pos, Opt lens, Opt slots, Tensor state, Tensor ring, Tensor y, bool fused) {
+  const bool f32 = act_f32(proj, "proj");
+  same_act(ring, proj, "ring");
+  same_act(y, proj, "y");
+  TORCH_CHECK(sizes.size() == 4, "delta_rule: sizes (H, G, D, V)");
+  nxd::DeltaParams p{};
+  p.B = (int)B;
+  p.T = (int)T;
+  p.H = (int)sizes[0];
+  p.G = (int)sizes[1];
+  p.D = (int)sizes[2];
+  p.V = (int)sizes[3];
+  TORCH_CHECK(B >= 1 && T >= 1 && B * T <= (1 << 30), "delta_rule: rows");
+  TORCH_CHECK(p.G >= 1 && p.H >= 1 && p.H % p.G == 0 && p.H <= 65535 && B <= 65535, "delta_rule: head layout");
+  TORCH_CHECK(p.D >= 1 && p.D <= 256 && p.V >= 1 && p.V <= 256, "delta_rule: head sizes up to 256");
+  p.DP = (p.D + 31) / 32 * 32;
+  p.C = 2 * p.G * p.D + p.H * p.V;
+  TORCH_CHECK(conv.dim() == 2 && conv.size(1) == p.C && conv.size(0) >= 1, "delta_rule: conv [taps, C]");
+  p.taps = (int)conv.size(0);
+  TORCH_CHECK(proj.dim() == 2 && proj.size(0) == B * T && proj.size(1) >= p.C + p.H * p.V + 2 * p.H, "delta_rule: proj columns");
+  TORCH_CHECK(y.dim() == 2 && y.size(0) == B * T && y.size(1) == p.H * p.V, "delta_rule: y [B T, H V]");
+  TORCH_CHECK(state.dim() == 4 && state.is_contiguous() && state.scalar_type() == at::kFloat && state.is_cuda() &&
+                  state.size(1) == p.H && state.size(2) == p.V && state.size(3) == p.DP,
+              "delta_rule: state fp32 [slots, H, V, D rounded up to 32]");
+  const int64_t ns = state.size(0);
+  TORCH_CHECK(ring.is_contiguous() && ring.dim() == 3 && ring.size(0) == ns && ring.size(1) == p.taps && ring.size(2) == p.C,
+              "delta_rule: ring [slots, taps, C]");
+  TORCH_CHECK(slots.has_value() || B <= ns, "delta_rule: more sequences than slots");
+  check_align(state, "state");
+  p.proj = proj.data_ptr();
+  p.ldp = proj.stride(0);
+  p.conv = f32_ptr(conv, (int64_t)p.taps * p.C, "conv");
+  p.a_log = f32_ptr(a_log, p.H, "a_log");
+  p.dt_bias = f32_ptr(dt_bias, p.H, "dt_bias");
+  p.norm_w = f32_ptr(norm_w, p.V, "norm_w");
+  p.qscale = (float)(1.0 / std::sqrt((double)p.D));
+  p.eps = (float)eps;
+  p.pos = pos_ptr(pos, B, &p.pos_stride);
+  p.lens = i32_opt(lens, B, "lens");
+  p.slots = i32_opt(slots, B, "slots");
+  p.nslots = (int)ns;
+  p.state = state.data_ptr<float>();
+  p.ring = ring.data_ptr();
+  p.y = y.data_ptr();
+  p.ldy = y.stride(0);
+  if (fused && T == 1 && !lens.has_value()) {
+    check_rc(nxd::delta_decode_launch(f32, p, cur_stream()), "delta_decode");
+    return;
+  }
+  auto opt = proj.options().dtype(at::kFloat);
+  const int64_t M = B * T;
+  Tensor qk = at::empty({2, M, p.G, p.D}, opt), vo = at::empty({2, M, p.H, p.V}, opt), gb = at::empty({2, M, p.H}, opt);
+  p.qn = qk.data_ptr<float>();
+  p.kn = p.qn + M * p.G * p.D;
+  p.vn = vo.data_ptr<float>();
+  p.o = p.vn + M * p.H * p.V;
+  p.lg = gb.data_ptr<float>();
+  p.beta = p.lg + M * p.H;
+  check_rc(nxd::delta_prep_launch(f32, p, cur_stream()), "delta_prep");
+  check_rc(nxd::delta_scan_launch(f32, p, cur_stream()), "delta_scan");
+  check_rc(nxd::delta_out_launch(f32, p, cur_stream()), "delta_out");
+}
+
+// sizes (H, G, maps, D, V)
+nxd::WindowAttnParams attn_params(const Tensor& buf, int64_t B, int64_t T, const std::vector<int64_t>& sizes,
+                                  const Tensor& pos, const Opt& lens, const Opt& slots, const Tensor& kc, const Tensor& vc) {
+  act_f32(buf, "buf");
+  same_act(kc, buf, "k cache");
+  same_act(vc, buf, "v cache");
+  TORCH_CHECK(sizes.size() == 5, "attention: sizes (H, G, maps, D, V)");
+  nxd::WindowAttnParams p{};
+  p.B = (int)B;
+  p.T = (int)T;
+  p.H = (int)sizes[0];
+  p.G = (int)sizes[1];
+  p.maps = (int)sizes[2];
+  p.D = (int)sizes[3];
+  p.V = (int)sizes[4];
+  TORCH_CHECK(B >= 1 && T >= 1 && B * T <= (1 << 30), "attention: rows");
+  TORCH_CHECK(p.G >= 1 && p.H % p.G == 0 && p.H >= 1 && (p.maps == 1 || p.maps == 2), "attention: head layout");
+  TORCH_CHECK(p.D >= 2 && p.D <= 256 && p.V >= 1 && p.V <= 256, "attention: head sizes up to 256");
+  TORCH_CHECK(buf.dim() == 2 && buf.size(0) == B * T && buf.size(1) >= (p.H + p.G) * p.maps * p.D + p.G * p.V,
+              "attention: projection columns");
+  TORCH_CHECK(kc.dim() == 4 && kc.is_contiguous() && kc.size(1) == p.G * p.maps && kc.size(3) == p.D,
+              "attention: k cache [slots, G maps, cap, D]");
+  TORCH_CHECK(vc.dim() == 4 && vc.is_contiguous() && vc.size(0) == kc.size(0) && vc.size(1) == p.G && vc.size(2) == kc.size(2) &&
+                  vc.size(3) == p.V,
+              "attention: v cache [slots, G, cap, V]");
+  TORCH_CHECK(kc.size(2) >= 1 && kc.size(2) < (1 << 30), "attention: cache length");
+  TORCH_CHECK(slots.has_value() || B <= kc.size(0), "attention: more sequences than slots");
+  p.buf = buf.data_ptr();
+  p.ldb = buf.stride(0);
+  p.pos = pos_ptr(pos, B, &p.pos_stride);
+  p.lens = i32_opt(lens, B, "lens");
+  p.slots = i32_opt(slots, B, "slots");
+  p.nslots = (int)kc.size(0);
+  p.kc = kc.data_ptr();
+  p.vc = vc.data_ptr();
+  p.cap = (int)kc.size(2);
+  return p;
+}
+
+void attn_prep(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, Opt bias, Opt qn_w, Opt kn_w, double eps,
+               Tensor cos_t, Tensor sin_t, Tensor pos, Opt lens, Opt slots, Tensor kc, Tensor vc) {
+  auto p = attn_params(buf, B, T, sizes, pos, lens, slots, kc, vc);
+  p.bias = f32_opt(bias, (p.H + p.G) * p.maps * p.D + p.G * p.V, "bias");
+  TORCH_CHECK(qn_w.has_value() == kn_w.has_value(), "attn_prep: both head norms or none");
+  p.qn_w = f32_opt(qn_w, p.D, "qn_w");
+  p.kn_w = f32_opt(kn_w, p.D, "kn_w");
+  p.eps = (float)eps;
+  TORCH_CHECK(cos_t.dim() == 2 && cos_t.sizes() == sin_t.sizes() && cos_t.size(0) >= 1 && 2 * cos_t.size(1) <= p.D,
+              "attn_prep: cos / sin [positions, rotated pairs]");
+  p.cos_t = f32_ptr(cos_t, cos_t.numel(), "cos");
+  p.sin_t = f32_ptr(sin_t, sin_t.numel(), "sin");
+  p.rot = 2 * (int)cos_t.size(1);
+  p.max_pos = (int)cos_t.size(0);
+  check_rc(nxd::attn_prep_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "attn_prep");
+}
+
+// from_buf: the new tokens start at position 0 and see only each other
+void window_attn(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, double scale, double softcap, int64_t window,
+                 double lam, double out_scale, double out_eps, Tensor pos, Opt lens, Opt slots, Tensor kc, Tensor vc, Tensor y,
+                 bool from_buf) {
+  auto p = attn_params(buf, B, T, sizes, pos, lens, slots, kc, vc);
+  same_act(y, buf, "y");
+  TORCH_CHECK(y.dim() == 2 && y.size(0) == B * T && y.size(1) == p.H * p.V, "window_attn: y [B T, H V]");
+  TORCH_CHECK(from_buf || window <= 0 || T <= p.cap - window + 1, "window_attn: ", T, " new tokens do not fit a ring of ", p.cap,
+              " with a window of ", window);
+  p.scale = (float)scale;
+  p.softcap = (float)softcap;
+  p.window = window > 0 && window < (1 << 30) ? (int)window : 0;
+  p.lam = (float)lam;
+  p.out_scale = (float)out_scale;
+  p.out_eps = (float)out_eps;
+  p.y = y.data_ptr();
+  p.ldy = y.stride(0);
+  p.from_buf = from_buf ? 1 : 0;
+  check_rc(nxd::attn_row_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "window_attn");
+}
+
+}  // namespace
+
+PYBIND11_MODULE(_hybrid, m) {
+  register_gemm(m);
+  namespace py = pybind11;
+  m.def("hyper_step", &hyper_step, py::arg("x"), py::arg("embed") = py::none(), py::arg("ids") = py::none(),
+        py::arg("y") = py::none(), py::arg("bias") = py::none(), py::arg("mix") = py::none(), py::arg("write") = py::none(),
+        py::arg("read") = py::none(), py::arg("norm_w") = py::none(), py::arg("eps") = 0.0, py::arg("h") = py::none(),
+        py::arg("rows") = py::none(), py::arg("store") = true);
+  m.def("relu_squared", &relu_squared);
+  m.def("softcap_", &softcap_);
+  m.def("delta_rule", &delta_rule, py::arg("proj"), py::arg("B"), py::arg("T"), py::arg("sizes"), py::arg("conv"),
+        py::arg("a_log"), py::arg("dt_bias"), py::arg("norm_w"), py::arg("eps"), py::arg("pos"), py::arg("lens"),
+        py::arg("slots"), py::arg("state"), py::arg("ring"), py::arg("y"), py::arg("fused") = true);
+  m.def("attn_prep", &attn_prep, py::arg("buf"), py::arg("B"), py::arg("T"), py::arg("sizes"), py::arg("bias"),
+        py::arg("qn_w"), py::arg("kn_w"), py::arg("eps"), py::arg("cos"), py::arg("sin"), py::arg("pos"), py::arg("lens"),
+        py::arg("slots"), py::arg("kc"), py::arg("vc"));
+  m.def("window_attn", &window_attn, py::arg("buf"), py::arg("B"), py::arg("T"), py::arg("sizes"), py::arg("scale"),
+        py::arg("softcap"), py::arg("window"), py::arg("lam"), py::arg("out_scale"), py::arg("out_eps"), py::arg("pos"),
+        py::arg("lens"), py::arg("slots"), py::arg("kc"), py::arg("vc"), py::arg("y"), py::arg("from_buf"));
+}

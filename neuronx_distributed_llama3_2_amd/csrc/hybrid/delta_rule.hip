@@ -1,0 +1,333 @@
+// Gated delta rule (a linear-attention recurrence with a matrix state per head):
+//
+//   q, k, v <- silu(causal conv of the projections); q, k unit vectors per head (q also * D^-1/2)
+//   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+//   y = o / rms(o) * norm_w * silu(gate)                        (per head, over its V values)
+//
+// Everything here after the projections is computed in fp32.  The state of a sequence lives in the
+// cache: S as [slot][H][V][DP] fp32 (DP = D rounded up to 32, the padding stays zero), and the
+// convolution's inputs as a ring [slot][taps][C] in the activation type, position p in entry p % taps.
+// Whether a token has a predecessor is decided by its position, so a slot needs no clearing before it
+// is used again.  The projection buffer's columns are [q (G D) | k (G D) | v (H V) | gate (H V) |
+// beta (H) | decay (H)].
+//
+//   delta_prep   : convolution, silu, unit norms, gates of all tokens of a step (one workgroup a row)
+//   delta_scan   : the recurrence, token by token, from the cached state (8 lanes a state column)
+//   delta_out    : the gated head norm
+//   delta_decode : all of it for one new token per sequence, one workgroup per (sequence, head)
+#include "hybrid.h"
+#include "delta_rule.h"
+
+namespace nxd {
+namespace hybrid {
+
+// convolution + silu of one channel for the token of row m (position ps): earlier tokens of this
+// step come from the projection buffer, older ones from the ring
+template <typename T>
+__device__ __forceinline__ float conv_silu(const DeltaParams& p, const T* proj, const T* ring, int64_t m, int t,
+                                           int64_t ps, int c) {
+  const int C = p.C, n = p.taps;
+  float a = 0.f;
+  for (int j = 0; j < n; ++j) {
+    const int back = n - 1 - j;
+    const int64_t q = ps - back;
+    if (q < 0) continue;
+    const float x = back <= t ? ld(proj + (m - back) * p.ldp + c) : ld(ring + (q % n) * C + c);
+    a += p.conv[(int64_t)j * C + c] * x;
+  }
+  return siluf_(a);
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256) delta_prep_kernel(DeltaParams p) {
+  const int64_t m = blockIdx.x;
+  const int b = (int)(m / p.T), t = (int)(m % p.T);
+  if (p.lens && t >= p.lens[b]) return;
+  const int64_t ps = pos_of(p.pos, p.pos_stride, b) + t;
+  const int slot = slot_of(p.slots, b, p.nslots);
+  const T* proj = static_cast<const T*>(p.proj);
+  const T* ring = static_cast<const T*>(p.ring) + (int64_t)slot * p.taps * p.C;
+  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+  const int G = p.G, D = p.D, H = p.H, HV = p.H * p.V;
+  for (int hd = wid; hd < 2 * G; hd += 4) {   // q heads, then k heads: a wave per unit vector
+    float x[4], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = lane + 64 * i;
+      x[i] = d < D ? conv_silu<T>(p, proj, ring, m, t, ps, hd * D + d) : 0.f;
+      ss += x[i] * x[i];
+    }
+    ss = wave_sum(ss);
+    float r = 1.f / sqrtf(ss + 1e-6f);
+    if (hd < G) r *= p.qscale;
+    float* out = (hd < G ? p.qn : p.kn) + (m * G + (hd < G ? hd : hd - G)) * D;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int d = lane + 64 * i;
+      if (d < D) out[d] = x[i] * r;
+    }
+  }
+  float* vo = p.vn + m * HV;
+  for (int c = tid; c < HV; c += 256) vo[c] = conv_silu<T>(p, proj, ring, m, t, ps, 2 * G * D + c);
+  const T* gates = proj + m * p.ldp + p.C + HV;
+  for (int h = tid; h < H; h += 256) {
+    p.beta[m * H + h] = sigmoidf_(ld(gates + h));
+    p.lg[m * H + h] = -expf(p.a_log[h]) * softplusf_(ld(gates + H + h) + p.dt_bias[h]);
+  }
+}
+
+// ---- the recurrence, one token after another.  A workgroup owns 32 columns of one head's state
+// (8 lanes a column, NI float4 of the column's DP entries each).
+template <typename T, int NI>
+__global__ void __launch_bounds__(256) delta_scan_kernel(DeltaParams p) {
+  constexpr int TK = 16, DP = NI * 32;
+  __shared__ __attribute__((aligned(16))) float ks[TK][DP], qs[TK][DP];
+  __shared__ float vs[TK][32], gs[TK], bs[TK];
+  const int tid = threadIdx.x, l = tid & 7, col = tid >> 3;
+  const int h = blockIdx.y, b = blockIdx.z, v = blockIdx.x * 32 + col;
+  const int H = p.H, G = p.G, D = p.D, V = p.V, g = h / (H / G);
+  const int len = p.lens ? min(p.lens[b], p.T) : p.T;
+  if (len <= 0) return;
+  const int slot = slot_of(p.slots, b, p.nslots);
+  const int64_t p0 = pos_of(p.pos, p.pos_stride, b);
+  float* state = p.state + (((int64_t)slot * H + h) * V + min(v, V - 1)) * DP;
+  f32x4_t S[NI];
+#pragma unroll
+  for (int i = 0; i < NI; ++i) S[i] = p0 > 0 ? ld4(state + i * 32 + l * 4) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const int64_t m0 = (int64_t)b * p.T;
+  for (int t0 = 0; t0 < len; t0 += TK) {
+    const int n = min(TK, len - t0);
+    __syncthreads();
+    for (int i = tid; i < n * DP; i += 256) {
+      const int t = i / DP, d = i % DP;
+      const int64_t o = ((m0 + t0 + t) * G + g) * D + d;
+      ks[t][d] = d < D ? p.kn[o] : 0.f;
+      qs[t][d] = d < D ? p.qn[o] : 0.f;
+    }
+    for (int i = tid; i < n * 32; i += 256) {
+      const int t = i >> 5, c = blockIdx.x * 32 + (i & 31);
+      vs[t][i & 31] = c < V ? p.vn[((m0 + t0 + t) * H + h) * V + c] : 0.f;
+    }
+    if (tid < n) {
+      gs[tid] = expf(p.lg[(m0 + t0 + tid) * H + h]);
+      bs[tid] = p.beta[(m0 + t0 + tid) * H + h];
+    }
+    __syncthreads();
+    for (int t = 0; t < n; ++t) {
+      const float gt = gs[t];
+      f32x4_t k[NI];
+      float dot = 0.f;
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        k[i] = ld4(&ks[t][i * 32 + l * 4]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          S[i][e] *= gt;
+          dot += S[i][e] * k[i][e];
+        }
+      }
+#pragma unroll
+      for (int o = 4; o > 0; o >>= 1) dot += __shfl_xor(dot, o, 64);
+      const float u = bs[t] * (vs[t][col] - dot);
+      float out = 0.f;
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        const f32x4_t q = ld4(&qs[t][i * 32 + l * 4]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          S[i][e] += k[i][e] * u;
+          out += S[i][e] * q[e];
+        }
+      }
+#pragma unroll
+      for (int o = 4; o > 0; o >>= 1) out += __shfl_xor(out, o, 64);
+      if (l == 0 && v < V) p.o[((m0 + t0 + t) * H + h) * V + v] = out;
+    }
+  }
+  if (v < V) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) st4(state + i * 32 + l * 4, S[i]);
+  }
+  if (blockIdx.x == 0 && h == 0) ring_write<T>(p, b, slot, p0, len, tid, 256);
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256) delta_out_kernel(DeltaParams p) {
+  const int lane = threadIdx.x & 63;
+  const int64_t i = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);   // (row, head)
+  const int H = p.H, V = p.V;
+  if (i >= (int64_t)p.B * p.T * H) return;
+  const int64_t m = i / H;
+  const int h = (int)(i % H);
+  T* y = static_cast<T*>(p.y) + m * p.ldy + h * V;
+  if (p.lens && (int)(m % p.T) >= p.lens[m / p.T]) {   // padding: a defined value for the projection
+    for (int v = lane; v < V; v += 64) st(y + v, 0.f);
+    return;
+  }
+  const float* o = p.o + i * V;
+  const T* gate = static_cast<const T*>(p.proj) + m * p.ldp + p.C + h * V;
+  float x[4], ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int v = lane + 64 * j;
+    x[j] = v < V ? o[v] : 0.f;
+    ss += x[j] * x[j];
+  }
+  const float r = 1.f / sqrtf(wave_sum(ss) / (float)V + p.eps);
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int v = lane + 64 * j;
+    if (v < V) st(y + v, x[j] * r * p.norm_w[v] * siluf_(ld(gate + v)));
+  }
+}
+
+// ---- one new token per sequence: a workgroup of NTH threads per (head, sequence)
+template <typename T, int NI, int NTH>
+__global__ void __launch_bounds__(NTH) delta_decode_kernel(DeltaParams p) {
+  constexpr int DP = NI * 32, COLS = NTH / 8;
+  __shared__ __attribute__((aligned(16))) float qs[DP], ks[DP];
+  __shared__ float vs[256], os[256], red[16];
+  const int tid = threadIdx.x, l = tid & 7, col = tid >> 3;
+  const int h = blockIdx.x, b = blockIdx.y;
+  const int H = p.H, G = p.G, D = p.D, V = p.V, rep = H / G, g = h / rep, C = p.C;
+  const int slot = slot_of(p.slots, b, p.nslots);
+  const int64_t ps = pos_of(p.pos, p.pos_stride, b);
+  const T* proj = static_cast<const T*>(p.proj);
+  T* ring = static_cast<T*>(p.ring) + (int64_t)slot * p.taps * C;
+  float* state = p.state + ((int64_t)slot * H + h) * V * DP;
+  // the first columns of the state are on their way while the inputs are prepared
+  f32x4_t S[NI];
+  {
+    const float* sp = state + (int64_t)min(col, V - 1) * DP;
+#pragma unroll
+    for (int i = 0; i < NI; ++i) S[i] = ld4(sp + i * 32 + l * 4);
+  }
+  T* entry = ring + (ps % p.taps) * C;   // this token's ring entry: read by nobody in this launch
+  float sq = 0.f, sk = 0.f;
+  for (int i = tid; i < 2 * DP + V; i += NTH) {
+    const int part = i < DP ? 0 : (i < 2 * DP ? 1 : 2);
+    const int d = part == 0 ? i : (part == 1 ? i - DP : i - 2 * DP);
+    float x = 0.f;
+    if (part == 2 || d < D) {
+      const int c = part == 0 ? g * D + d : (part == 1 ? (G + g) * D + d : 2 * G * D + h * V + d);
+      x = conv_silu<T>(p, proj, ring, b, 0, ps, c);
+      if (part == 2 || h % rep == 0) entry[c] = proj[(int64_t)b * p.ldp + c];
+    }
+    if (part == 0) { qs[d] = x; sq += x * x; }
+    else if (part == 1) { ks[d] = x; sk += x * x; }
+    else vs[d] = x;
+  }
+  const float rq = p.qscale / sqrtf(block_sum(sq, red) + 1e-6f);
+  const float rk = 1.f / sqrtf(block_sum(sk, red) + 1e-6f);
+  const T* gates = proj + (int64_t)b * p.ldp + C + H * V;
+  const float beta = sigmoidf_(ld(gates + h));
+  const float gt = expf(-expf(p.a_log[h]) * softplusf_(ld(gates + H + h) + p.dt_bias[h]));
+  f32x4_t k[NI], q[NI];
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    k[i] = ld4(&ks[i * 32 + l * 4]) * rk;
+    q[i] = ld4(&qs[i * 32 + l * 4]) * rq;
+  }
+  for (int v = col; v < V; v += COLS) {
+    float* sp = state + (int64_t)v * DP;
+    if (v != col) {
+#pragma unroll
+      for (int i = 0; i < NI; ++i) S[i] = ld4(sp + i * 32 + l * 4);
+    }
+    float dot = 0.f;
+#pragma unroll
+    for (int i = 0; i < NI; ++i)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        S[i][e] = ps > 0 ? S[i][e] * gt : 0.f;   // a sequence's first token starts from zero
+        dot += S[i][e] * k[i][e];
+      }
+#pragma unroll
+    for (int o = 4; o > 0; o >>= 1) dot += __shfl_xor(dot, o, 64);
+    const float u = beta * (vs[v] - dot);
+    float out = 0.f;
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        S[i][e] += k[i][e] * u;
+        out += S[i][e] * q[i][e];
+      }
+      st4(sp + i * 32 + l * 4, S[i]);
+    }
+#pragma unroll
+    for (int o = 4; o > 0; o >>= 1) out += __shfl_xor(out, o, 64);
+    if (l == 0) os[v] = out;
+  }
+  __syncthreads();
+  float ss = 0.f;
+  for (int v = tid; v < V; v += NTH) ss += os[v] * os[v];
+  const float r = 1.f / sqrtf(block_sum(ss, red) / (float)V + p.eps);
+  T* y = static_cast<T*>(p.y) + (int64_t)b * p.ldy + h * V;
+  const T* gate = proj + (int64_t)b * p.ldp + C + h * V;
+  for (int v = tid; v < V; v += NTH) st(y + v, os[v] * r * p.norm_w[v] * siluf_(ld(gate + v)));
+}
+
+#define NXD_BY_NI(CALL)                                                     \
+  switch (p.DP / 32) {                                                      \
+    case 1: CALL(1); break;                                                 \
+    case 2: CALL(2); break;                                                 \
+    case 3: CALL(3); break;                                                 \
+    case 4: CALL(4); break;                                                 \
+    case 5: CALL(5); break;                                                 \
+    case 6: CALL(6); break;                                                 \
+    case 7: CALL(7); break;                                                 \
+    case 8: CALL(8); break;                                                 \
+    default: return -1;                                                     \
+  }
+
+template <typename T>
+static int run_prep(const DeltaParams& p, hipStream_t s) {
+  hipLaunchKernelGGL((delta_prep_kernel<T>), dim3((unsigned)(p.B * p.T)), dim3(256), 0, s, p);
+  return hipGetLastError() == hipSuccess ? 0 : 1;
+}
+template <typename T>
+static int run_scan(const DeltaParams& p, hipStream_t s) {
+  const dim3 grid((unsigned)ceil_div(p.V, 32), (unsigned)p.H, (unsigned)p.B);
+#define NXD_CALL(N) hipLaunchKernelGGL((delta_scan_kernel<T, N>), grid, dim3(256), 0, s, p)
+  NXD_BY_NI(NXD_CALL)
+#undef NXD_CALL
+  return hipGetLastError() == hipSuccess ? 0 : 1;
+}
+template <typename T>
+static int run_out(const DeltaParams& p, hipStream_t s) {
+  const int64_t n = (int64_t)p.B * p.T * p.H;
+  hipLaunchKernelGGL((delta_out_kernel<T>), dim3((unsigned)ceil_div64(n, 4)), dim3(256), 0, s, p);
+  return hipGetLastError() == hipSuccess ? 0 : 1;
+}
+template <typename T>
+static int run_decode(const DeltaParams& p, hipStream_t s) {
+  const dim3 grid((unsigned)p.H, (unsigned)p.B);
+  if (p.V > 64) {
+#define NXD_CALL(N) hipLaunchKernelGGL((delta_decode_kernel<T, N, 1024>), grid, dim3(1024), 0, s, p)
+    NXD_BY_NI(NXD_CALL)
+#undef NXD_CALL
+  } else {
+#define NXD_CALL(N) hipLaunchKernelGGL((delta_decode_kernel<T, N, 256>), grid, dim3(256), 0, s, p)
+    NXD_BY_NI(NXD_CALL)
+#undef NXD_CALL
+  }
+  return hipGetLastError() == hipSuccess ? 0 : 1;
+}
+
+}  // namespace hybrid
+
+int delta_prep_launch(bool f32, const DeltaParams& p, hipStream_t s) {
+  return f32 ? hybrid::run_prep<float>(p, s) : hybrid::run_prep<uint16_t>(p, s);
+}
+int delta_scan_launch(bool f32, const DeltaParams& p, hipStream_t s) {
+  return f32 ? hybrid::run_scan<float>(p, s) : hybrid::run_scan<uint16_t>(p, s);
+}
+int delta_out_launch(bool f32, const DeltaParams& p, hipStream_t s) {
+  return f32 ? hybrid::run_out<float>(p, s) : hybrid::run_out<uint16_t>(p, s);
+}
+int delta_decode_launch(bool f32, const DeltaParams& p, hipStream_t s) {
+  return f32 ? hybrid::run_decode<float>(p, s) : hybrid::run_decode<uint16_t>(p, s);
+}
+
+}  // namespace nxd

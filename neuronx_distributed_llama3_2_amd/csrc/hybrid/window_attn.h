@@ -1,0 +1,38 @@
+// Parameters of the windowed / differential attention kernels (csrc/hybrid/window_attn*.hip).
+#pragma once
+#include "hybrid.h"
+
+namespace nxd {
+
+struct WindowAttnParams {
+  int B, T;               // sequences, new tokens per sequence (row b * T + t)
+  int H, G, maps, D, V;   // query heads, key/value heads, maps per head (1: plain, 2: differential), sizes
+  void* buf;              // [B T, ldb]: q (H maps D) | k (G maps D) | v (G V), activation type
+  int64_t ldb;
+  const int64_t* pos;     // position of each sequence's first new token: pos[b * pos_stride]
+  int64_t pos_stride;
+  const int* lens;        // [B] valid new tokens (nullable: T)
+  const int* slots;       // [B] cache slots (nullable: identity)
+  int nslots;
+  void* kc;               // [slots, G maps, cap, D] ring by position: p in entry p % cap
+  void* vc;               // [slots, G, cap, V]
+  int cap;
+  // qkv preparation
+  const float* bias;      // [H maps D + G maps D + G V] (nullable)
+  const float *qn_w, *kn_w;   // [D] (nullable: no norm)
+  float eps;
+  const float *cos_t, *sin_t; // [max_pos, rot / 2]
+  int rot, max_pos;
+  // attention
+  float scale, softcap;   // softcap <= 0: none
+  int window;             // <= 0: all earlier tokens
+  float lam, out_scale, out_eps;   // differential: (a1 - lam a2) / rms * out_scale
+  void* y;                // [B T, ldy] heads side by side
+  int64_t ldy;
+  int from_buf;           // keys of this step's buffer (prompt from position 0) instead of the cache
+  // split decode
+  float* part;            // [B H, splits, maps (V + 2)] partial sums
+  int splits;
+};
+
+}  // namespace nxd

@@ -239,8 +239,10 @@ class LlamaForCausalLMInference:
             not self.model.lm_head.weight.is_floating_point()
         if tied_q and "lm_head.weight" not in local and "model.embed_tokens.weight" in local:
             local["lm_head.weight"] = local["model.embed_tokens.weight"]   # quantized copy of the tied table
-        local = {k: (v.to(self.dtype) if v.is_floating_point() and k.split(".")[-1] != "scale" else v)
-                 for k, v in local.items()}
+        # the model's dtype, except for parameters that a model keeps in fp32 whatever that is
+        kept = {n for n, p in self.model.named_parameters() if p.dtype == torch.float32}
+        local = {k: (v.to(torch.float32 if k in kept else self.dtype)
+                     if v.is_floating_point() and k.split(".")[-1] != "scale" else v) for k, v in local.items()}
         missing, unexpected = self.model.load_state_dict(local, strict=False)
         missing = [m for m in missing if not (getattr(self.model_config, "tie_word_embeddings", False)
                                               and m == "lm_head.weight" and not tied_q)]
@@ -294,6 +296,15 @@ class LlamaForCausalLMInference:
         self._load_local(local)
         return self
 
+    def ensure_slots(self, n: int) -> None:
+        """At least n cache slots.  A larger cache replaces the present one (and the graphs captured over
+        it): only between batches."""
+        if n > self.max_batch:
+            self.max_batch = n
+            self._graphs.clear()
+            self._prefill_cache.clear()
+            self.model.setup_kv_cache(self.max_batch, self.cache_len, self.device)
+
     # ------------------------------------------------------------------ model calls
     def reset(self) -> None:
         self.kv_cache_populated = False
@@ -305,8 +316,10 @@ class LlamaForCausalLMInference:
         self.model._decode_fused_ok = None if enabled else False
 
     def _context_encode(self, input_ids: torch.Tensor, attention_mask: Optional[torch.Tensor] = None,
-                        position_ids: Optional[torch.Tensor] = None, seq_ids: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """Prefill; returns logits [B, V] of each sequence's last valid token (fp32)."""
+                        position_ids: Optional[torch.Tensor] = None, seq_ids: Optional[torch.Tensor] = None,
+                        want: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """Prefill; returns logits [B, V] of each sequence's last valid token, or with `want` [R, 2]
+        (sequence, token) pairs the logits [R, V] of those tokens (fp32)."""
         dev = self.device
         input_ids = input_ids.to(dev)
         B, T = input_ids.shape
@@ -318,7 +331,12 @@ class LlamaForCausalLMInference:
         ids, mask = pad_to_bucket(input_ids, attention_mask, self.config.buckets + [self.config.max_length], pad)
         Tb = ids.shape[1]
         seq_ids = torch.arange(B, device=dev) if seq_ids is None else seq_ids.to(dev)
-        if self._prefill_graphs_on():
+        if want is not None:
+            positions = torch.arange(Tb, device=dev).unsqueeze(0).expand(B, Tb)
+            want = want.to(dev)
+            logits = self.model.forward_tokens(ids, positions, seq_ids, prefill=True, lengths=lengths,
+                                               logit_rows=want[:, 0] * Tb + want[:, 1])
+        elif self._prefill_graphs_on():
             logits = self._prefill_graph(B, Tb).run(ids, seq_ids, lengths - 1)
         else:
             positions = torch.arange(Tb, device=dev).unsqueeze(0).expand(B, Tb)
@@ -495,7 +513,6 @@ class LlamaForCausalLMInference:
 
 
 def _init_single_process():
+    """A one-process group without a TCP rendezvous (no port to collide on)."""
     if not dist.is_initialized():
-        os.environ.setdefault("MASTER_ADDR", "127.0.0.1")
-        os.environ.setdefault("MASTER_PORT", str(29500 + os.getpid() % 1000))
-        dist.init_process_group("gloo", rank=0, world_size=1)
+        dist.init_process_group("gloo", store=dist.HashStore(), rank=0, world_size=1)

@@ -84,6 +84,9 @@ class DecodeGraph:
     def _capture(self):
         st = self.state
         saved = [t.clone() for t in (st.tokens, st.positions, st.cache_len, st.step)]
+        # the warm-up below decodes for real: a cache with a recurrent state (or a ring of recent keys)
+        # is put back afterwards, a plain key cache is simply written again by the replay
+        cache = self.model.save_cache() if hasattr(self.model, "save_cache") else None
         s = torch.cuda.Stream()
         s.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(s):
@@ -91,6 +94,8 @@ class DecodeGraph:
         torch.cuda.current_stream().wait_stream(s)
         for t, v in zip((st.tokens, st.positions, st.cache_len, st.step), saved):
             t.copy_(v)
+        if cache is not None:
+            self.model.load_cache(cache)
         self.graph = torch.cuda.CUDAGraph()
         with graph_capture(self.graph):
             self._run_eager()

@@ -105,14 +105,18 @@ class DecoderInferenceMixin:
     @torch.no_grad()
     def forward_tokens(self, input_ids: torch.Tensor, positions: torch.Tensor, seq_ids: Optional[torch.Tensor] = None,
                        cache_len: Optional[torch.Tensor] = None, last_index: Optional[torch.Tensor] = None,
-                       prefill: bool = False, return_hidden: bool = False):
+                       prefill: bool = False, return_hidden: bool = False, lengths: Optional[torch.Tensor] = None,
+                       logit_rows: Optional[torch.Tensor] = None):
         """input_ids [B, T]; positions [B, T] (int64) absolute positions of the new tokens;
         seq_ids [B] cache rows; cache_len [B] int32 valid cache length AFTER this step (decode);
-        last_index [B] -> logits [B, V] of that token per sequence, else logits [B, T, V].
-        prefill=True: the new tokens start at position 0 (causal flash attention over them)."""
+        last_index [B] -> logits [B, V] of that token per sequence, logit_rows [R] -> logits [R, V] of
+        those rows b * T + t, else logits [B, T, V].
+        prefill=True: the new tokens start at position 0 (causal flash attention over them).
+        lengths [B]: valid new tokens, the rest is right padding (a causal key cache needs no notice of
+        it; models with a recurrent state do)."""
         assert self.kv_cache is not None, "call setup_kv_cache() first"
         B, T = input_ids.shape
-        if not prefill and self._decode_fusable(input_ids):
+        if not prefill and logit_rows is None and self._decode_fusable(input_ids):
             return self._forward_decode_fused(input_ids, positions, seq_ids, cache_len, last_index, return_hidden)
         nq, nkv, D = self.nq, self.nkv, self.head_dim
         W = (nq + 2 * nkv) * D
@@ -141,7 +145,10 @@ class DecoderInferenceMixin:
             x = self._row(attn.o_proj, o.reshape(B, T, nq * D))
             h, residual = self._norm(x, layer.post_attention_layernorm.weight, residual)
             x = self._ffn(layer, h)
-        if last_index is not None:
+        if logit_rows is not None:
+            x = x.reshape(B * T, -1)[logit_rows]
+            residual = residual.reshape(B * T, -1)[logit_rows]
+        elif last_index is not None:
             rows = torch.arange(B, device=x.device)
             x = x[rows, last_index]
             residual = residual[rows, last_index]

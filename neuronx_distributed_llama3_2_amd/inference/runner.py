@@ -95,8 +95,7 @@ class InferenceRunner:
         if int(cfg.tp_degree) > 1 and not dist.is_initialized():
             from .spmd_server import SpmdGenerationServer
 
-            app = "llama" if self.app_cls is LlamaForCausalLMInference else self.app_cls.__name__
-            m = SpmdGenerationServer.from_compiled(traced_model_path, int(cfg.tp_degree), app=app)
+            m = SpmdGenerationServer.from_compiled(traced_model_path, int(cfg.tp_degree))
             self.config = m.config
             return m
         m = self.app_cls.load(traced_model_path)

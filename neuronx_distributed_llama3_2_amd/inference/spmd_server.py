@@ -25,15 +25,10 @@ from ..trace.runtime import SpmdWorkerPool
 _DTYPES = {"bfloat16": torch.bfloat16, "float16": torch.float16, "float32": torch.float32}
 
 
-def _build_compiled(rank: int, world: int, path: str, dtype: str, app: str):
-    from . import LlamaForCausalLMInference
+def _build_compiled(rank: int, world: int, path: str, dtype: str):
+    from .registry import app_class
 
-    cls = LlamaForCausalLMInference
-    if app != "llama":
-        from . import moe as _moe
-
-        cls = getattr(_moe, app)
-    return cls.load(path, dtype=_DTYPES[dtype])
+    return app_class(path).load(path, dtype=_DTYPES[dtype])
 
 
 def _build_from_full(rank: int, world: int, model_config: Dict[str, Any], full_sd_path: str,
@@ -55,11 +50,12 @@ class SpmdGenerationServer:
         self.config = config      # InferenceConfig of the served model (runners read max_length etc.)
 
     @classmethod
-    def from_compiled(cls, path: str, tp_degree: int, dtype: str = "bfloat16", app: str = "llama"):
-        """Workers load the per-rank shards written by `compile()` (tp{r}_sharded_checkpoint.safetensors)."""
+    def from_compiled(cls, path: str, tp_degree: int, dtype: str = "bfloat16"):
+        """Workers load the per-rank shards written by `compile()` (tp{r}_sharded_checkpoint.safetensors);
+        the application follows from the directory's config.json (inference/registry.py)."""
         from .config import InferenceConfig
 
-        return cls(SpmdWorkerPool(tp_degree, _build_compiled, (path, dtype, app)), InferenceConfig.from_pretrained(path))
+        return cls(SpmdWorkerPool(tp_degree, _build_compiled, (path, dtype)), InferenceConfig.from_pretrained(path))
 
     @classmethod
     def from_full_state_dict(cls, model_config: Dict[str, Any], full_sd_path: str, tp_degree: int,

@@ -36,6 +36,36 @@ def ext():
     return _C
 
 
+_H = None
+
+
+def hybrid_ext():
+    """The `_hybrid` module: the kernels of the hybrid decoders (csrc/hybrid/) and the GEMM dispatch;
+    raise loudly if it is not built."""
+    global _H
+    if _H is None:
+        try:
+            from .. import _hybrid as h
+        except ImportError as e:  # pragma: no cover - depends on the build
+            raise RuntimeError(
+                "neuronx_distributed_llama3_2_amd HIP extension (_hybrid) is not built; run "
+                "`python -m neuronx_distributed_llama3_2_amd._build --target _hybrid`") from e
+        _H = h
+    return _H
+
+
+_G = None
+
+
+def gemm_ext():
+    """The module whose GEMM dispatch (csrc/gemm.cpp, linked into both) serves the linear layers: `_C`,
+    or `_hybrid` where only that one is built (a process that serves a hybrid decoder and nothing else)."""
+    global _G
+    if _G is None:
+        _G = ext() if ext_available() else hybrid_ext()
+    return _G
+
+
 def ext_available() -> bool:
     try:
         ext()

@@ -11,7 +11,7 @@ import os
 
 import torch
 
-from ._ext import ext, use_native
+from ._ext import ext, gemm_ext, use_native
 
 _ENABLED = os.environ.get("NXD_TUNED_GEMM", "1") == "1"
 
@@ -38,7 +38,7 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias=None, out: torch.Tensor = None
     if _native(x, w) and x.stride(-1) == 1:
         x2 = x.reshape(-1, x.shape[-1])
         y = out if out is not None else torch.empty(shape, dtype=x.dtype, device=x.device)
-        ext().gemm(x2, w.t(), y.view(-1, w.shape[0]), None, 1.0, 0.0)
+        gemm_ext().gemm(x2, w.t(), y.view(-1, w.shape[0]), None, 1.0, 0.0)
         return y + bias if bias is not None else y
     y = torch.nn.functional.linear(x, w, bias)
     if out is not None:
@@ -47,13 +47,22 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias=None, out: torch.Tensor = None
     return y
 
 
+def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x [..., K] @ w[N, K]^T -> fp32 [..., N]: the accumulator unrounded (logits of 16-bit weights)."""
+    if _native(x, w) and x.stride(-1) == 1:
+        y = torch.empty(x.shape[:-1] + (w.shape[0],), dtype=torch.float32, device=x.device)
+        gemm_ext().gemm(x.reshape(-1, x.shape[-1]), w.t(), y.view(-1, w.shape[0]), None, 1.0, 0.0)
+        return y
+    return torch.nn.functional.linear(x.float(), w.float())
+
+
 def matmul(a: torch.Tensor, b: torch.Tensor, out: torch.Tensor = None) -> torch.Tensor:
     """a [..., K] @ b [K, N] -> [..., N] (written into `out` if given: contiguous [..., N])."""
     shape = a.shape[:-1] + (b.shape[1],)
     if _native(a, b) and a.stride(-1) == 1:
         a2 = a.reshape(-1, a.shape[-1])
         y = out if out is not None else torch.empty(shape, dtype=a.dtype, device=a.device)
-        ext().gemm(a2, b, y.view(-1, b.shape[1]), None, 1.0, 0.0)
+        gemm_ext().gemm(a2, b, y.view(-1, b.shape[1]), None, 1.0, 0.0)
         return y
     y = torch.matmul(a, b)
     if out is not None:

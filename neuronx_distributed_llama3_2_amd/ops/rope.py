@@ -17,10 +17,11 @@ from ._ext import ext, use_native
 
 
 def llama3_inv_freq(dim: int, base: float = 500000.0, factor: Optional[float] = None, low_freq_factor: float = 1.0,
-                    high_freq_factor: float = 4.0, original_max_position_embeddings: int = 8192) -> torch.Tensor:
+                    high_freq_factor: float = 4.0, original_max_position_embeddings: int = 8192,
+                    dtype: torch.dtype = torch.float32) -> torch.Tensor:
     inv_freq = 1.0 / (base ** (torch.arange(0, dim, 2, dtype=torch.int64).double() / dim))
     if factor is None:
-        return inv_freq.float()
+        return inv_freq.to(dtype)
     low_wl = original_max_position_embeddings / low_freq_factor
     high_wl = original_max_position_embeddings / high_freq_factor
     wavelen = 2 * math.pi / inv_freq
@@ -28,7 +29,7 @@ def llama3_inv_freq(dim: int, base: float = 500000.0, factor: Optional[float] = 
     scaled = torch.where(wavelen > low_wl, inv_freq / factor, inv_freq)
     mid = (wavelen <= low_wl) & (wavelen >= high_wl)
     scaled = torch.where(mid, (1 - smooth) * inv_freq / factor + smooth * inv_freq, scaled)
-    return scaled.float()
+    return scaled.to(dtype)
 
 
 def inv_freq_from_config(config, head_dim: int) -> torch.Tensor:
