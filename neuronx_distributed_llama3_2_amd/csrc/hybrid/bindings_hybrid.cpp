@@ -18,9 +18,12 @@ int relu_squared_launch(bool, const void*, void*, int64_t, hipStream_t);
 int softcap_launch(float*, int64_t, float, hipStream_t);
 int delta_prep_launch(bool, const DeltaParams&, hipStream_t);
 int delta_scan_launch(bool, const DeltaParams&, hipStream_t);
+int delta_chunk_launch(bool, const DeltaParams&, hipStream_t);
 int delta_out_launch(bool, const DeltaParams&, hipStream_t);
 int delta_decode_launch(bool, const DeltaParams&, hipStream_t);
 int attn_prep_launch(bool, const WindowAttnParams&, hipStream_t);
+bool attn_prompt_supported(const WindowAttnParams&);
+int attn_prompt_launch(const WindowAttnParams&, hipStream_t);
 int attn_row_launch(bool, const WindowAttnParams&, hipStream_t);
 }  // namespace nxd
 
@@ -133,7 +136,8 @@ void softcap_(Tensor x, double cap) {
 // The recurrence over T new tokens of B sequences.  one launch (T == 1 and `fused`) or three with the
 // fp32 intermediates; sizes (H, G, D, V).
 void delta_rule(Tensor proj, int64_t B, int64_t T, std::vector<int64_t> sizes, Tensor conv, Tensor a_log, Tensor dt_bias,
-                Tensor norm_w, double eps, Tensor pos, Opt lens, Opt slots, Tensor state, Tensor ring, Tensor y, bool fused) {
+                Tensor norm_w, double eps, Tensor pos, Opt lens, Opt slots, Tensor state, Tensor ring, Tensor y, bool fused,
+                int64_t chunk_from) {
   const bool f32 = act_f32(proj, "proj");
   same_act(ring, proj, "ring");
   same_act(y, proj, "y");
@@ -184,15 +188,29 @@ void delta_rule(Tensor proj, int64_t B, int64_t T, std::vector<int64_t> sizes, T
   }
   auto opt = proj.options().dtype(at::kFloat);
   const int64_t M = B * T;
-  Tensor qk = at::empty({2, M, p.G, p.D}, opt), vo = at::empty({2, M, p.H, p.V}, opt), gb = at::empty({2, M, p.H}, opt);
+  if (T >= chunk_from) p.nch = (int)((T + 63) / 64);
+  TORCH_CHECK(p.nch <= 65535, "delta_rule: tokens of one step");
+  const int64_t Mq = p.nch > 0 ? B * p.nch * 64 : M;   // whole chunks of q and k
+  Tensor qk = at::empty({2, Mq, p.G, p.DP}, opt), vo = at::empty({2, M, p.H, p.V}, opt), gb = at::empty({2, M, p.H}, opt);
   p.qn = qk.data_ptr<float>();
-  p.kn = p.qn + M * p.G * p.D;
+  p.kn = p.qn + Mq * p.G * p.DP;
   p.vn = vo.data_ptr<float>();
   p.o = p.vn + M * p.H * p.V;
   p.lg = gb.data_ptr<float>();
   p.beta = p.lg + M * p.H;
   check_rc(nxd::delta_prep_launch(f32, p, cur_stream()), "delta_prep");
-  check_rc(nxd::delta_scan_launch(f32, p, cur_stream()), "delta_scan");
+  Tensor cells;   // (outlives the launches below)
+  if (p.nch > 0) {
+    const int64_t n = B * p.nch * p.H;
+    cells = at::empty({n * 64 * (p.DP + (p.V + 15) / 16 * 16 + 64 + 2)}, opt);
+    p.cw = cells.data_ptr<float>();
+    p.cp = p.cw + n * 64 * p.DP;
+    p.ceg = p.cp + n * 64 * 64;
+    p.cy = p.ceg + n * 64 * 2;
+    check_rc(nxd::delta_chunk_launch(f32, p, cur_stream()), "delta_chunk");
+  } else {
+    check_rc(nxd::delta_scan_launch(f32, p, cur_stream()), "delta_scan");
+  }
   check_rc(nxd::delta_out_launch(f32, p, cur_stream()), "delta_out");
 }
 
@@ -255,7 +273,7 @@ void attn_prep(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, Opt
 // from_buf: the new tokens start at position 0 and see only each other
 void window_attn(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, double scale, double softcap, int64_t window,
                  double lam, double out_scale, double out_eps, Tensor pos, Opt lens, Opt slots, Tensor kc, Tensor vc, Tensor y,
-                 bool from_buf) {
+                 bool from_buf, bool fused) {
   auto p = attn_params(buf, B, T, sizes, pos, lens, slots, kc, vc);
   same_act(y, buf, "y");
   TORCH_CHECK(y.dim() == 2 && y.size(0) == B * T && y.size(1) == p.H * p.V, "window_attn: y [B T, H V]");
@@ -270,6 +288,11 @@ void window_attn(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, d
   p.y = y.data_ptr();
   p.ldy = y.stride(0);
   p.from_buf = from_buf ? 1 : 0;
+  const bool f32 = buf.scalar_type() == at::kFloat;
+  if (fused && !f32 && nxd::attn_prompt_supported(p)) {
+    check_rc(nxd::attn_prompt_launch(p, cur_stream()), "attn_prompt");
+    return;
+  }
   check_rc(nxd::attn_row_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "window_attn");
 }
 
@@ -286,11 +309,11 @@ PYBIND11_MODULE(_hybrid, m) {
   m.def("softcap_", &softcap_);
   m.def("delta_rule", &delta_rule, py::arg("proj"), py::arg("B"), py::arg("T"), py::arg("sizes"), py::arg("conv"),
         py::arg("a_log"), py::arg("dt_bias"), py::arg("norm_w"), py::arg("eps"), py::arg("pos"), py::arg("lens"),
-        py::arg("slots"), py::arg("state"), py::arg("ring"), py::arg("y"), py::arg("fused") = true);
+        py::arg("slots"), py::arg("state"), py::arg("ring"), py::arg("y"), py::arg("fused") = true, py::arg("chunk_from") = 32);
   m.def("attn_prep", &attn_prep, py::arg("buf"), py::arg("B"), py::arg("T"), py::arg("sizes"), py::arg("bias"),
         py::arg("qn_w"), py::arg("kn_w"), py::arg("eps"), py::arg("cos"), py::arg("sin"), py::arg("pos"), py::arg("lens"),
         py::arg("slots"), py::arg("kc"), py::arg("vc"));
   m.def("window_attn", &window_attn, py::arg("buf"), py::arg("B"), py::arg("T"), py::arg("sizes"), py::arg("scale"),
         py::arg("softcap"), py::arg("window"), py::arg("lam"), py::arg("out_scale"), py::arg("out_eps"), py::arg("pos"),
-        py::arg("lens"), py::arg("slots"), py::arg("kc"), py::arg("vc"), py::arg("y"), py::arg("from_buf"));
+        py::arg("lens"), py::arg("slots"), py::arg("kc"), py::arg("vc"), py::arg("y"), py::arg("from_buf"), py::arg("fused") = true);
 }

@@ -22,10 +22,14 @@ struct DeltaParams {
   int nslots;
   float* state;              // [slots, H, V, DP]
   void* ring;                // [slots, taps, C] (activation type)
-  float *qn, *kn;            // [B T, G, D]
+  float *qn, *kn;            // unit q, k: [B T, G, DP], or with nch > 0 [chunks, G, 64 DP] in fragment order
   float* vn;                 // [B T, H, V]
   float *lg, *beta;          // [B T, H] log decay, write strength
   float* o;                  // [B T, H, V]
+  // 64-token chunks (csrc/hybrid/delta_chunk.hip)
+  int nch;                   // chunks per sequence (0: token by token)
+  float *cw, *cy, *cp;       // W [cells, 64 DP], Y [cells, 64 V rounded up to 16], P [cells, 64 64]
+  float* ceg;                // [cells, 2, 64] e^G, e^(G_C - G)
   void* y;                   // [B T, ldy] mixer output before its projection (activation type)
   int64_t ldy;
 };

@@ -11,8 +11,9 @@
 // is used again.  The projection buffer's columns are [q (G D) | k (G D) | v (H V) | gate (H V) |
 // beta (H) | decay (H)].
 //
-//   delta_prep   : convolution, silu, unit norms, gates of all tokens of a step (one workgroup a row)
+//   delta_prep   : convolution, silu, unit norms, gates of all tokens of a step
 //   delta_scan   : the recurrence, token by token, from the cached state (8 lanes a state column)
+//                  (long runs of tokens: 64 at a time, delta_chunk.hip)
 //   delta_out    : the gated head norm
 //   delta_decode : all of it for one new token per sequence, one workgroup per (sequence, head)
 #include "hybrid.h"
@@ -38,39 +39,143 @@ __device__ __forceinline__ float conv_silu(const DeltaParams& p, const T* proj, 
   return siluf_(a);
 }
 
-template <typename T>
+// the same for TT consecutive tokens t0 .. of sequence b and N neighbouring channels c ..: every input is
+// read once (up to 4 taps; more fall back to the single-token form)
+template <typename T, int TT, int N>
+__device__ __forceinline__ void conv_silu_run(const DeltaParams& p, const T* proj, const T* ring, int64_t m0, int t0, int n,
+                                              int64_t p0, int c, float (&out)[N][TT]) {
+  if (p.taps > 4) {
+#pragma unroll
+    for (int k = 0; k < N; ++k)
+#pragma unroll
+      for (int i = 0; i < TT; ++i) out[k][i] = i < n ? conv_silu<T>(p, proj, ring, m0 + i, t0 + i, p0 + i, c + k) : 0.f;
+    return;
+  }
+  float x[N][TT + 3], wt[N][4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+#pragma unroll
+    for (int k = 0; k < N; ++k) wt[k][j] = j < 4 - p.taps ? 0.f : p.conv[(int64_t)(j - 4 + p.taps) * p.C + c + k];
+  auto get = [&](const T* s, int i) {
+    if constexpr (N == 2) ld2(s, x[0][i], x[1][i]);
+    else x[0][i] = ld(s);
+  };
+  if (t0 >= 3 && n == TT) {   // (uniform) no edge of the sequence or of the step in sight
+#pragma unroll
+    for (int i = 0; i < TT + 3; ++i) get(proj + (m0 + i - 3) * p.ldp + c, i);
+  } else {
+#pragma unroll
+    for (int i = 0; i < TT + 3; ++i) {   // token t0 + i - 3
+      const int64_t q = p0 + i - 3;
+#pragma unroll
+      for (int k = 0; k < N; ++k) x[k][i] = 0.f;
+      if (i - 3 < n && q >= 0 && 3 - i < p.taps) get(t0 + i - 3 >= 0 ? proj + (m0 + i - 3) * p.ldp + c : ring + (q % p.taps) * p.C + c, i);
+    }
+  }
+#pragma unroll
+  for (int k = 0; k < N; ++k)
+#pragma unroll
+    for (int i = 0; i < TT; ++i)
+      out[k][i] = siluf_(wt[k][0] * x[k][i] + wt[k][1] * x[k][i + 1] + wt[k][2] * x[k][i + 2] + wt[k][3] * x[k][i + 3]);
+}
+
+constexpr int PREP_TOKENS = 8;   // tokens of one sequence a prep workgroup handles
+
+// N = 2: two neighbouring channels a lane (even head sizes), 1: one.  NJ steps of 64 N columns cover DP.
+template <typename T, int N, int NJ>
 __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaParams p) {
-  const int64_t m = blockIdx.x;
-  const int b = (int)(m / p.T), t = (int)(m % p.T);
-  if (p.lens && t >= p.lens[b]) return;
-  const int64_t ps = pos_of(p.pos, p.pos_stride, b) + t;
+  constexpr int TT = PREP_TOKENS;
+  const int b = blockIdx.y, t0 = blockIdx.x * TT;
+  const int len = p.lens ? min(p.lens[b], p.T) : p.T;
+  const bool frag = p.nch > 0;
+  // the chunked scan reads whole chunks: their last tokens past the sequence are zeros
+  if (t0 >= (frag ? (len + 63) / 64 * 64 : len)) return;
+  const int n = max(0, min(TT, len - t0));
+  const int64_t m0 = (int64_t)b * p.T + t0;
+  const int64_t p0 = pos_of(p.pos, p.pos_stride, b) + t0;
   const int slot = slot_of(p.slots, b, p.nslots);
   const T* proj = static_cast<const T*>(p.proj);
   const T* ring = static_cast<const T*>(p.ring) + (int64_t)slot * p.taps * p.C;
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
-  const int G = p.G, D = p.D, H = p.H, HV = p.H * p.V;
+  const int G = p.G, D = p.D, DP = p.DP, H = p.H, HV = p.H * p.V, NB = DP / 16;
   for (int hd = wid; hd < 2 * G; hd += 4) {   // q heads, then k heads: a wave per unit vector
-    float x[4], ss = 0.f;
+    const bool isq = hd < G;
+    const int g = isq ? hd : hd - G;
+    float x[NJ][N][TT], ss[TT];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = lane + 64 * i;
-      x[i] = d < D ? conv_silu<T>(p, proj, ring, m, t, ps, hd * D + d) : 0.f;
-      ss += x[i] * x[i];
-    }
-    ss = wave_sum(ss);
-    float r = 1.f / sqrtf(ss + 1e-6f);
-    if (hd < G) r *= p.qscale;
-    float* out = (hd < G ? p.qn : p.kn) + (m * G + (hd < G ? hd : hd - G)) * D;
+    for (int i = 0; i < TT; ++i) ss[i] = 0.f;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = lane + 64 * i;
-      if (d < D) out[d] = x[i] * r;
+    for (int j = 0; j < NJ; ++j) {
+      const int d = N * lane + 64 * N * j;
+#pragma unroll
+      for (int k = 0; k < N; ++k)
+#pragma unroll
+        for (int i = 0; i < TT; ++i) x[j][k][i] = 0.f;
+      if (d < D && n > 0) conv_silu_run<T, TT, N>(p, proj, ring, m0, t0, n, p0, hd * D + d, x[j]);
+#pragma unroll
+      for (int k = 0; k < N; ++k)
+#pragma unroll
+        for (int i = 0; i < TT; ++i) ss[i] += x[j][k][i] * x[j][k][i];
     }
+#pragma unroll
+    for (int i = 0; i < TT; ++i) {
+      float r = __builtin_amdgcn_rsqf(sum64(ss[i]) + 1e-6f);
+      if (isq) r *= p.qscale;
+      if (i >= n) r = 0.f;
+#pragma unroll
+      for (int j = 0; j < NJ; ++j)
+#pragma unroll
+        for (int k = 0; k < N; ++k) x[j][k][i] *= r;
+    }
+    if (!frag) {
+      float* out = (isq ? p.qn : p.kn) + (m0 * G + g) * DP;
+#pragma unroll
+      for (int j = 0; j < NJ; ++j)
+#pragma unroll
+        for (int k = 0; k < N; ++k) {
+          const int d = N * lane + 64 * N * j + k;
+#pragma unroll
+          for (int i = 0; i < TT; ++i)
+            if (i < n && d < DP) out[(int64_t)i * G * DP + d] = x[j][k][i];
+        }
+      continue;
+    }
+    // fragment order of the chunk (delta_chunk.hip): q as rows of tokens, k as rows of columns
+    const int tc = t0 & 63, tb = tc >> 4;
+    const int64_t cell = (((int64_t)b * p.nch + t0 / 64) * G + g) * 64 * DP;
+#pragma unroll
+    for (int j = 0; j < NJ; ++j)
+#pragma unroll
+      for (int k = 0; k < N; ++k) {
+        const int d = N * lane + 64 * N * j + k;
+        if (d >= DP) continue;
+        if (isq) {
+          float* out = p.qn + cell + ((((int64_t)tb * NB + d / 16) * 4 + (d & 15) / 4) * 16 + (tc & 15)) * 4 + (d & 3);
+#pragma unroll
+          for (int i = 0; i < TT; ++i) out[4 * i] = x[j][k][i];
+        } else {
+          float* out = p.kn + cell + ((((int64_t)(d / 16) * 4 + tb) * 4 + (tc & 15) / 4) * 16 + (d & 15)) * 4;
+          st4(out, f32x4_t{x[j][k][0], x[j][k][1], x[j][k][2], x[j][k][3]});
+          st4(out + 64, f32x4_t{x[j][k][4], x[j][k][5], x[j][k][6], x[j][k][7]});
+        }
+      }
   }
-  float* vo = p.vn + m * HV;
-  for (int c = tid; c < HV; c += 256) vo[c] = conv_silu<T>(p, proj, ring, m, t, ps, 2 * G * D + c);
-  const T* gates = proj + m * p.ldp + p.C + HV;
-  for (int h = tid; h < H; h += 256) {
+  if (n <= 0) return;
+  float* vo = p.vn + m0 * HV;
+  for (int c = N * tid; c < HV; c += 256 * N) {
+    float x[N][TT];
+    conv_silu_run<T, TT, N>(p, proj, ring, m0, t0, n, p0, 2 * G * D + c, x);
+#pragma unroll
+    for (int i = 0; i < TT; ++i)
+      if (i < n) {
+        if constexpr (N == 2) *reinterpret_cast<float2*>(vo + (int64_t)i * HV + c) = float2{x[0][i], x[1][i]};
+        else vo[(int64_t)i * HV + c] = x[0][i];
+      }
+  }
+  for (int i = tid; i < n * H; i += 256) {
+    const int h = i % H;
+    const int64_t m = m0 + i / H;
+    const T* gates = proj + m * p.ldp + p.C + HV;
     p.beta[m * H + h] = sigmoidf_(ld(gates + h));
     p.lg[m * H + h] = -expf(p.a_log[h]) * softplusf_(ld(gates + H + h) + p.dt_bias[h]);
   }
@@ -85,7 +190,7 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaParams p) {
   __shared__ float vs[TK][32], gs[TK], bs[TK];
   const int tid = threadIdx.x, l = tid & 7, col = tid >> 3;
   const int h = blockIdx.y, b = blockIdx.z, v = blockIdx.x * 32 + col;
-  const int H = p.H, G = p.G, D = p.D, V = p.V, g = h / (H / G);
+  const int H = p.H, G = p.G, V = p.V, g = h / (H / G);
   const int len = p.lens ? min(p.lens[b], p.T) : p.T;
   if (len <= 0) return;
   const int slot = slot_of(p.slots, b, p.nslots);
@@ -100,9 +205,9 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaParams p) {
     __syncthreads();
     for (int i = tid; i < n * DP; i += 256) {
       const int t = i / DP, d = i % DP;
-      const int64_t o = ((m0 + t0 + t) * G + g) * D + d;
-      ks[t][d] = d < D ? p.kn[o] : 0.f;
-      qs[t][d] = d < D ? p.qn[o] : 0.f;
+      const int64_t o = ((m0 + t0 + t) * G + g) * DP + d;
+      ks[t][d] = p.kn[o];
+      qs[t][d] = p.qn[o];
     }
     for (int i = tid; i < n * 32; i += 256) {
       const int t = i >> 5, c = blockIdx.x * 32 + (i & 31);
@@ -126,8 +231,7 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaParams p) {
           dot += S[i][e] * k[i][e];
         }
       }
-#pragma unroll
-      for (int o = 4; o > 0; o >>= 1) dot += __shfl_xor(dot, o, 64);
+      dot = sum8(dot);
       const float u = bs[t] * (vs[t][col] - dot);
       float out = 0.f;
 #pragma unroll
@@ -139,8 +243,7 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaParams p) {
           out += S[i][e] * q[e];
         }
       }
-#pragma unroll
-      for (int o = 4; o > 0; o >>= 1) out += __shfl_xor(out, o, 64);
+      out = sum8(out);
       if (l == 0 && v < V) p.o[((m0 + t0 + t) * H + h) * V + v] = out;
     }
   }
@@ -173,7 +276,7 @@ __global__ void __launch_bounds__(256) delta_out_kernel(DeltaParams p) {
     x[j] = v < V ? o[v] : 0.f;
     ss += x[j] * x[j];
   }
-  const float r = 1.f / sqrtf(wave_sum(ss) / (float)V + p.eps);
+  const float r = 1.f / sqrtf(sum64(ss) / (float)V + p.eps);
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int v = lane + 64 * j;
@@ -242,8 +345,7 @@ __global__ void __launch_bounds__(NTH) delta_decode_kernel(DeltaParams p) {
         S[i][e] = ps > 0 ? S[i][e] * gt : 0.f;   // a sequence's first token starts from zero
         dot += S[i][e] * k[i][e];
       }
-#pragma unroll
-    for (int o = 4; o > 0; o >>= 1) dot += __shfl_xor(dot, o, 64);
+    dot = sum8(dot);
     const float u = beta * (vs[v] - dot);
     float out = 0.f;
 #pragma unroll
@@ -255,8 +357,7 @@ __global__ void __launch_bounds__(NTH) delta_decode_kernel(DeltaParams p) {
       }
       st4(sp + i * 32 + l * 4, S[i]);
     }
-#pragma unroll
-    for (int o = 4; o > 0; o >>= 1) out += __shfl_xor(out, o, 64);
+    out = sum8(out);
     if (l == 0) os[v] = out;
   }
   __syncthreads();
@@ -283,7 +384,11 @@ __global__ void __launch_bounds__(NTH) delta_decode_kernel(DeltaParams p) {
 
 template <typename T>
 static int run_prep(const DeltaParams& p, hipStream_t s) {
-  hipLaunchKernelGGL((delta_prep_kernel<T>), dim3((unsigned)(p.B * p.T)), dim3(256), 0, s, p);
+  const dim3 grid((unsigned)ceil_div(p.nch > 0 ? p.nch * 64 : p.T, PREP_TOKENS), (unsigned)p.B);
+  const bool pairs = p.D % 2 == 0 && p.V % 2 == 0 && p.ldp % 2 == 0;
+  if (pairs && p.DP <= 128) hipLaunchKernelGGL((delta_prep_kernel<T, 2, 1>), grid, dim3(256), 0, s, p);
+  else if (pairs) hipLaunchKernelGGL((delta_prep_kernel<T, 2, 2>), grid, dim3(256), 0, s, p);
+  else hipLaunchKernelGGL((delta_prep_kernel<T, 1, 4>), grid, dim3(256), 0, s, p);
   return hipGetLastError() == hipSuccess ? 0 : 1;
 }
 template <typename T>

@@ -5,6 +5,7 @@
 //                 `rot` dimensions, in place in the projection buffer; k and v also to the cache
 //   attn_row    : one wave per (token, head), keys across lanes -- any size, fp32 or bf16, keys of the
 //                 buffer (prompt) or of the cache (any number of new tokens)
+//   attn_prompt : bf16 prompts on the matrix cores (window_attn_prompt.h)
 //   attn_split / attn_merge : one new token per sequence, the visible keys split over workgroups
 //
 // A key at position p lives in entry p % cap of the cache, so a windowed layer keeps about a window of
@@ -221,6 +222,25 @@ int attn_prep_launch(bool f32, const WindowAttnParams& p, hipStream_t s) {
   if (f32) hipLaunchKernelGGL((hybrid::attn_prep_kernel<float>), grid, dim3(256), 0, s, p);
   else hipLaunchKernelGGL((hybrid::attn_prep_kernel<uint16_t>), grid, dim3(256), 0, s, p);
   return hipGetLastError() == hipSuccess ? 0 : 1;
+}
+
+int attn_prompt_d32_launch(const WindowAttnParams&, hipStream_t);
+int attn_prompt_d48_launch(const WindowAttnParams&, hipStream_t);
+int attn_prompt_d64_launch(const WindowAttnParams&, hipStream_t);
+int attn_prompt_d96_launch(const WindowAttnParams&, hipStream_t);
+int attn_prompt_d128_launch(const WindowAttnParams&, hipStream_t);
+
+// bf16 prompts on the matrix cores: 16-byte pieces of every head, head sizes the kernels are built for
+bool attn_prompt_supported(const WindowAttnParams& p) {
+  return p.from_buf && p.T > 1 && p.D <= 128 && p.V <= 256 && p.D % 8 == 0 && p.V % 8 == 0 && p.ldb % 8 == 0 &&
+         p.ldy % 4 == 0 && reinterpret_cast<uintptr_t>(p.buf) % 16 == 0 && reinterpret_cast<uintptr_t>(p.y) % 16 == 0;
+}
+int attn_prompt_launch(const WindowAttnParams& p, hipStream_t s) {
+  if (p.D <= 32) return attn_prompt_d32_launch(p, s);
+  if (p.D <= 48) return attn_prompt_d48_launch(p, s);
+  if (p.D <= 64) return attn_prompt_d64_launch(p, s);
+  if (p.D <= 96) return attn_prompt_d96_launch(p, s);
+  return attn_prompt_d128_launch(p, s);
 }
 
 int attn_row_launch(bool f32, const WindowAttnParams& p, hipStream_t s) {

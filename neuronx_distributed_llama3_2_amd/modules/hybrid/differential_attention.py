@@ -95,5 +95,5 @@ class DifferentialAttentionMixer(nn.Module):
         ops.attn_prep_(buf, ctx.B, ctx.T, self.sizes, self.qkv_bias, self.q_norm, self.k_norm, self.eps, cos_t, sin_t,
                        ctx.positions, ctx.lengths, ctx.slots, cache["k"], cache["v"])
         y = ops.window_attention(buf, ctx.B, ctx.T, self.sizes, self.rule, ctx.positions, ctx.lengths, ctx.slots,
-                                 cache["k"], cache["v"], ctx.prompt)
+                                 cache["k"], cache["v"], ctx.prompt, ctx.fused)
         return linear(y, self.o_proj)

@@ -16,6 +16,11 @@ import torch.nn.functional as F
 from ._ext import hybrid_ext, use_native
 
 
+# new tokens per sequence from which the recurrence runs 64 tokens at a time on the matrix cores
+# (csrc/hybrid/delta_chunk.hip) instead of token by token
+CHUNK_FROM = 32
+
+
 @dataclass(frozen=True)
 class DeltaSizes:
     heads: int
@@ -39,16 +44,16 @@ class DeltaSizes:
 def delta_rule(proj: torch.Tensor, B: int, T: int, sizes: DeltaSizes, conv: torch.Tensor, a_log: torch.Tensor,
                dt_bias: torch.Tensor, norm_w: torch.Tensor, eps: float, positions: torch.Tensor,
                lengths: Optional[torch.Tensor], slots: Optional[torch.Tensor], state: torch.Tensor,
-               ring: torch.Tensor, fused: bool = True) -> torch.Tensor:
+               ring: torch.Tensor, fused: bool = True, chunk_from: int = CHUNK_FROM) -> torch.Tensor:
     """proj [B T, >= columns]: [q | k | v | gate | beta | decay] of T new tokens per sequence, the first
     at positions[b] (int64 [B] or [B, T]); lengths [B] int32: valid new tokens (None: T).  conv
     [taps, C] fp32.  Updates state / ring of slots[b]; returns [B T, H V] (padding rows are zero).
-    fused: one launch when T == 1."""
+    fused: one launch when T == 1.  chunk_from: steps of at least so many tokens take the chunked form."""
     H, G, D, V = sizes.heads, sizes.kv_heads, sizes.dim, sizes.vdim
     y = torch.empty((B * T, H * V), dtype=proj.dtype, device=proj.device)
     if use_native(proj):
         hybrid_ext().delta_rule(proj, B, T, [H, G, D, V], conv, a_log, dt_bias, norm_w, float(eps), positions,
-                                lengths, slots, state, ring, y, fused)
+                                lengths, slots, state, ring, y, fused, chunk_from)
         return y
     C, taps = sizes.channels, conv.shape[0]
     y.zero_()

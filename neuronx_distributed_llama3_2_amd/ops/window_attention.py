@@ -93,14 +93,15 @@ def attn_prep_(buf: torch.Tensor, B: int, T: int, sizes: AttnSizes, bias: Option
 
 def window_attention(buf: torch.Tensor, B: int, T: int, sizes: AttnSizes, rule: AttnRule, positions: torch.Tensor,
                      lengths: Optional[torch.Tensor], slots: Optional[torch.Tensor], k_cache: torch.Tensor,
-                     v_cache: torch.Tensor, prompt: bool) -> torch.Tensor:
+                     v_cache: torch.Tensor, prompt: bool, fused: bool = True) -> torch.Tensor:
     """Attention of the queries in buf (after attn_prep_): over the tokens of this step when they start
-    at position 0 (`prompt`), else over the cache.  Returns [B T, H V] (padding rows are zero)."""
+    at position 0 (`prompt`), else over the cache.  Returns [B T, H V] (padding rows are zero).
+    fused: the matrix-core prompt kernel and the split decode kernel where the sizes allow (bf16)."""
     H, G, R, D, V = sizes.as_list()
     y = torch.empty((B * T, H * V), dtype=buf.dtype, device=buf.device)
     if use_native(buf):
         hybrid_ext().window_attn(buf, B, T, sizes.as_list(), rule.scale, rule.softcap, rule.window, rule.lam,
-                                 rule.out_scale, rule.eps, positions, lengths, slots, k_cache, v_cache, y, prompt)
+                                 rule.out_scale, rule.eps, positions, lengths, slots, k_cache, v_cache, y, prompt, fused)
         return y
     y.zero_()
     cap = k_cache.shape[2]
