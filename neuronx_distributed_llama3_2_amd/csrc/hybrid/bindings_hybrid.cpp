@@ -6,6 +6,7 @@
 #include <hip/hip_runtime.h>
 
 #include "delta_rule.h"
+#include "gemv_hyper.h"
 #include "window_attn.h"
 
 void register_gemm(pybind11::module& m);  // ../gemm.cpp
@@ -25,6 +26,8 @@ int attn_prep_launch(bool, const WindowAttnParams&, hipStream_t);
 bool attn_prompt_supported(const WindowAttnParams&);
 int attn_prompt_launch(const WindowAttnParams&, hipStream_t);
 int attn_row_launch(bool, const WindowAttnParams&, hipStream_t);
+int attn_decode_launch(bool, const WindowAttnParams&, hipStream_t);
+int gemv_hyper_launch(int, bool, const GemvHyperParams&, hipStream_t);
 }  // namespace nxd
 
 namespace {
@@ -253,32 +256,25 @@ nxd::WindowAttnParams attn_params(const Tensor& buf, int64_t B, int64_t T, const
   return p;
 }
 
-void attn_prep(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, Opt bias, Opt qn_w, Opt kn_w, double eps,
-               Tensor cos_t, Tensor sin_t, Tensor pos, Opt lens, Opt slots, Tensor kc, Tensor vc) {
-  auto p = attn_params(buf, B, T, sizes, pos, lens, slots, kc, vc);
+void set_prep(nxd::WindowAttnParams& p, const Opt& bias, const Opt& qn_w, const Opt& kn_w, double eps, const Tensor& cos_t,
+              const Tensor& sin_t) {
   p.bias = f32_opt(bias, (p.H + p.G) * p.maps * p.D + p.G * p.V, "bias");
-  TORCH_CHECK(qn_w.has_value() == kn_w.has_value(), "attn_prep: both head norms or none");
+  TORCH_CHECK(qn_w.has_value() == kn_w.has_value(), "attention: both head norms or none");
   p.qn_w = f32_opt(qn_w, p.D, "qn_w");
   p.kn_w = f32_opt(kn_w, p.D, "kn_w");
   p.eps = (float)eps;
   TORCH_CHECK(cos_t.dim() == 2 && cos_t.sizes() == sin_t.sizes() && cos_t.size(0) >= 1 && 2 * cos_t.size(1) <= p.D,
-              "attn_prep: cos / sin [positions, rotated pairs]");
+              "attention: cos / sin [positions, rotated pairs]");
   p.cos_t = f32_ptr(cos_t, cos_t.numel(), "cos");
   p.sin_t = f32_ptr(sin_t, sin_t.numel(), "sin");
   p.rot = 2 * (int)cos_t.size(1);
   p.max_pos = (int)cos_t.size(0);
-  check_rc(nxd::attn_prep_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "attn_prep");
 }
 
-// from_buf: the new tokens start at position 0 and see only each other
-void window_attn(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, double scale, double softcap, int64_t window,
-                 double lam, double out_scale, double out_eps, Tensor pos, Opt lens, Opt slots, Tensor kc, Tensor vc, Tensor y,
-                 bool from_buf, bool fused) {
-  auto p = attn_params(buf, B, T, sizes, pos, lens, slots, kc, vc);
+void set_rule(nxd::WindowAttnParams& p, double scale, double softcap, int64_t window, double lam, double out_scale,
+              double out_eps, const Tensor& buf, const Tensor& y) {
   same_act(y, buf, "y");
-  TORCH_CHECK(y.dim() == 2 && y.size(0) == B * T && y.size(1) == p.H * p.V, "window_attn: y [B T, H V]");
-  TORCH_CHECK(from_buf || window <= 0 || T <= p.cap - window + 1, "window_attn: ", T, " new tokens do not fit a ring of ", p.cap,
-              " with a window of ", window);
+  TORCH_CHECK(y.dim() == 2 && y.size(0) == (int64_t)p.B * p.T && y.size(1) == p.H * p.V, "attention: y [B T, H V]");
   p.scale = (float)scale;
   p.softcap = (float)softcap;
   p.window = window > 0 && window < (1 << 30) ? (int)window : 0;
@@ -287,13 +283,104 @@ void window_attn(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, d
   p.out_eps = (float)out_eps;
   p.y = y.data_ptr();
   p.ldy = y.stride(0);
+}
+
+void attn_prep(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, Opt bias, Opt qn_w, Opt kn_w, double eps,
+               Tensor cos_t, Tensor sin_t, Tensor pos, Opt lens, Opt slots, Tensor kc, Tensor vc) {
+  auto p = attn_params(buf, B, T, sizes, pos, lens, slots, kc, vc);
+  set_prep(p, bias, qn_w, kn_w, eps, cos_t, sin_t);
+  check_rc(nxd::attn_prep_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "attn_prep");
+}
+
+// from_buf: the new tokens start at position 0 and see only each other
+void window_attn(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, double scale, double softcap, int64_t window,
+                 double lam, double out_scale, double out_eps, Tensor pos, Opt lens, Opt slots, Tensor kc, Tensor vc, Tensor y,
+                 bool from_buf, bool fused) {
+  auto p = attn_params(buf, B, T, sizes, pos, lens, slots, kc, vc);
+  set_rule(p, scale, softcap, window, lam, out_scale, out_eps, buf, y);
   p.from_buf = from_buf ? 1 : 0;
   const bool f32 = buf.scalar_type() == at::kFloat;
   if (fused && !f32 && nxd::attn_prompt_supported(p)) {
     check_rc(nxd::attn_prompt_launch(p, cur_stream()), "attn_prompt");
     return;
   }
-  check_rc(nxd::attn_row_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "window_attn");
+  check_rc(nxd::attn_row_launch(f32, p, cur_stream()), "window_attn");
+}
+
+// one new token per sequence: preparation, cache write and attention.  tickets: int32, zero, at least B H
+void attn_decode(Tensor buf, std::vector<int64_t> sizes, Opt bias, Opt qn_w, Opt kn_w, double eps, Tensor cos_t, Tensor sin_t,
+                 double scale, double softcap, int64_t window, double lam, double out_scale, double out_eps, Tensor pos,
+                 Opt slots, Tensor kc, Tensor vc, Tensor tickets, Tensor y) {
+  const int64_t B = buf.size(0);
+  auto p = attn_params(buf, B, 1, sizes, pos, Opt(), slots, kc, vc);
+  set_prep(p, bias, qn_w, kn_w, eps, cos_t, sin_t);
+  set_rule(p, scale, softcap, window, lam, out_scale, out_eps, buf, y);
+  TORCH_CHECK(p.H <= 65535 && B <= 65535, "attn_decode: grid");
+  const int64_t seen = p.window > 0 ? std::min<int64_t>(p.window, p.cap) : p.cap;
+  p.splits = (int)((seen + 255) / 256);
+  TORCH_CHECK(tickets.is_cuda() && tickets.scalar_type() == at::kInt && tickets.is_contiguous() && tickets.numel() >= B * p.H,
+              "attn_decode: int32 tickets, B H of them");
+  Tensor part;
+  if (p.splits > 1) {
+    part = at::empty({B * p.H * p.splits * p.maps * (p.V + 2)}, buf.options().dtype(at::kFloat));
+    p.part = part.data_ptr<float>();
+    p.tickets = tickets.data_ptr<int>();
+  }
+  check_rc(nxd::attn_decode_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "attn_decode");
+}
+
+// y = epi(x w^T), 1..16 rows of bf16; x bf16 [M, K], or u fp32 [M, K] normalised on the way in.  epi: 0 bf16,
+// 1 squared ReLU, 2 fp32 with cap, 3 into the streams (y unused, `un` receives the next sublayer's input)
+void gemv_hyper(int64_t epi, Opt x, Opt u, Opt norm_w, double eps, Tensor w, Opt y, double cap, Opt streams, Opt bias, Opt mix,
+                Opt write, Opt read, Opt un) {
+  nxd::GemvHyperParams p{};
+  TORCH_CHECK(epi >= 0 && epi <= 3, "gemv_hyper: epi 0..3");
+  TORCH_CHECK(x.has_value() != u.has_value() && u.has_value() == norm_w.has_value(), "gemv_hyper: x, or u with norm_w");
+  TORCH_CHECK(w.is_cuda() && w.dim() == 2 && w.scalar_type() == at::kBFloat16 && w.stride(1) == 1 && w.stride(0) % 8 == 0,
+              "gemv_hyper: w bf16 [N, K]");
+  const Tensor& in = x.has_value() ? *x : *u;
+  TORCH_CHECK(in.is_cuda() && in.dim() == 2 && in.size(1) == w.size(1) && in.stride(1) == 1, "gemv_hyper: input [M, K]");
+  const int64_t M = in.size(0), N = w.size(0), K = w.size(1);
+  TORCH_CHECK(M >= 1 && M <= 16 && N >= 1 && K >= 8 && K % 8 == 0, "gemv_hyper: 1..16 rows, K a multiple of 8");
+  check_align(in, "input");
+  check_align(w, "w");
+  p.M = (int)M;
+  p.N = (int)N;
+  p.K = (int)K;
+  p.w = static_cast<const uint16_t*>(w.data_ptr());
+  p.ldw = w.stride(0);
+  p.eps = (float)eps;
+  p.cap = (float)cap;
+  if (x.has_value()) {
+    TORCH_CHECK(x->scalar_type() == at::kBFloat16 && x->stride(0) % 8 == 0, "gemv_hyper: x bf16, rows 16-byte aligned");
+    p.x = static_cast<const uint16_t*>(x->data_ptr());
+    p.ldx = x->stride(0);
+  } else {
+    p.u = f32_ptr(*u, M * K, "u");
+    p.norm_w = f32_ptr(*norm_w, K, "norm_w");
+    check_align(*norm_w, "norm_w");
+    TORCH_CHECK(M * K <= 32768, "gemv_hyper: normalised rows must fit 64 KB of LDS");
+  }
+  if (epi == 3) {
+    TORCH_CHECK(x.has_value() && streams.has_value() && mix.has_value() && write.has_value() && read.has_value() && un.has_value(),
+                "gemv_hyper: streams, mix, write, read, un");
+    TORCH_CHECK(streams->dim() == 3 && streams->size(0) == M && streams->size(2) == N && streams->size(1) >= 1 && streams->size(1) <= 8,
+                "gemv_hyper: streams [M, S, N]");
+    p.S = (int)streams->size(1);
+    p.streams = f32_ptr(*streams, M * p.S * N, "streams");
+    p.bias = f32_opt(bias, N, "bias");
+    p.mix = f32_ptr(*mix, p.S * p.S, "mix");
+    p.write = f32_ptr(*write, p.S, "write");
+    p.read = f32_ptr(*read, p.S, "read");
+    p.un = f32_ptr(*un, M * N, "un");
+  } else {
+    TORCH_CHECK(y.has_value() && y->is_cuda() && y->dim() == 2 && y->size(0) == M && y->size(1) == N && y->stride(1) == 1 &&
+                    y->scalar_type() == (epi == 2 ? at::kFloat : at::kBFloat16),
+                "gemv_hyper: y [M, N]");
+    p.y = y->data_ptr();
+    p.ldy = y->stride(0);
+  }
+  check_rc(nxd::gemv_hyper_launch((int)epi, u.has_value(), p, cur_stream()), "gemv_hyper");
 }
 
 }  // namespace
@@ -316,4 +403,9 @@ PYBIND11_MODULE(_hybrid, m) {
   m.def("window_attn", &window_attn, py::arg("buf"), py::arg("B"), py::arg("T"), py::arg("sizes"), py::arg("scale"),
         py::arg("softcap"), py::arg("window"), py::arg("lam"), py::arg("out_scale"), py::arg("out_eps"), py::arg("pos"),
         py::arg("lens"), py::arg("slots"), py::arg("kc"), py::arg("vc"), py::arg("y"), py::arg("from_buf"), py::arg("fused") = true);
+  m.def("attn_decode", &attn_decode);
+  m.def("gemv_hyper", &gemv_hyper, py::arg("epi"), py::arg("x") = py::none(), py::arg("u") = py::none(),
+        py::arg("norm_w") = py::none(), py::arg("eps") = 0.0, py::arg("w"), py::arg("y") = py::none(), py::arg("cap") = 0.0,
+        py::arg("streams") = py::none(), py::arg("bias") = py::none(), py::arg("mix") = py::none(),
+        py::arg("write") = py::none(), py::arg("read") = py::none(), py::arg("un") = py::none());
 }

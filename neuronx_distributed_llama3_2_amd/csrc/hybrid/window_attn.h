@@ -31,8 +31,9 @@ struct WindowAttnParams {
   int64_t ldy;
   int from_buf;           // keys of this step's buffer (prompt from position 0) instead of the cache
   // split decode
-  float* part;            // [B H, splits, maps (V + 2)] partial sums
-  int splits;
+  int splits;             // workgroups per (sequence, head)
+  float* part;            // [B H, splits, maps (V + 2)] partial sums (splits > 1)
+  int* tickets;           // [B H] arrivals, zero between launches (splits > 1)
 };
 
 }  // namespace nxd

@@ -6,7 +6,7 @@
 //   attn_row    : one wave per (token, head), keys across lanes -- any size, fp32 or bf16, keys of the
 //                 buffer (prompt) or of the cache (any number of new tokens)
 //   attn_prompt : bf16 prompts on the matrix cores (window_attn_prompt.h)
-//   attn_split / attn_merge : one new token per sequence, the visible keys split over workgroups
+//   attn_decode : one new token per sequence, preparation included (window_attn_decode.hip)
 //
 // A key at position p lives in entry p % cap of the cache, so a windowed layer keeps about a window of
 // keys however long the sequence is.  Scores and weights are fp32.

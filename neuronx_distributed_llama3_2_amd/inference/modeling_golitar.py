@@ -3,8 +3,9 @@ attention mixers and squared-ReLU feed-forwards.
 
 The residual is [rows, streams, width] in fp32; between two sublayers one kernel (ops.hyper_step)
 writes the last sublayer's output into the streams and reads and normalises the next one's input, so a
-layer of the unfused forward is: hyper_step, projection GEMM, mixer kernels, output GEMM (and the same
-around the feed-forward).  The step function, cache set-up and decode-graph hooks are those of every
+layer of the forward is: hyper_step, projection GEMM, mixer kernels, output GEMM (and the same around the
+feed-forward).  A decode step of up to 16 sequences folds the norms into the input projections and the
+stream updates into the output projections (_forward_decode_fused_streams).  The step function, cache set-up and decode-graph hooks are those of every
 model of the framework (model_base.DecoderInferenceMixin); the cache is a LayerCache.
 """
 
@@ -21,6 +22,7 @@ from ..modules.hybrid import (DifferentialAttentionMixer, GatedDeltaMixer, Hyper
                               StepContext)
 from ..modules.hybrid.context import small
 from ..ops.gemm import linear_f32
+from ..ops.hyper import FUSED_NORM_ELEMENTS, FUSED_ROWS
 from ..parallel_layers.parallel_state import get_tensor_model_parallel_size
 from .layer_cache import LayerCache
 from .model_base import DecoderInferenceMixin
@@ -82,7 +84,8 @@ class GolitarInferenceModel(DecoderInferenceMixin, nn.Module):
         for layer in self.model.layers:
             if hasattr(layer.mixer, "weights_changed"):
                 layer.mixer.weights_changed()
-        self._plan = None
+        if self._decode_fused_ok:   # (kept off when it was switched off)
+            self._decode_fused_ok = None
 
     # ------------------------------------------------------------------ cache
     def setup_kv_cache(self, max_batch: int, max_len: int, device=None) -> LayerCache:
@@ -105,14 +108,30 @@ class GolitarInferenceModel(DecoderInferenceMixin, nn.Module):
 
     # ------------------------------------------------------------------ forward
     def _sublayers(self):
-        """(kind, module, output bias, hyper-connection, norm) of every sublayer in order."""
+        """(cache index, module, hyper-connection, norm) of every sublayer in order."""
         for i, layer in enumerate(self.model.layers):
-            yield i, layer.mixer, layer.mixer.o_bias, layer.hyper[0], layer.norms[0]
+            yield i, layer.mixer, layer.hyper[0], layer.norms[0]
             if layer.mlp is not None:
-                yield None, layer.mlp, None, layer.hyper[1], layer.norms[1]
+                yield None, layer.mlp, layer.hyper[1], layer.norms[1]
+
+    def _fused(self, input_ids: torch.Tensor) -> bool:
+        """Fused kernels wanted (set_fused_decode) and possible (GPU)."""
+        return self._decode_fused_ok is not False and input_ids.is_cuda
+
+    def _check_decode_fusable(self) -> bool:
+        ws = [self.lm_head.weight] + [m.weight for _, mod, _, _ in self._sublayers() for m in (mod.in_linear, mod.out_linear)]
+        return all(w.dtype == torch.bfloat16 and w.shape[1] % 8 == 0 and w.is_contiguous() for w in ws)
 
     def _decode_fusable(self, input_ids: torch.Tensor) -> bool:
-        return self._decode_fused_ok is not False and input_ids.is_cuda
+        """One new token for up to FUSED_ROWS sequences with every projection a fused GEMV."""
+        if not self._fused(input_ids):
+            return False
+        if self._decode_fused_ok is None:
+            self._gemv_ok = self._check_decode_fusable()
+            self._decode_fused_ok = True
+        M = input_ids.shape[0]
+        return (self._gemv_ok and input_ids.shape[1] == 1 and M <= FUSED_ROWS
+                and M * self.config.hidden_size <= FUSED_NORM_ELEMENTS)
 
     @torch.no_grad()
     def forward_tokens(self, input_ids: torch.Tensor, positions: torch.Tensor, seq_ids: Optional[torch.Tensor] = None,
@@ -131,23 +150,48 @@ class GolitarInferenceModel(DecoderInferenceMixin, nn.Module):
         ctx = StepContext(B, T, positions if positions.dtype == torch.int64 else positions.long(),
                           lengths.to(torch.int32) if lengths is not None else None,
                           seq_ids.to(torch.int32) if seq_ids is not None else None, prefill,
-                          self._decode_fusable(input_ids))
+                          self._fused(input_ids))
         emb = self.model.embed_tokens.weight
         M, dt = B * T, emb.dtype
         if logit_rows is None and last_index is not None:
             logit_rows = torch.arange(B, device=input_ids.device) * T + last_index
         streams = torch.empty((M, self.config.streams, emb.shape[1]), dtype=torch.float32, device=emb.device)
         last = dict(embed=emb, ids=input_ids.reshape(-1).to(torch.int64).contiguous())
-        for index, mod, bias, hc, norm in self._sublayers():
+        if not prefill and lengths is None and self._decode_fusable(input_ids):
+            return self._forward_decode_fused_streams(streams, last, ctx, logit_rows, return_hidden)
+        for index, mod, hc, norm in self._sublayers():
             h = ops.hyper_step(streams, read=hc.read, norm_w=norm, eps=self.eps, dtype=dt, **last)
-            y = mod(h) if index is None else mod(h, self.kv_cache[index], ctx)
-            last = dict(y=y, y_bias=bias, mix=hc.mix, write=hc.write)
+            y = mod(h, self.kv_cache[index] if index is not None else None, ctx)
+            last = dict(y=y, y_bias=mod.o_bias, mix=hc.mix, write=hc.write)
         h = ops.hyper_step(streams, read=self._ones(emb.device), norm_w=self.model.norm.weight, eps=self.eps, dtype=dt,
                            rows=logit_rows, store=False, **last)
         logits = self._logits(h)
         if logit_rows is None:
             logits, h = logits.view(B, T, -1), h.view(B, T, -1)
         return (logits, h) if return_hidden else logits
+
+    def _forward_decode_fused_streams(self, streams, start, ctx, logit_rows, return_hidden):
+        """One new token per sequence.  A sublayer is three launches: norm + input projection, mixer core
+        (none for a feed-forward), output projection + streams; the first one's input comes from the
+        embedding launch, the last streams launch reads their sum for the final norm + lm_head."""
+        subs = list(self._sublayers())
+        ones = self._ones(streams.device)
+        dt = self.model.embed_tokens.weight.dtype
+        x, u = ops.hyper_step(streams, read=subs[0][2].read, norm_w=subs[0][3], eps=self.eps, dtype=dt, **start), None
+        for i, (index, mod, hc, norm) in enumerate(subs):
+            a = ops.decode_linear(mod.in_linear.weight, x, u, None if u is None else norm, self.eps, mod.in_epilogue)
+            a = mod.core(a, self.kv_cache[index] if index is not None else None, ctx)
+            read = subs[i + 1][2].read if i + 1 < len(subs) else ones
+            u = ops.decode_linear_into_streams(mod.out_linear.weight, a, streams, mod.o_bias, hc.mix, hc.write, read)
+            x = None
+        norm = self.model.norm.weight
+        if logit_rows is not None:
+            u = u[logit_rows]
+        logits = ops.decode_linear(self.lm_head.weight, None, u, norm, self.eps, "f32", self.config.logit_softcap)
+        if not return_hidden:
+            return logits if logit_rows is not None else logits.unsqueeze(1)
+        h = (u * torch.rsqrt(u.square().mean(-1, keepdim=True) + self.eps) * (1 + norm)).to(dt)
+        return (logits, h) if logit_rows is not None else (logits.unsqueeze(1), h.unsqueeze(1))
 
     def _forward_in_steps(self, input_ids, positions, seq_ids, last_index, return_hidden, lengths, logit_rows, step):
         B, T = input_ids.shape

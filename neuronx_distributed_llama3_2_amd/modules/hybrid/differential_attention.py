@@ -28,6 +28,7 @@ def interleaved_rope_tables(dims: int, base: float, max_pos: int, factor: Option
 
 
 class DifferentialAttentionMixer(nn.Module):
+    in_epilogue = "store"
     recurrent = False
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, diff: float, scale: float,
@@ -82,18 +83,33 @@ class DifferentialAttentionMixer(nn.Module):
         if self.window:
             cap = min(max_len, (self.window + RING_SLACK + 63) // 64 * 64)
         z = lambda *shape: torch.zeros(shape, dtype=dtype, device=device)  # noqa: E731
-        return {"k": z(slots, s.kv_heads * s.maps, cap, s.dim), "v": z(slots, s.kv_heads, cap, s.vdim)}
+        return {"k": z(slots, s.kv_heads * s.maps, cap, s.dim), "v": z(slots, s.kv_heads, cap, s.vdim),
+                "tickets": torch.zeros(slots * s.heads, dtype=torch.int32, device=device)}
 
     def max_new_tokens(self, cache: Dict[str, torch.Tensor], max_len: int) -> int:
         """Tokens one decode step may bring: the ring must still hold what the first of them sees."""
         cap = cache["k"].shape[2]
         return max_len if cap >= max_len else cap - self.window + 1
 
-    def forward(self, h: torch.Tensor, cache: Dict[str, torch.Tensor], ctx: StepContext) -> torch.Tensor:
+    @property
+    def in_linear(self) -> nn.Linear:
+        return self.qkv_proj
+
+    @property
+    def out_linear(self) -> nn.Linear:
+        return self.o_proj
+
+    def core(self, buf: torch.Tensor, cache: Dict[str, torch.Tensor], ctx: StepContext) -> torch.Tensor:
+        """From the input projection's output (whose q / k / v it may overwrite) to the output projection's
+        input."""
         cos_t, sin_t = self._tables
-        buf = linear(h, self.qkv_proj)
+        if ctx.fused and ctx.T == 1 and not ctx.prompt and ctx.lengths is None:
+            return ops.attn_decode(buf, self.sizes, self.rule, self.qkv_bias, self.q_norm, self.k_norm, self.eps, cos_t,
+                                   sin_t, ctx.positions, ctx.slots, cache["k"], cache["v"], cache["tickets"])
         ops.attn_prep_(buf, ctx.B, ctx.T, self.sizes, self.qkv_bias, self.q_norm, self.k_norm, self.eps, cos_t, sin_t,
                        ctx.positions, ctx.lengths, ctx.slots, cache["k"], cache["v"])
-        y = ops.window_attention(buf, ctx.B, ctx.T, self.sizes, self.rule, ctx.positions, ctx.lengths, ctx.slots,
-                                 cache["k"], cache["v"], ctx.prompt, ctx.fused)
-        return linear(y, self.o_proj)
+        return ops.window_attention(buf, ctx.B, ctx.T, self.sizes, self.rule, ctx.positions, ctx.lengths, ctx.slots,
+                                    cache["k"], cache["v"], ctx.prompt, ctx.fused)
+
+    def forward(self, h: torch.Tensor, cache: Dict[str, torch.Tensor], ctx: StepContext) -> torch.Tensor:
+        return linear(self.core(linear(h, self.qkv_proj), cache, ctx), self.o_proj)

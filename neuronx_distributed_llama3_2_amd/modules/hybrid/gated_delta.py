@@ -13,6 +13,7 @@ from .context import StepContext, linear, padded_rows, small
 
 
 class GatedDeltaMixer(nn.Module):
+    in_epilogue = "store"
     recurrent = True   # a step changes what the cache holds of earlier tokens
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, conv: int, eps: float,
@@ -44,8 +45,18 @@ class GatedDeltaMixer(nn.Module):
     def max_new_tokens(self, cache: Dict[str, torch.Tensor], max_len: int) -> int:
         return max_len
 
+    @property
+    def in_linear(self) -> nn.Linear:
+        return self.in_proj
+
+    @property
+    def out_linear(self) -> nn.Linear:
+        return self.o_proj
+
+    def core(self, proj: torch.Tensor, cache: Dict[str, torch.Tensor], ctx: StepContext) -> torch.Tensor:
+        """From the input projection's output to the output projection's input."""
+        return ops.delta_rule(proj, ctx.B, ctx.T, self.sizes, self.conv, self.a_log, self.dt_bias, self.out_norm,
+                              self.eps, ctx.positions, ctx.lengths, ctx.slots, cache["state"], cache["ring"], ctx.fused)
+
     def forward(self, h: torch.Tensor, cache: Dict[str, torch.Tensor], ctx: StepContext) -> torch.Tensor:
-        y = ops.delta_rule(linear(h, self.in_proj), ctx.B, ctx.T, self.sizes, self.conv, self.a_log, self.dt_bias,
-                           self.out_norm, self.eps, ctx.positions, ctx.lengths, ctx.slots, cache["state"],
-                           cache["ring"], ctx.fused)
-        return linear(y, self.o_proj)
+        return linear(self.core(linear(h, self.in_proj), cache, ctx), self.o_proj)

@@ -66,3 +66,30 @@ def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
         hybrid_ext().softcap_(x, float(cap))
         return x
     return x.copy_(cap * torch.tanh(x / cap))
+
+
+# most rows the fused decode projections take, and the LDS limit on normalised rows (rows x columns)
+FUSED_ROWS = 16
+FUSED_NORM_ELEMENTS = 32768
+
+_EPI = {"store": 0, "relu2": 1, "f32": 2, "streams": 3}
+
+
+def decode_linear(w: torch.Tensor, x: Optional[torch.Tensor] = None, u: Optional[torch.Tensor] = None,
+                  norm_w: Optional[torch.Tensor] = None, eps: float = 0.0, epilogue: str = "store", cap: float = 0.0):
+    """epilogue(x w^T) for a few rows in one launch (csrc/hybrid/gemv_hyper.hip, GPU, bf16 weights): x
+    bf16 [M, K], or u fp32 [M, K], normalised as hyper_step does on the way in.  "store": bf16, "relu2":
+    bf16 squared ReLU, "f32": fp32, with cap > 0 cap tanh(y / cap)."""
+    M = (x if x is not None else u).shape[0]
+    y = torch.empty((M, w.shape[0]), dtype=torch.float32 if epilogue == "f32" else torch.bfloat16, device=w.device)
+    hybrid_ext().gemv_hyper(_EPI[epilogue], x, u, norm_w, float(eps), w, y, float(cap))
+    return y
+
+
+def decode_linear_into_streams(w: torch.Tensor, x: torch.Tensor, streams: torch.Tensor, bias: Optional[torch.Tensor],
+                               mix: torch.Tensor, write: torch.Tensor, read: torch.Tensor) -> torch.Tensor:
+    """The output projection of a sublayer with the write into the streams as its epilogue (in place);
+    returns u [M, W] fp32, what the next sublayer reads before its norm."""
+    un = torch.empty((x.shape[0], w.shape[0]), dtype=torch.float32, device=w.device)
+    hybrid_ext().gemv_hyper(_EPI["streams"], x, None, None, 0.0, w, None, 0.0, streams, bias, mix, write, read, un)
+    return un

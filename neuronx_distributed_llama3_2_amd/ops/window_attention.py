@@ -138,3 +138,22 @@ def window_attention(buf: torch.Tensor, B: int, T: int, sizes: AttnSizes, rule: 
             o = o / torch.sqrt(o.square().mean(-1, keepdim=True) + rule.eps) * rule.out_scale
         y[b * T:b * T + n] = o.reshape(n, H * V).to(y.dtype)
     return y
+
+
+def attn_decode(buf: torch.Tensor, sizes: AttnSizes, rule: AttnRule, bias: Optional[torch.Tensor],
+                q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor], eps: float, cos_t: torch.Tensor,
+                sin_t: torch.Tensor, positions: torch.Tensor, slots: Optional[torch.Tensor], k_cache: torch.Tensor,
+                v_cache: torch.Tensor, tickets: torch.Tensor) -> torch.Tensor:
+    """attn_prep_ and window_attention for one new token per sequence in one launch
+    (csrc/hybrid/window_attn_decode.hip); buf [B, >= columns] is left as it is.  tickets: int32 zeros,
+    B * heads of them, left at zero."""
+    B = buf.shape[0]
+    if use_native(buf):
+        y = torch.empty((B, sizes.heads * sizes.vdim), dtype=buf.dtype, device=buf.device)
+        hybrid_ext().attn_decode(buf, sizes.as_list(), bias, q_norm, k_norm, float(eps), cos_t, sin_t, rule.scale,
+                                 rule.softcap, rule.window, rule.lam, rule.out_scale, rule.eps, positions, slots,
+                                 k_cache, v_cache, tickets, y)
+        return y
+    buf = buf.clone()
+    attn_prep_(buf, B, 1, sizes, bias, q_norm, k_norm, eps, cos_t, sin_t, positions, None, slots, k_cache, v_cache)
+    return window_attention(buf, B, 1, sizes, rule, positions, None, slots, k_cache, v_cache, False)
