@@ -46,11 +46,10 @@ def causal_conv(x, taps):
     """x [T, C], taps [C, n] (last column = current token) -> [T, C]; zeros before the start."""
     T, n = x.shape[0], taps.shape[1]
     out = torch.zeros_like(x)
-    for t in range(T):
-        for j in range(n):
-            src = t - (n - 1 - j)
-            if src >= 0:
-                out[t] += taps[:, j] * x[src]
+    for j in range(n):
+        back = n - 1 - j   # column j meets the input `back` tokens ago
+        if back < T:
+            out[back:] += taps[:, j] * x[:T - back]
     return out
 
 
@@ -113,13 +112,12 @@ def rotary_frequencies(rot):
 def rotate_interleaved(x, freqs, pos0=0):
     """x [T, ..., D]: pair (2i, 2i + 1) of row t turned by (pos0 + t) freqs[i]; the rest unchanged."""
     out = x.clone()
-    for t in range(x.shape[0]):
-        for i, f in enumerate(freqs):
-            a = (pos0 + t) * f
-            c, s = math.cos(a), math.sin(a)
-            u, v = x[t, ..., 2 * i], x[t, ..., 2 * i + 1]
-            out[t, ..., 2 * i] = u * c - v * s
-            out[t, ..., 2 * i + 1] = v * c + u * s
+    pos = torch.arange(pos0, pos0 + x.shape[0], dtype=x.dtype).view((-1,) + (1,) * (x.dim() - 2))
+    for i, f in enumerate(freqs):
+        c, s = torch.cos(pos * f), torch.sin(pos * f)
+        u, v = x[..., 2 * i], x[..., 2 * i + 1]
+        out[..., 2 * i] = u * c - v * s
+        out[..., 2 * i + 1] = v * c + u * s
     return out
 
 
@@ -130,14 +128,11 @@ def visible(i, j, window):
 def attention_map(q, k, v, scale, softcap, window):
     """One head's map: q, k [T, D], v [T, V] -> [T, V]."""
     T = q.shape[0]
-    out = torch.zeros(T, v.shape[1], dtype=q.dtype)
-    for i in range(T):
-        js = [j for j in range(T) if visible(i, j, window)]
-        s = (k[js] @ q[i]) * scale
-        if softcap:
-            s = softcap * torch.tanh(s / softcap)
-        out[i] = torch.softmax(s, 0) @ v[js]
-    return out
+    seen = torch.tensor([[visible(i, j, window) for j in range(T)] for i in range(T)])
+    s = (q @ k.T) * scale
+    if softcap:
+        s = softcap * torch.tanh(s / softcap)
+    return torch.softmax(s.masked_fill(~seen, float("-inf")), -1) @ v
 
 
 def lambda_of(W, pre, diff):

@@ -1,0 +1,329 @@
+"""The Golitar model through the framework's own loader, registry, cache, batch sessions and generate(),
+against the plain implementation in golitar_oracle.py (CPU: the package's reference operations; GPU: the
+HIP kernels in fp32 and bf16)."""
+
+import io
+import json
+import os
+import subprocess
+import sys
+
+import pytest
+import torch
+
+import golitar_oracle as O
+from golitar_cases import CONFIGS, attention, config, delta, doubles, rel_err, tokens, weights, write_model
+from neuronx_distributed_llama3_2_amd.inference import (BatchSession, GolitarForCausalLMInference, GolitarRunner,
+                                                        InferenceConfig, app_class, runner_class)
+from neuronx_distributed_llama3_2_amd.inference.registry import family_name
+from neuronx_distributed_llama3_2_amd.inference.trace_replay import replay
+from neuronx_distributed_llama3_2_amd.models.golitar import GolitarConfig
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+GPU = pytest.mark.gpu
+# (device, dtype, relative tolerance); the CPU variants stay on the CPU also where a GPU is visible
+WHERE = [pytest.param((torch.device("cpu"), torch.float32, 3e-4), id="cpu"),
+         pytest.param((torch.device("cuda", 0), torch.float32, 3e-4), id="gpu-fp32", marks=GPU),
+         pytest.param((torch.device("cuda", 0), torch.bfloat16, 6e-2), id="gpu-bf16", marks=GPU)]
+
+
+_ORACLE = {}
+
+
+def oracle_logits(name, toks, seed=0):
+    key = (name, tuple(toks), seed)
+    if key not in _ORACLE:
+        _ORACLE[key] = O.forward(CONFIGS[name], doubles(weights(CONFIGS[name], seed)), toks)
+    return _ORACLE[key]
+
+
+def make_app(path, device, dtype, max_len=256, batch=4, **kw):
+    kw.setdefault("enable_bucketing", True)
+    cfg = InferenceConfig(batch_size=batch, seq_len=max_len, **kw)
+    mc = GolitarConfig.from_pretrained(path)
+    app = GolitarForCausalLMInference(mc, cfg, dtype, device=device, init_weights=False)
+    from neuronx_distributed_llama3_2_amd.inference.generation import load_hf_state_dict
+
+    app._load_full(app._hf_to_nxd(load_hf_state_dict(path), mc))
+    return app
+
+
+@pytest.fixture(scope="module")
+def model_dirs(tmp_path_factory):
+    out = {}
+    for name, cfg in CONFIGS.items():
+        out[name] = write_model(tmp_path_factory.mktemp(name), cfg, weights(cfg))
+    return out
+
+
+NAMES = sorted(CONFIGS)
+
+
+@pytest.mark.parametrize("where", WHERE)
+@pytest.mark.parametrize("name", NAMES)
+def test_prompt_portions_and_decoding(where, name, model_dirs):
+    """One sequence: the whole prompt in one step; the prompt cut at several places (down to two tokens);
+    most of it decoded token by token."""
+    device, dtype, tol = where
+    T = 120
+    toks = tokens(T, CONFIGS[name]["vocab"])
+    want = oracle_logits(name, toks)
+    app = make_app(model_dirs[name], device, dtype)
+    s = BatchSession(app)
+    assert rel_err(s.step([("a", toks, range(T))]), want) < tol
+    s.end(["a"])
+    got = [s.step([("a", toks[:40], range(40))])]
+    for t in range(40, T):
+        got.append(s.step([("a", [toks[t]], [0])]))
+    assert rel_err(torch.cat(got), want) < tol
+    s.end(["a"])
+    # several new tokens at a time over the cache (the step function's general form)
+    for first, cut in ((1, 2), (30, 16), (50, 70)):
+        ids = torch.tensor([toks], device=device)
+        pos = torch.arange(T, device=device).unsqueeze(0)
+        slot = torch.tensor([2], device=device)
+        fwd = app.model.forward_tokens
+        got = [fwd(ids[:, :first], pos[:, :first], slot, prefill=True)[0]]
+        for t in range(first, T, cut):
+            got.append(fwd(ids[:, t:t + cut], pos[:, t:t + cut], slot)[0])
+        assert rel_err(torch.cat(got), want) < tol, (first, cut)
+
+
+@pytest.mark.parametrize("where", WHERE)
+@pytest.mark.parametrize("name", ["mixed", "one_stream"])
+def test_batches_of_unequal_requests(where, name, model_dirs):
+    """Requests of different lengths together, each leaving as it ends, against each alone; then another
+    batch in the slots they have left."""
+    device, dtype, tol = where
+    app = make_app(model_dirs[name], device, dtype)
+    s = BatchSession(app)
+    V = CONFIGS[name]["vocab"]
+    for rnd, plan in enumerate(({"a": (1, 4), "b": (33, 12), "c": (90, 8), "d": (7, 15)}, {"e": (64, 9), "f": (2, 5)})):
+        seqs = {r: tokens(p + d, V, seed=10 * rnd + i) for i, (r, (p, d)) in enumerate(plan.items())}
+        want = {r: oracle_logits(name, t) for r, t in seqs.items()}
+        out = s.step([(r, seqs[r][:p], range(p)) for r, (p, _) in plan.items()])
+        got = dict(zip(plan, torch.split(out, [p for p, _ in plan.values()])))
+        done = 0
+        live = list(plan)
+        while live:
+            out = s.step([(r, [seqs[r][plan[r][0] + done]], [0]) for r in live])
+            for r, row in zip(live, out):
+                got[r] = torch.cat([got[r], row[None]])
+            done += 1
+            gone = [r for r in live if plan[r][1] == done]
+            s.end(gone)
+            live = [r for r in live if r not in gone]
+        for r in plan:
+            assert rel_err(got[r], want[r]) < tol, r
+    assert s._free == list(range(app.max_batch))
+
+
+@pytest.mark.parametrize("where", WHERE)
+def test_long_decoding(where, tmp_path):
+    """Decoding far past every window, so that the key rings wrap several times."""
+    device, dtype, tol = where
+    name = "long"
+    CONFIGS[name] = config([attention(window=17, ff=None), delta(conv=3), attention(window=66, ff=40)], width=48, vocab=71)
+    toks = tokens(300 if device.type == "cuda" else 220, 71)
+    want = oracle_logits(name, toks)
+    app = make_app(write_model(tmp_path / "m", CONFIGS[name], weights(CONFIGS[name])), device, dtype, max_len=len(toks), batch=1)
+    assert app.model.kv_cache[0]["k"].shape[2] == 64   # one window and some, not the whole sequence
+    s = BatchSession(app)
+    got = [s.step([("a", toks[:3], range(3))])]
+    for t in range(3, len(toks)):
+        got.append(s.step([("a", [toks[t]], [0])]))
+    assert rel_err(torch.cat(got), want) < tol
+
+
+def greedy(name, prompt, n, seed=0):
+    W, cfg, toks = doubles(weights(CONFIGS[name], seed)), CONFIGS[name], list(prompt)
+    for _ in range(n):
+        toks.append(int(O.forward(cfg, W, toks)[-1].argmax()))
+    return toks
+
+
+@pytest.mark.parametrize("where", WHERE[:2])
+def test_greedy_generation(where, model_dirs):
+    """generate(): right-padded prompts of different lengths, greedy, decode graphs on the GPU.  Twice with
+    the same application: the second call finds captured graphs and used slots."""
+    name = "mixed"
+    app = make_app(model_dirs[name], where[0], where[1], max_len=64, decode_graph_steps=4)
+    V = CONFIGS[name]["vocab"]
+    prompts = [tokens(9, V, seed=21), tokens(17, V, seed=22)]
+    ids = torch.zeros((2, 17), dtype=torch.long)
+    mask = torch.zeros((2, 17), dtype=torch.long)
+    for i, p in enumerate(prompts):
+        ids[i, :len(p)] = torch.tensor(p)
+        mask[i, :len(p)] = 1
+    want = [greedy(name, p, 10)[len(p):] for p in prompts]
+    for _ in range(2):
+        out = app.generate(ids, mask, max_new_tokens=10).cpu()
+        assert [out[i, 17:].tolist() for i in range(2)] == want
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("graphs", [True, False])
+def test_generation_bf16(graphs, model_dirs):
+    """bf16: every generated token has the largest logit, or one within rounding of it, when the same
+    tokens are fed step by step; captured graphs and eager steps, replays after the first."""
+    device = torch.device("cuda", 0)
+    app = make_app(model_dirs["wide_heads"], device, torch.bfloat16, max_len=200, decode_graph_steps=8, use_hip_graphs=graphs)
+    V = CONFIGS["wide_heads"]["vocab"]
+    prompts = torch.tensor([tokens(40, V, seed=31), tokens(40, V, seed=32)])
+    out = app.generate(prompts, max_new_tokens=100, eos_token_id=-1).cpu()
+    s = BatchSession(app)
+    logits = [s.step([("a", out[0, :40].tolist(), [39]), ("b", out[1, :40].tolist(), [39])])]
+    for t in range(40, 139):
+        logits.append(s.step([("a", [int(out[0, t])], [0]), ("b", [int(out[1, t])], [0])]))
+    logits = torch.stack(logits, 1).float().cpu()   # [2, 100, V]
+    chosen = logits.gather(2, out[:, 40:].unsqueeze(-1)).squeeze(-1)
+    assert float((logits.max(-1).values - chosen).max()) < 0.1
+
+
+@pytest.mark.gpu
+def test_sampling(model_dirs):
+    app = make_app(model_dirs["mixed"], torch.device("cuda", 0), torch.bfloat16, max_len=96)
+    ids = torch.tensor([tokens(20, CONFIGS["mixed"]["vocab"])])
+    a = app.generate(ids, max_new_tokens=30, do_sample=True, top_k=8, temperature=1.2, seed=5)
+    b = app.generate(ids, max_new_tokens=30, do_sample=True, top_k=8, temperature=1.2, seed=5)
+    c = app.generate(ids, max_new_tokens=30, do_sample=True, top_k=8, temperature=1.2, seed=6)
+    assert torch.equal(a, b) and not torch.equal(a, c)
+
+
+@pytest.mark.gpu
+def test_fused_decode_switch(model_dirs):
+    """set_fused_decode(False) takes the unfused operations: the same logits up to rounding."""
+    app = make_app(model_dirs["wide_heads"], torch.device("cuda", 0), torch.bfloat16)
+    toks = tokens(60, CONFIGS["wide_heads"]["vocab"])
+    outs = []
+    for on in (True, False):
+        app.set_fused_decode(on)
+        s = BatchSession(app)
+        o = [s.step([("a", toks[:30], range(30))])]
+        o += [s.step([("a", [t], [0])]) for t in toks[30:]]
+        outs.append(torch.cat(o))
+        s.end(["a"])
+    assert rel_err(outs[0], outs[1].cpu()) < 4e-2
+
+
+def test_registry_and_runner(model_dirs, tmp_path):
+    path = model_dirs["mixed"]
+    assert app_class(path) is GolitarForCausalLMInference and runner_class(path) is GolitarRunner
+    assert family_name({"architectures": ["LlamaForCausalLM"], "model_type": "llama"}) == "llama"
+    assert family_name({"architectures": ["MixtralForCausalLM"]}) == "mixtral"
+    with pytest.raises(ValueError):
+        family_name({"architecture": "SomethingElse"})
+    r = GolitarRunner(path)
+    m = r.load_neuron_model_on_cpu(16, 32, 1)
+    if m.device.type == "cpu":
+        out = r.generate_on_neuron([tokens(8, 211)], m, max_length=14)
+        assert out[0].tolist() == greedy("mixed", tokens(8, 211), 6)
+
+
+def test_compile_and_load(model_dirs, tmp_path):
+    """The compiled form (framework names, per-rank file) serves the same logits."""
+    device = torch.device("cpu")
+    app = make_app(model_dirs["mixed"], device, torch.float32, batch=1)
+    app.compile(str(tmp_path / "c"))
+    toks = tokens(25, 211)
+    a = BatchSession(app).step([("x", toks, range(25))])
+    assert app_class(str(tmp_path / "c")) is GolitarForCausalLMInference
+    if torch.cuda.is_available():
+        return   # load() picks the GPU there; covered by the bf16 test below
+    again = GolitarForCausalLMInference.load(str(tmp_path / "c"), dtype=torch.float32)
+    assert torch.equal(a, BatchSession(again).step([("x", toks, range(25))]))
+
+
+@pytest.mark.gpu
+def test_runner_on_gpu(model_dirs, tmp_path):
+    r = GolitarRunner(model_dirs["wide_heads"])
+    r.trace(str(tmp_path / "t"), batch_size=1, max_prompt_length=32, sequence_length=64)
+    m = r.load_neuron_model(str(tmp_path / "t"))
+    out = r.generate_on_neuron([tokens(20, 130)], m, max_length=40)
+    assert out.shape == (1, 40)
+    rep = r.benchmark_sampling(m, num_runs=2, report_path=str(tmp_path / "r.json"))
+    assert rep["e2e_model"]["throughput"] > 0
+
+
+def test_config_is_checked():
+    base = CONFIGS["mixed"]
+    for change in (lambda c: c["layers"][0].__setitem__("type", "other"),
+                   lambda c: c["layers"][2]["mlp"].__setitem__("kind", "sparse"),
+                   lambda c: c["layers"][0]["mixer"].__setitem__("kv_heads", 3),
+                   lambda c: c["layers"][1]["mixer"]["rot"].__setitem__("dims", 18),
+                   lambda c: c.__setitem__("streams", 9)):
+        c = json.loads(json.dumps(base))
+        change(c)
+        with pytest.raises(ValueError):
+            GolitarConfig(c)
+    c = json.loads(json.dumps(base))
+    del c["layers"][1]["mixer"]["softcap"], c["logit_softcap"], c["layers"][1]["mixer"]["mask"]
+    cfg = GolitarConfig(c)
+    assert cfg.layers[1].mixer.softcap == 0 and cfg.layers[1].mixer.window == 0 and cfg.logit_softcap == 0
+
+
+def test_missing_weights_are_reported(tmp_path):
+    cfg = CONFIGS["mixed"]
+    sd = weights(cfg)
+    del sd["l1.hc2.mix"]
+    with pytest.raises(KeyError):
+        make_app(write_model(tmp_path, cfg, sd), torch.device("cpu"), torch.float32)
+
+
+def test_session_and_replay_errors(model_dirs):
+    app = make_app(model_dirs["one_stream"], torch.device("cpu"), torch.float32, max_len=32, batch=1)
+    s = BatchSession(app)
+    toks = tokens(12, 53)
+    with pytest.raises(ValueError):
+        s.step([("a", toks, [12])])
+    s.step([("a", toks[:5], []), ("b", toks[:3], [])])   # more requests than slots: the cache grows
+    assert app.max_batch == 2
+    for bad in ([("c", toks[:2], [])], [("a", toks[:2], [])], [("a", [1], []), ("a", [1], [])], [("a", [], [])]):
+        with pytest.raises(ValueError):
+            s.step(bad)
+    s.end(["a", "b"])
+    with pytest.raises(ValueError):
+        s.step([("a", tokens(40, 53), [])])
+
+
+def test_replay_writes_the_wanted_logits(model_dirs, tmp_path):
+    name = "one_stream"
+    app = make_app(model_dirs[name], torch.device("cpu"), torch.float32, max_len=64, batch=1)
+    a, b = tokens(11, 53, seed=1), tokens(6, 53, seed=2)
+    lines = [json.dumps({"step": 0, "entries": [{"id": "a", "tokens": a[:9], "want": [8, 2]}, {"id": "b", "tokens": b[:5], "want": []}],
+                         "end": []}),
+             json.dumps({"step": 1, "entries": [{"id": "b", "tokens": b[5:], "want": [0]}, {"id": "a", "tokens": a[9:10], "want": []}],
+                         "end": ["b"]}),
+             json.dumps({"step": 2, "entries": [{"id": "a", "tokens": a[10:], "want": []}], "end": ["a"]})]
+    out = io.StringIO()
+    replay(BatchSession(app), lines, str(tmp_path), out)
+    assert out.getvalue().split("\n")[:3] == ["done 0", "done 1", "done 2"]
+    load = lambda n: torch.frombuffer(bytearray((tmp_path / n).read_bytes()), dtype=torch.float32).view(-1, 53)  # noqa: E731
+    wa, wb = oracle_logits(name, a), oracle_logits(name, b)
+    assert rel_err(load("0.f32"), wa[[8, 2]]) < 3e-4 and rel_err(load("1.f32"), wb[[5]]) < 3e-4
+    assert not (tmp_path / "2.f32").exists()
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype,tol", [("bfloat16", 6e-2), ("float32", 3e-4)])
+def test_trace_run_program(dtype, tol, model_dirs, tmp_path):
+    name = "mixed"
+    toks = tokens(30, 211, seed=4)
+    steps = [{"step": 0, "entries": [{"id": "q", "tokens": toks[:28], "want": list(range(28))}], "end": []},
+             {"step": 1, "entries": [{"id": "q", "tokens": toks[28:29], "want": [0]}], "end": []},
+             {"step": 2, "entries": [{"id": "q", "tokens": toks[29:], "want": [0]}], "end": ["q"]}]
+    r = subprocess.run([os.path.join(ROOT, "bin", "trace_run"), "--model", model_dirs[name], "--dtype", dtype, "--out",
+                        str(tmp_path), "--max-tokens", "30"], input="".join(json.dumps(s) + "\n" for s in steps),
+                       capture_output=True, text=True, timeout=110, env=dict(os.environ, HOME=str(tmp_path)))
+    assert r.returncode == 0, r.stderr[-2000:]
+    got = torch.cat([torch.frombuffer(bytearray((tmp_path / f"{i}.f32").read_bytes()), dtype=torch.float32).view(-1, 211)
+                     for i in range(3)])
+    assert rel_err(got, oracle_logits(name, toks)) < tol
+
+
+def test_trace_run_needs_a_gpu(model_dirs, tmp_path):
+    """No CPU path behind the program."""
+    env = dict(os.environ, HIP_VISIBLE_DEVICES="", CUDA_VISIBLE_DEVICES="")
+    r = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", model_dirs["mixed"], "--out", str(tmp_path),
+                        "--max-tokens", "8"], input="", capture_output=True, text=True, timeout=600, env=env)
+    assert r.returncode != 0 and "GPU" in r.stderr
