@@ -106,7 +106,20 @@ def tokens(n, vocab, seed=1):
     return torch.randint(0, vocab, (n,), generator=torch.Generator().manual_seed(seed)).tolist()
 
 
-def rel_err(got, want):
-    """Root mean square of the difference over that of `want`, per row; the largest."""
+def row_errs(got, want):
+    """Root mean square of the difference over that of `want`, per row."""
     got, want = got.double().cpu(), want.double()
-    return float(((got - want).square().mean(-1).sqrt() / want.square().mean(-1).sqrt().clamp_min(1e-9)).max())
+    return (got - want).square().mean(-1).sqrt() / want.square().mean(-1).sqrt().clamp_min(1e-9)
+
+
+def rel_err(got, want):
+    return float(row_errs(got, want).max())
+
+
+def logits_agree(got, want, dtype):
+    """fp32: every row within 3e-4.  bf16: rounding alone moves single rows of these random models by up to
+    a tenth, so the average is what is held small."""
+    e = row_errs(got, want)
+    if dtype == torch.float32:
+        return float(e.max()) < 3e-4
+    return float(e.mean()) < 4e-2 and float(e.max()) < 0.25
