@@ -11,6 +11,8 @@ on a side stream), global batch 32 by default (the 1F1B bubble is (P-1)/(M+P-1) 
     python -m torch.distributed.run --nnodes=1 --nproc-per-node N --master-addr 127.0.0.1 \
         --master-port P bench.py --gpus N --steps K --warmup W
 
+`--serve golitar | llama` measures serving instead (prefill and decode tokens/s of one GPU).
+
 Without a launcher (no WORLD_SIZE in the environment) and N > 1, bench.py starts the N rank
 processes itself (child processes, before any HIP call) and waits for them.
 
@@ -73,6 +75,11 @@ def parse():
     ap.add_argument("--no-sp", action="store_true")
     ap.add_argument("--ckpt", default=None, help="activation checkpointing: None | full | selective")
     ap.add_argument("--lr", type=float, default=1e-5, help="AdamW learning rate (tests raise it so the loss moves)")
+    ap.add_argument("--serve", choices=["golitar", "llama"], default=None,
+                    help="instead of the training step: prefill and decode throughput of this model family at layer "
+                         "sizes of a real model, one GPU (inference/serve_bench.py; --steps timed repetitions)")
+    ap.add_argument("--serve-size", action="append", choices=["2k", "4k"], default=None, help="default: both")
+    ap.add_argument("--serve-phase", choices=["both", "prefill", "decode"], default="both")
     ap.add_argument("--cpu", action="store_true", help="force the CPU/gloo path (plumbing tests)")
     ap.add_argument("--gloo-gpu", action="store_true",
                     help="test mode: every rank on cuda:0 with gloo collectives on staged GPU tensors (multi-rank "
@@ -644,6 +651,11 @@ def main(a):
 
 if __name__ == "__main__":
     args = parse()
+    if args.serve is not None:
+        from neuronx_distributed_llama3_2_amd.inference.serve_bench import run
+
+        run(args.serve, args.serve_size, args.steps, args.serve_phase)
+        sys.exit(0)
     ladder = os.environ.get("NXD_BENCH_LADDER", "1") == "1" and os.environ.get("NXD_BENCH_CHILD") != "1"
     if "WORLD_SIZE" not in os.environ:
         if args.gpus > 1 or ladder:
