@@ -26,8 +26,9 @@ int attn_prep_launch(bool, const WindowAttnParams&, hipStream_t);
 bool attn_prompt_supported(const WindowAttnParams&);
 int attn_prompt_launch(const WindowAttnParams&, hipStream_t);
 int attn_row_launch(bool, const WindowAttnParams&, hipStream_t);
+void attn_decode_plan(WindowAttnParams&, int64_t);
 int attn_decode_launch(bool, const WindowAttnParams&, hipStream_t);
-int gemv_hyper_launch(int, bool, const GemvHyperParams&, hipStream_t);
+int gemv_hyper_launch(int, const GemvHyperParams&, hipStream_t);
 }  // namespace nxd
 
 namespace {
@@ -317,7 +318,7 @@ void attn_decode(Tensor buf, std::vector<int64_t> sizes, Opt bias, Opt qn_w, Opt
   set_rule(p, scale, softcap, window, lam, out_scale, out_eps, buf, y);
   TORCH_CHECK(p.H <= 65535 && B <= 65535, "attn_decode: grid");
   const int64_t seen = p.window > 0 ? std::min<int64_t>(p.window, p.cap) : p.cap;
-  p.splits = (int)((seen + 255) / 256);
+  nxd::attn_decode_plan(p, seen);
   TORCH_CHECK(tickets.is_cuda() && tickets.scalar_type() == at::kInt && tickets.is_contiguous() && tickets.numel() >= B * p.H,
               "attn_decode: int32 tickets, B H of them");
   Tensor part;
@@ -329,7 +330,7 @@ void attn_decode(Tensor buf, std::vector<int64_t> sizes, Opt bias, Opt qn_w, Opt
   check_rc(nxd::attn_decode_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "attn_decode");
 }
 
-// y = epi(x w^T), 1..16 rows of bf16; x bf16 [M, K], or u fp32 [M, K] normalised on the way in.  epi: 0 bf16,
+// y = epi(x w^T), 1..4 rows of bf16; x bf16 [M, K], or u fp32 [M, K] normalised on the way in.  epi: 0 bf16,
 // 1 squared ReLU, 2 fp32 with cap, 3 into the streams (y unused, `un` receives the next sublayer's input)
 void gemv_hyper(int64_t epi, Opt x, Opt u, Opt norm_w, double eps, Tensor w, Opt y, double cap, Opt streams, Opt bias, Opt mix,
                 Opt write, Opt read, Opt un) {
@@ -341,7 +342,7 @@ void gemv_hyper(int64_t epi, Opt x, Opt u, Opt norm_w, double eps, Tensor w, Opt
   const Tensor& in = x.has_value() ? *x : *u;
   TORCH_CHECK(in.is_cuda() && in.dim() == 2 && in.size(1) == w.size(1) && in.stride(1) == 1, "gemv_hyper: input [M, K]");
   const int64_t M = in.size(0), N = w.size(0), K = w.size(1);
-  TORCH_CHECK(M >= 1 && M <= 16 && N >= 1 && K >= 8 && K % 8 == 0, "gemv_hyper: 1..16 rows, K a multiple of 8");
+  TORCH_CHECK(M >= 1 && M <= 4 && N >= 1 && K >= 8 && K % 8 == 0, "gemv_hyper: 1..4 rows, K a multiple of 8");
   check_align(in, "input");
   check_align(w, "w");
   p.M = (int)M;
@@ -359,7 +360,7 @@ void gemv_hyper(int64_t epi, Opt x, Opt u, Opt norm_w, double eps, Tensor w, Opt
     p.u = f32_ptr(*u, M * K, "u");
     p.norm_w = f32_ptr(*norm_w, K, "norm_w");
     check_align(*norm_w, "norm_w");
-    TORCH_CHECK(M * K <= 32768, "gemv_hyper: normalised rows must fit 64 KB of LDS");
+    TORCH_CHECK(M * K <= 24576, "gemv_hyper: normalised rows must fit 48 KB of LDS");
   }
   if (epi == 3) {
     TORCH_CHECK(x.has_value() && streams.has_value() && mix.has_value() && write.has_value() && read.has_value() && un.has_value(),
@@ -380,7 +381,7 @@ void gemv_hyper(int64_t epi, Opt x, Opt u, Opt norm_w, double eps, Tensor w, Opt
     p.y = y->data_ptr();
     p.ldy = y->stride(0);
   }
-  check_rc(nxd::gemv_hyper_launch((int)epi, u.has_value(), p, cur_stream()), "gemv_hyper");
+  check_rc(nxd::gemv_hyper_launch((int)epi, p, cur_stream()), "gemv_hyper");
 }
 
 }  // namespace

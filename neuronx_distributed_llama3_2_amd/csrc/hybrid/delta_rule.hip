@@ -39,6 +39,21 @@ __device__ __forceinline__ float conv_silu(const DeltaParams& p, const T* proj, 
   return siluf_(a);
 }
 
+// the same with every load of up to 4 taps issued at once
+template <typename T>
+__device__ __forceinline__ float conv_silu4(const DeltaParams& p, const T* row, const T* ring, int64_t ps, int c) {
+  float a = p.conv[(int64_t)(p.taps - 1) * p.C + c] * ld(row + c);
+#pragma unroll
+  for (int back = 1; back < 4; ++back) {
+    const int64_t q = ps - back;
+    const bool in = back < p.taps && q >= 0;
+    const int e = in ? (int)(q % p.taps) : 0, j = in ? p.taps - 1 - back : 0;
+    const float x = ld(ring + (int64_t)e * p.C + c), w = p.conv[(int64_t)j * p.C + c];
+    a += in ? x * w : 0.f;
+  }
+  return siluf_(a);
+}
+
 // the same for TT consecutive tokens t0 .. of sequence b and N neighbouring channels c ..: every input is
 // read once (up to 4 taps; more fall back to the single-token form)
 template <typename T, int TT, int N>
@@ -289,7 +304,7 @@ template <typename T, int NI, int NTH>
 __global__ void __launch_bounds__(NTH) delta_decode_kernel(DeltaParams p) {
   constexpr int DP = NI * 32, COLS = NTH / 8;
   __shared__ __attribute__((aligned(16))) float qs[DP], ks[DP];
-  __shared__ float vs[256], os[256], red[16];
+  __shared__ float vs[256], os[256], red[16], red2[16], red3[16];
   const int tid = threadIdx.x, l = tid & 7, col = tid >> 3;
   const int h = blockIdx.x, b = blockIdx.y;
   const int H = p.H, G = p.G, D = p.D, V = p.V, rep = H / G, g = h / rep, C = p.C;
@@ -313,15 +328,22 @@ __global__ void __launch_bounds__(NTH) delta_decode_kernel(DeltaParams p) {
     float x = 0.f;
     if (part == 2 || d < D) {
       const int c = part == 0 ? g * D + d : (part == 1 ? (G + g) * D + d : 2 * G * D + h * V + d);
-      x = conv_silu<T>(p, proj, ring, b, 0, ps, c);
+      x = p.taps <= 4 ? conv_silu4<T>(p, proj + (int64_t)b * p.ldp, ring, ps, c) : conv_silu<T>(p, proj, ring, b, 0, ps, c);
       if (part == 2 || h % rep == 0) entry[c] = proj[(int64_t)b * p.ldp + c];
     }
     if (part == 0) { qs[d] = x; sq += x * x; }
     else if (part == 1) { ks[d] = x; sk += x * x; }
     else vs[d] = x;
   }
-  const float rq = p.qscale / sqrtf(block_sum(sq, red) + 1e-6f);
-  const float rk = 1.f / sqrtf(block_sum(sk, red) + 1e-6f);
+  const int lane = tid & 63, wid = tid >> 6;
+  sq = sum64(sq);
+  sk = sum64(sk);
+  if (lane == 0) red[wid] = sq, red2[wid] = sk;
+  __syncthreads();
+  sq = sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < NTH / 64; ++i) sq += red[i], sk += red2[i];
+  const float rq = p.qscale / sqrtf(sq + 1e-6f), rk = 1.f / sqrtf(sk + 1e-6f);
   const T* gates = proj + (int64_t)b * p.ldp + C + H * V;
   const float beta = sigmoidf_(ld(gates + h));
   const float gt = expf(-expf(p.a_log[h]) * softplusf_(ld(gates + H + h) + p.dt_bias[h]));
@@ -331,6 +353,7 @@ __global__ void __launch_bounds__(NTH) delta_decode_kernel(DeltaParams p) {
     k[i] = ld4(&ks[i * 32 + l * 4]) * rk;
     q[i] = ld4(&qs[i * 32 + l * 4]) * rq;
   }
+  float so = 0.f;
   for (int v = col; v < V; v += COLS) {
     float* sp = state + (int64_t)v * DP;
     if (v != col) {
@@ -358,12 +381,18 @@ __global__ void __launch_bounds__(NTH) delta_decode_kernel(DeltaParams p) {
       st4(sp + i * 32 + l * 4, S[i]);
     }
     out = sum8(out);
-    if (l == 0) os[v] = out;
+    if (l == 0) {
+      os[v] = out;
+      so += out * out;
+    }
   }
+  so = sum64(so);   // (l == 0 lanes hold their columns' squares)
+  if (lane == 0) red3[wid] = so;
   __syncthreads();
   float ss = 0.f;
-  for (int v = tid; v < V; v += NTH) ss += os[v] * os[v];
-  const float r = 1.f / sqrtf(block_sum(ss, red) / (float)V + p.eps);
+#pragma unroll
+  for (int i = 0; i < NTH / 64; ++i) ss += red3[i];
+  const float r = 1.f / sqrtf(ss / (float)V + p.eps);
   T* y = static_cast<T*>(p.y) + (int64_t)b * p.ldy + h * V;
   const T* gate = proj + (int64_t)b * p.ldp + C + h * V;
   for (int v = tid; v < V; v += NTH) st(y + v, os[v] * r * p.norm_w[v] * siluf_(ld(gate + v)));

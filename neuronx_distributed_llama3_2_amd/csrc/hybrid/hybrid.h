@@ -65,6 +65,25 @@ __device__ __forceinline__ float sum64(float x) {
   auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(x), __float_as_uint(x), false, false);
   return __uint_as_float(b[0]) + __uint_as_float(b[1]);
 }
+template <int CTRL>
+__device__ __forceinline__ float dpp_max(float x) {
+  return fmaxf(x, __uint_as_float(__builtin_amdgcn_update_dpp(0, __float_as_uint(x), CTRL, 0xf, 0xf, true)));
+}
+__device__ __forceinline__ float max64(float x) {
+  x = dpp_max<0x140>(dpp_max<0x141>(dpp_max<0x4E>(dpp_max<0xB1>(x))));
+  auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+  x = fmaxf(__uint_as_float(a[0]), __uint_as_float(a[1]));
+  auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+  return fmaxf(__uint_as_float(b[0]), __uint_as_float(b[1]));
+}
+template <int N>
+__device__ __forceinline__ float sum_lanes(float x) {   // each aligned group of N = 4, 8 or 16 lanes
+  x = dpp_add<0xB1>(x);
+  x = dpp_add<0x4E>(x);
+  if (N >= 8) x = dpp_add<0x141>(x);
+  if (N >= 16) x = dpp_add<0x140>(x);
+  return x;
+}
 __device__ __forceinline__ float sum8(float x) {   // each aligned group of 8 lanes
   x = dpp_add<0xB1>(x);
   x = dpp_add<0x4E>(x);

@@ -1,10 +1,10 @@
 // One new token per sequence: q / k preparation, cache write and attention in one launch.
 //
-// A workgroup takes 256 of the visible keys of one (sequence, head), 64 a wave: scores with a key a lane,
-// then value columns four a lane.  Every workgroup prepares the head's query itself; the one that owns
-// the new key prepares key and value too (the group's first head also stores them in the cache), so
-// nothing waits for another launch.  With more than 256 visible keys the partial sums go to `part` and
-// the last workgroup of the head to arrive (a ticket in `tickets`, left at zero) merges them in order.
+// A workgroup takes some of the visible keys of one (sequence, head): scores with a key a lane, then value
+// columns four a lane.  Every workgroup prepares the head's query itself; the one that owns the new key
+// prepares key and value too (the group's first head also stores them in the cache), so nothing waits for
+// another launch.  With several workgroups a head the partial sums go to `part` and the last one to arrive
+// (a ticket in `tickets`, left at zero) merges them in order.
 #include "window_attn.h"
 
 namespace nxd {
@@ -49,31 +49,66 @@ __device__ __forceinline__ void prepare_head(const WindowAttnParams& p, const T*
   }
 }
 
-__device__ __forceinline__ float dot_row(const float* k, const float* q, int D) {
-  float s = 0.f;
-  for (int d = 0; d < D; ++d) s += k[d] * q[d];
-  return s;
-}
-__device__ __forceinline__ float dot_row8(const uint16_t* k, const float* q, int D) {   // D % 8 == 0, aligned
-  float s = 0.f, s2 = 0.f;
-#pragma unroll 4
-  for (int d = 0; d < D; d += 8) {
-    float f[8];
-    unpack8(*reinterpret_cast<const u32x4_t*>(k + d), f);
-    const f32x4_t a = ld4(q + d), b = ld4(q + d + 4);
+// A workgroup's sums over its keys (thread = value column): merged with the head's other workgroups if
+// there are any, combined over the maps and stored.
+template <typename T, int MAPS>
+__device__ __forceinline__ void finish(const WindowAttnParams& p, int b, int h, int sp, float (&m)[MAPS], float (&l)[MAPS],
+                                       float (&a)[MAPS], float* red, int* arrival) {
+  const int tid = threadIdx.x, V = p.V;
+  if (p.splits > 1) {
+    const int64_t head = (int64_t)b * p.H + h, stride = MAPS * (V + 2);
+    float* part = p.part + (head * p.splits + sp) * stride;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      s += f[i] * a[i];
-      s2 += f[4 + i] * b[i];
+    for (int c = 0; c < MAPS; ++c) {
+      if (tid < V) __hip_atomic_store(part + c * (V + 2) + 2 + tid, a[c], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      if (tid == 0) {
+        __hip_atomic_store(part + c * (V + 2), m[c], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        __hip_atomic_store(part + c * (V + 2) + 1, l[c], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      }
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // every wave's stores have left before the ticket
+    __syncthreads();
+    if (tid == 0) *arrival = __hip_atomic_fetch_add(p.tickets + head, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    __syncthreads();
+    if (*arrival != p.splits - 1) return;
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup");
+    if (tid == 0) __hip_atomic_store(p.tickets + head, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+#pragma unroll
+    for (int c = 0; c < MAPS; ++c) m[c] = -INFINITY, l[c] = a[c] = 0.f;
+    for (int s0 = 0; s0 < p.splits; s0 += 8) {   // eight splits' partial sums per round trip
+      float ms[MAPS][8], lsum[MAPS][8], as[MAPS][8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i)
+#pragma unroll
+        for (int c = 0; c < MAPS; ++c) {
+          const float* o = p.part + (head * p.splits + min(s0 + i, p.splits - 1)) * stride + c * (V + 2);
+          ms[c][i] = __hip_atomic_load(o, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+          lsum[c][i] = __hip_atomic_load(o + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+          as[c][i] = __hip_atomic_load(o + 2 + min(tid, V - 1), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        }
+#pragma unroll
+      for (int i = 0; i < 8; ++i)
+#pragma unroll
+        for (int c = 0; c < MAPS; ++c) {
+          if (s0 + i >= p.splits || ms[c][i] == -INFINITY) continue;   // (no split, or one past the visible keys)
+          const float m2 = fmaxf(m[c], ms[c][i]), f = m[c] == -INFINITY ? 0.f : expf(m[c] - m2), fs = expf(ms[c][i] - m2);
+          l[c] = l[c] * f + lsum[c][i] * fs;
+          a[c] = a[c] * f + as[c][i] * fs;
+          m[c] = m2;
+        }
     }
   }
-  return s + s2;
+  float o = a[0] / l[0];
+  if constexpr (MAPS == 2) {
+    o -= p.lam * (a[1] / l[1]);
+    o *= p.out_scale / sqrtf(block_sum(tid < V ? o * o : 0.f, red) / (float)V + p.out_eps);
+  }
+  if (tid < V) st(static_cast<T*>(p.y) + (int64_t)b * p.ldy + (int64_t)h * V + tid, o);
 }
-__device__ __forceinline__ float dot_row8(const float* k, const float* q, int D) { return dot_row(k, q, D); }
 
-// VEC: head sizes are multiples of 8 (16-byte key pieces, 4-column value pieces)
-template <typename T, int MAPS, bool VEC>
-__global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
+// ---- any head sizes: 256 keys a workgroup, 64 a wave
+template <typename T, int MAPS>
+__global__ void __launch_bounds__(256) attn_decode_any_kernel(WindowAttnParams p) {
   __shared__ __attribute__((aligned(16))) float q[MAPS][256], kn[MAPS][256], vn[256];
   __shared__ __attribute__((aligned(16))) float pw[4][MAPS][64], acc[4][MAPS][256];
   __shared__ float mw[4][MAPS], lw[4][MAPS], red[16];
@@ -89,6 +124,8 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
   const T* row = static_cast<const T*>(p.buf) + (int64_t)b * p.ldb;
   const T* kc = static_cast<const T*>(p.kc) + ((int64_t)slot * p.G + g) * MAPS * p.cap * D;
   const T* vc = static_cast<const T*>(p.vc) + ((int64_t)slot * p.G + g) * p.cap * V;
+  const int e0 = (int)(j0 % p.cap);                     // ring entry of key 0; key i is e0 + i, wrapped once
+  auto entry = [&](int i) { return e0 + i >= p.cap ? e0 + i - p.cap : e0 + i; };
   const int first = sp * 256, last = min(n, first + 256) - 1;
   const bool owner = first < n && last == n - 1;        // this workgroup has the new key
 
@@ -129,61 +166,40 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
   for (int i = lane; i < MAPS * V; i += 64) acc[w][i / V][i % V] = 0.f;
   if (cnt > 0) {
     const int key = k0 + min(lane, cnt - 1);
-    const int e = (int)((j0 + key) % p.cap);
+    const int e = entry(key);
+    // the new key's entry may hold an old key or the new one by now: its score comes from LDS
+    const bool has_new = k0 + cnt == n;
 #pragma unroll
     for (int c = 0; c < MAPS; ++c) {
       float s;
-      if (key == n - 1) s = dot_row(kn[c], q[c], D);
-      else if (VEC) s = dot_row8(kc + ((int64_t)c * p.cap + e) * D, q[c], D);
-      else {
-        const T* kr = kc + ((int64_t)c * p.cap + e) * D;
-        s = 0.f;
-        for (int d = 0; d < D; ++d) s += ld(kr + d) * q[c][d];
+      const T* kr = kc + ((int64_t)c * p.cap + e) * D;
+      s = 0.f;
+      for (int d = 0; d < D; ++d) s += ld(kr + d) * q[c][d];
+      if (has_new) {
+        float t = 0.f;
+        for (int d = lane; d < D; d += 64) t += kn[c][d] * q[c][d];
+        t = sum64(t);
+        if (key == n - 1) s = t;
       }
       s *= p.scale;
       if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
       if (lane >= cnt) s = -INFINITY;
-      mx[c] = wave_max(s);
+      mx[c] = max64(s);
       const float x = lane < cnt ? expf(s - mx[c]) : 0.f;
       ls[c] = sum64(x);
       pw[w][c][lane] = x;
     }
     __builtin_amdgcn_wave_barrier();
-    if (VEC) {
-      const int lpr = V <= 32 ? 8 : (V <= 64 ? 16 : (V <= 128 ? 32 : 64)), kpp = 64 / lpr;   // lanes a row, keys a pass
-      const int col = (lane % lpr) * 4, ks = lane / lpr;
-      f32x4_t a[MAPS];
+    for (int d = lane; d < V; d += 64) {
+      float a[MAPS] = {};
+      for (int j = 0; j < cnt; ++j) {
+        const int key2 = k0 + j;
+        const float x = key2 == n - 1 ? vn[d] : ld(vc + (int64_t)entry(key2) * V + d);
 #pragma unroll
-      for (int c = 0; c < MAPS; ++c) a[c] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-      if (col < V) {
-#pragma unroll 8
-        for (int j = 0; j < cnt; j += kpp) {
-          const int i = min(j + ks, cnt - 1), key2 = k0 + i;
-          const bool in = j + ks < cnt;
-          const f32x4_t x = key2 == n - 1 ? ld4(vn + col) : ld4(vc + (int64_t)((j0 + key2) % p.cap) * V + col);
-#pragma unroll
-          for (int c = 0; c < MAPS; ++c) a[c] += x * (in ? pw[w][c][i] : 0.f);
-        }
+        for (int c = 0; c < MAPS; ++c) a[c] += pw[w][c][j] * x;
       }
 #pragma unroll
-      for (int c = 0; c < MAPS; ++c) {
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-          for (int o = lpr; o < 64; o <<= 1) a[c][i] += __shfl_xor(a[c][i], o, 64);
-        if (ks == 0 && col < V) st4(&acc[w][c][col], a[c]);
-      }
-    } else {
-      for (int d = lane; d < V; d += 64) {
-        float a[MAPS] = {};
-        for (int j = 0; j < cnt; ++j) {
-          const int key2 = k0 + j;
-          const float x = key2 == n - 1 ? vn[d] : ld(vc + (int64_t)((j0 + key2) % p.cap) * V + d);
-#pragma unroll
-          for (int c = 0; c < MAPS; ++c) a[c] += pw[w][c][j] * x;
-        }
-#pragma unroll
-        for (int c = 0; c < MAPS; ++c) acc[w][c][d] = a[c];
-      }
+      for (int c = 0; c < MAPS; ++c) acc[w][c][d] = a[c];
     }
   }
   if (lane == 0) {
@@ -205,58 +221,218 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
       if (tid < V) a[c] += acc[i][c][tid] * f;
     }
   }
-  if (p.splits > 1) {
-    const int64_t head = (int64_t)b * p.H + h, stride = MAPS * (V + 2);
-    float* part = p.part + (head * p.splits + sp) * stride;
+  finish<T, MAPS>(p, b, h, sp, m, l, a, red, &arrival);
+}
+
+// ---- head sizes that are multiples of 8, D <= 128: 64 keys a tile.  Keys and values of a tile are on
+// their way before they are needed (the first tile's before the query is even prepared).  Neighbouring
+// lanes read neighbouring pieces of a row: a key's score is a sum over LR lanes, a value row is spread
+// over 8 to 64.  The keys of a map are shared by 4 / MAPS waves; every wave then has all 64 weights and
+// sums 16 keys.
+template <typename T>
+struct Raw;
+template <>
+struct Raw<uint16_t> {
+  typedef u32x2_t four;
+  struct eight {
+    u32x4_t v;
+  };
+};
+template <>
+struct Raw<float> {
+  typedef f32x4_t four;
+  struct eight {
+    f32x4_t a, b;
+  };
+};
+__device__ __forceinline__ f32x4_t widen(const u32x2_t& v) {
+  return f32x4_t{__uint_as_float(v[0] << 16), __uint_as_float(v[0] & 0xffff0000u), __uint_as_float(v[1] << 16),
+                 __uint_as_float(v[1] & 0xffff0000u)};
+}
+__device__ __forceinline__ f32x4_t widen(const f32x4_t& v) { return v; }
+__device__ __forceinline__ float dot8(const Raw<uint16_t>::eight& k, const float (&q)[8]) {
+  float f[8], s = 0.f;
+  unpack8(k.v, f);
 #pragma unroll
-    for (int c = 0; c < MAPS; ++c) {
-      if (tid < V) __hip_atomic_store(part + c * (V + 2) + 2 + tid, a[c], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-      if (tid == 0) {
-        __hip_atomic_store(part + c * (V + 2), m[c], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-        __hip_atomic_store(part + c * (V + 2) + 1, l[c], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-      }
+  for (int i = 0; i < 8; ++i) s += f[i] * q[i];
+  return s;
+}
+__device__ __forceinline__ float dot8(const Raw<float>::eight& k, const float (&q)[8]) {
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) s += k.a[i] * q[i] + k.b[i] * q[4 + i];
+  return s;
+}
+
+// LR lanes of 8 elements cover D
+template <typename T, int MAPS, int LR>
+__global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
+  constexpr int PARTS = 4 / MAPS, RPL = 64 / LR, NK = (64 / PARTS) / RPL;   // waves a map, keys a load, loads a wave
+  static_assert(NK >= 1, "whole loads");
+  typedef typename Raw<T>::four raw_t;
+  __shared__ __attribute__((aligned(16))) float q[MAPS][128], kn[MAPS][128], vn[256];
+  __shared__ __attribute__((aligned(16))) float sc[2][MAPS][64], pw[4][MAPS][64], acc[4][MAPS][256];
+  __shared__ float red[16];
+  __shared__ int arrival;
+  const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int sp = blockIdx.x, h = blockIdx.y, b = blockIdx.z, rep = p.H / p.G, g = h / rep, D = p.D, V = p.V;
+  const int slot = slot_of(p.slots, b, p.nslots);
+  const int64_t ps = pos_of(p.pos, p.pos_stride, b);
+  const int64_t pt = ps < p.max_pos ? ps : p.max_pos - 1;
+  int64_t j0 = p.window > 0 && ps - p.window + 1 > 0 ? ps - p.window + 1 : 0;
+  if (ps - j0 >= p.cap) j0 = ps - p.cap + 1;            // the ring holds no more (a position beyond the cache)
+  const int n = (int)(ps - j0 + 1);                     // visible keys, the new one last
+  const int e0 = (int)((uint32_t)j0 % (uint32_t)p.cap); // (positions are below 2^31)
+  auto entry = [&](int i) { return e0 + i >= p.cap ? e0 + i - p.cap : e0 + i; };
+  const T* row = static_cast<const T*>(p.buf) + (int64_t)b * p.ldb;
+  T* kc = static_cast<T*>(p.kc) + ((int64_t)slot * p.G + g) * MAPS * p.cap * D;
+  T* vc = static_cast<T*>(p.vc) + ((int64_t)slot * p.G + g) * p.cap * V;
+  const int first = sp * p.tiles * 64, end = min(n, first + p.tiles * 64);
+  const bool owner = first < n && end == n;             // this workgroup has the new key
+
+  // this wave's map and keys of the scores, and its columns of the sums
+  const int c = w % MAPS, part = w / MAPS, dl = (lane % LR) * 8, kl = lane / LR;
+  const bool dok = dl < D;
+  const int lpr = V <= 32 ? 8 : (V <= 64 ? 16 : (V <= 128 ? 32 : 64)), kpp = 64 / lpr;   // lanes a value row, rows a load
+  const int col = min((lane % lpr) * 4, V - 4), ks = lane / lpr;
+  typename Raw<T>::eight kr[NK];
+  raw_t vr[16];
+  auto fetch_k = [&](int k0) {   // (keys past the end re-read the last)
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int e = entry(min(k0 + part * (64 / PARTS) + i * RPL + kl, n - 1));
+      kr[i] = *reinterpret_cast<const typename Raw<T>::eight*>(kc + ((int64_t)c * p.cap + e) * D + (dok ? dl : 0));
     }
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // every wave's stores have left before the ticket
-    __syncthreads();
-    if (tid == 0) arrival = __hip_atomic_fetch_add(p.tickets + head, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    __syncthreads();
-    if (arrival != p.splits - 1) return;
-    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup");
-    if (tid == 0) __hip_atomic_store(p.tickets + head, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  };
+  auto fetch_v = [&](int k0) {
 #pragma unroll
-    for (int c = 0; c < MAPS; ++c) {
-      m[c] = -INFINITY;
-      l[c] = a[c] = 0.f;
-      for (int s = 0; s < p.splits; ++s) {
-        const float* o = p.part + (head * p.splits + s) * stride + c * (V + 2);
-        const float ms = __hip_atomic_load(o, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-        if (ms == -INFINITY) continue;   // a split past the visible keys
-        const float lsum = __hip_atomic_load(o + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-        const float as = tid < V ? __hip_atomic_load(o + 2 + tid, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) : 0.f;
-        const float m2 = fmaxf(m[c], ms), f = m[c] == -INFINITY ? 0.f : expf(m[c] - m2), fs = expf(ms - m2);
-        l[c] = l[c] * f + lsum * fs;
-        a[c] = a[c] * f + as * fs;
-        m[c] = m2;
+    for (int i = 0; i < 16; ++i)
+      if (i * kpp < 16) vr[i] = *reinterpret_cast<const raw_t*>(vc + (int64_t)entry(min(k0 + 16 * w + i * kpp + ks, n - 1)) * V + col);
+  };
+  if (first < n) {
+    fetch_k(first);
+    fetch_v(first);
+  }
+
+  if (first < n) {
+    const int64_t qk0 = (int64_t)p.H * MAPS * D;
+    for (int job = w; job < (owner ? 2 * MAPS + 1 : MAPS); job += 4) {
+      if (job < MAPS) {
+        const int64_t o = ((int64_t)h * MAPS + job) * D;
+        prepare_head<T>(p, row + o, p.bias ? p.bias + o : nullptr, p.qn_w, pt, q[job]);
+      } else if (job < 2 * MAPS) {
+        const int64_t o = qk0 + ((int64_t)g * MAPS + job - MAPS) * D;
+        prepare_head<T>(p, row + o, p.bias ? p.bias + o : nullptr, p.kn_w, pt, kn[job - MAPS]);
+      } else {
+        const int64_t o = qk0 + (int64_t)p.G * MAPS * D + (int64_t)g * V;
+        for (int d = lane; d < V; d += 64) {
+          T t;
+          st(&t, ld(row + o + d) + (p.bias ? p.bias[o + d] : 0.f));
+          vn[d] = ld(&t);
+        }
       }
     }
   }
-  float o = a[0] / l[0];
-  if constexpr (MAPS == 2) {
-    o -= p.lam * (a[1] / l[1]);
-    o *= p.out_scale / sqrtf(block_sum(tid < V ? o * o : 0.f, red) / (float)V + p.out_eps);
+  __syncthreads();
+  if (owner && h % rep == 0) {   // (the values are exact in the activation type)
+    const int e = entry(n - 1);
+    for (int i = tid; i < MAPS * D; i += 256) st(kc + ((int64_t)(i / D) * p.cap + e) * D + i % D, kn[i / D][i % D]);
+    for (int i = tid; i < V; i += 256) st(vc + (int64_t)e * V + i, vn[i]);
   }
-  if (tid < V) st(static_cast<T*>(p.y) + (int64_t)b * p.ldy + (int64_t)h * V + tid, o);
+
+  float mx[MAPS], ls[MAPS];
+  f32x4_t a4[MAPS];
+#pragma unroll
+  for (int i = 0; i < MAPS; ++i) mx[i] = -INFINITY, ls[i] = 0.f, a4[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float q8[8];
+#pragma unroll
+  for (int i = 0; i < 8; ++i) q8[i] = dok ? q[c][dl + i] : 0.f;
+  float snew = 0.f;   // the new key's score
+  if (owner) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) snew += dok ? kn[c][dl + i] * q8[i] : 0.f;
+    snew = sum_lanes<LR>(snew);
+  }
+  int flip = 0;
+  for (int k0 = first; k0 < end; k0 += 64, flip ^= 1) {
+    const int cnt = min(64, end - k0);
+    const bool has_new = k0 + cnt == n;   // its entry may hold an old key or the new one by now: taken from LDS
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int k = part * (64 / PARTS) + i * RPL + kl;
+      float s = sum_lanes<LR>(dot8(kr[i], q8));
+      if (has_new && k == cnt - 1) s = snew;
+      if (lane % LR == 0) sc[flip][c][k] = s;
+    }
+    if (k0 + 64 < end) fetch_k(k0 + 64);
+    __syncthreads();   // (two score buffers: the next tile's scores do not wait for this one's readers)
+#pragma unroll
+    for (int m = 0; m < MAPS; ++m) {
+      float s = sc[flip][m][lane] * p.scale;
+      if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
+      if (lane >= cnt) s = -INFINITY;
+      const float m2 = fmaxf(mx[m], max64(s));
+      const float f = mx[m] == -INFINITY ? 0.f : expf(mx[m] - m2), x = lane < cnt ? expf(s - m2) : 0.f;
+      mx[m] = m2;
+      ls[m] = ls[m] * f + sum64(x);
+      a4[m] *= f;
+      pw[w][m][lane] = x;
+    }
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      if (i * kpp < 16) {
+        const int k = 16 * w + i * kpp + ks;
+        f32x4_t x = widen(vr[i]);
+        if (has_new && k >= cnt - 1) x = ld4(vn + col);   // (past the end: any finite value, its weight is zero)
+#pragma unroll
+        for (int m = 0; m < MAPS; ++m) a4[m] += x * pw[w][m][k];
+      }
+    }
+    if (k0 + 64 < end) fetch_v(k0 + 64);
+  }
+#pragma unroll
+  for (int m = 0; m < MAPS; ++m) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      for (int o = lpr; o < 64; o <<= 1) a4[m][i] += __shfl_xor(a4[m][i], o, 64);
+    if (ks == 0 && (lane % lpr) * 4 < V) st4(&acc[w][m][col], a4[m]);
+  }
+  __syncthreads();
+  float a[MAPS];
+#pragma unroll
+  for (int m = 0; m < MAPS; ++m) a[m] = tid < V ? acc[0][m][tid] + acc[1][m][tid] + acc[2][m][tid] + acc[3][m][tid] : 0.f;
+  finish<T, MAPS>(p, b, h, sp, mx, ls, a, red, &arrival);
 }
 
 template <typename T, int MAPS>
 static int run_decode(const WindowAttnParams& p, hipStream_t s) {
   const dim3 grid((unsigned)p.splits, (unsigned)p.H, (unsigned)p.B);
-  if (p.D % 8 == 0 && p.V % 8 == 0) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, true>), grid, dim3(256), 0, s, p);
-  else hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, false>), grid, dim3(256), 0, s, p);
+  if (p.tiles > 0 && p.D <= 32) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 4>), grid, dim3(256), 0, s, p);
+  else if (p.tiles > 0 && p.D <= 64) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 8>), grid, dim3(256), 0, s, p);
+  else if (p.tiles > 0) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 16>), grid, dim3(256), 0, s, p);
+  else hipLaunchKernelGGL((attn_decode_any_kernel<T, MAPS>), grid, dim3(256), 0, s, p);
   return hipGetLastError() == hipSuccess ? 0 : 1;
 }
 
 }  // namespace hybrid
+
+// workgroups per head and 64-key tiles each (0: the any-size kernel) for at most `seen` visible keys
+void attn_decode_plan(WindowAttnParams& p, int64_t seen) {
+  if (p.D % 8 == 0 && p.V % 8 == 0 && p.D <= 128) {
+    // about 512 workgroups, but not more than 8 a head before each has 4 tiles: the merge has its price
+    // (16 heads, 1,024 visible keys, us: 1 sequence 8 / 16 workgroups a head 14.1 / 15.4; 8 sequences 1 / 2 /
+    // 4 / 8 of them 46 / 29 / 20 / 27)
+    const int64_t tiles = (seen + 63) / 64, heads = (int64_t)p.B * p.H, most = tiles / 4 > 8 ? tiles / 4 : (tiles < 8 ? tiles : 8);
+    int64_t splits = 512 / heads;
+    splits = splits < 1 ? 1 : (splits > most ? most : splits);
+    p.tiles = (int)((tiles + splits - 1) / splits);
+    p.splits = (int)((tiles + p.tiles - 1) / p.tiles);
+  } else {
+    p.tiles = 0;
+    p.splits = (int)((seen + 255) / 256);
+  }
+}
 
 int attn_decode_launch(bool f32, const WindowAttnParams& p, hipStream_t s) {
   if (p.maps == 2) return f32 ? hybrid::run_decode<float, 2>(p, s) : hybrid::run_decode<uint16_t, 2>(p, s);

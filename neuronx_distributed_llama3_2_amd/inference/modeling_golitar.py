@@ -4,7 +4,7 @@ attention mixers and squared-ReLU feed-forwards.
 The residual is [rows, streams, width] in fp32; between two sublayers one kernel (ops.hyper_step)
 writes the last sublayer's output into the streams and reads and normalises the next one's input, so a
 layer of the forward is: hyper_step, projection GEMM, mixer kernels, output GEMM (and the same around the
-feed-forward).  A decode step of up to 16 sequences folds the norms into the input projections and the
+feed-forward).  A decode step of up to 4 sequences folds the norms into the input projections and the
 stream updates into the output projections (_forward_decode_fused_streams).  The step function, cache set-up and decode-graph hooks are those of every
 model of the framework (model_base.DecoderInferenceMixin); the cache is a LayerCache.
 """

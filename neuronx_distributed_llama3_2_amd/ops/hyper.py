@@ -68,9 +68,8 @@ def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
     return x.copy_(cap * torch.tanh(x / cap))
 
 
-# most rows the fused decode projections take, and the LDS limit on normalised rows (rows x columns)
-FUSED_ROWS = 16
-FUSED_NORM_ELEMENTS = 32768
+FUSED_ROWS = 4               # most rows the fused decode projections take
+FUSED_NORM_ELEMENTS = 24576  # most elements of the rows they normalise (48 KB of LDS)
 
 _EPI = {"store": 0, "relu2": 1, "f32": 2, "streams": 3}
 

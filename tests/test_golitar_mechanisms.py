@@ -332,7 +332,7 @@ def test_first_tokens_see_only_what_is_there(where):
 
 
 @pytest.mark.gpu
-@pytest.mark.parametrize("visible", [255, 256, 257, 600])
+@pytest.mark.parametrize("visible", [63, 64, 65, 255, 257, 600, 2200])
 def test_split_decode(visible):
     """Decoding over more than 256 visible keys (several workgroups per head and a merge), repeated: the
     arrival counters are left at zero; a key that outweighs all others is far away."""
@@ -354,20 +354,19 @@ def test_split_decode(visible):
 
 # ------------------------------------------------------------------ fused decode projections
 @pytest.mark.gpu
-@pytest.mark.parametrize("M", [1, 2, 3, 8, 16])
-@pytest.mark.parametrize("N,K", [(80, 72), (33, 8), (200, 2048), (1000, 1000), (48, 4096)])
+@pytest.mark.parametrize("M", [1, 2, 3, 4])
+@pytest.mark.parametrize("N,K", [(80, 72), (33, 8), (200, 2048), (1000, 1000), (48, 4096), (24, 6144)])
 def test_decode_projections(M, N, K):
     d, bf = "cuda", torch.bfloat16
     w = (rnd(N, K) * K ** -0.5).to(bf)
     x, u, nw = rnd(M, K, seed=1).to(bf), rnd(M, K, seed=2, std=3.0).float(), rnd(K, seed=3, std=0.2).float()
     wd, wo = w.to(d), w.double()
     assert rel_err(ops.decode_linear(wd, x.to(d)), x.double() @ wo.T) < 5e-3
-    if M * K <= 32768:
-        h = O.zero_centred_norm(u.double(), nw.double(), 1e-5).to(bf).double() @ wo.T
-        norm = (None, u.to(d), nw.to(d), 1e-5)
-        assert rel_err(ops.decode_linear(wd, *norm), h) < 8e-3
-        assert rel_err(ops.decode_linear(wd, *norm, "relu2"), torch.clamp(h, min=0) ** 2) < 1.6e-2
-        assert rel_err(ops.decode_linear(wd, *norm, "f32", 2.5), 2.5 * torch.tanh(h / 2.5)) < 5e-3
+    h = O.zero_centred_norm(u.double(), nw.double(), 1e-5).to(bf).double() @ wo.T
+    norm = (None, u.to(d), nw.to(d), 1e-5)
+    assert rel_err(ops.decode_linear(wd, *norm), h) < 8e-3
+    assert rel_err(ops.decode_linear(wd, *norm, "relu2"), torch.clamp(h, min=0) ** 2) < 1.6e-2
+    assert rel_err(ops.decode_linear(wd, *norm, "f32", 2.5), 2.5 * torch.tanh(h / 2.5)) < 5e-3
     for S in (1, 3, 8):
         st, mix, wr, rd, b = rnd(M, S, N), rnd(S, S, seed=4), rnd(S, seed=5), rnd(S, seed=6), rnd(N, seed=7)
         f = lambda t: t.float().to(d)  # noqa: E731
