@@ -158,6 +158,29 @@ __global__ void __launch_bounds__(256) delta_prep_kernel(DeltaParams p) {
     // fragment order of the chunk (delta_chunk.hip): q as rows of tokens, k as rows of columns
     const int tc = t0 & 63, tb = tc >> 4;
     const int64_t cell = (((int64_t)b * p.nch + t0 / 64) * G + g) * 64 * DP;
+    if constexpr (N == 2) {
+      if (isq) {   // neighbouring lanes swap halves: four channels of four tokens each, 16 bytes a token
+        const bool odd = lane & 1;
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+          const int d = (2 * lane + 128 * j) & ~3;
+          float* out = p.qn + cell + ((((int64_t)tb * NB + d / 16) * 4 + (d & 15) / 4) * 16 + (tc & 15) + (odd ? 4 : 0)) * 4;
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            float mine[2], other[2];
+#pragma unroll
+            for (int k = 0; k < 2; ++k) {
+              const float send = odd ? x[j][k][i] : x[j][k][4 + i];
+              other[k] = __uint_as_float(__builtin_amdgcn_update_dpp(0, __float_as_uint(send), 0xB1, 0xf, 0xf, true));
+              mine[k] = odd ? x[j][k][4 + i] : x[j][k][i];
+            }
+            if (d < DP)
+              st4(out + 4 * i, odd ? f32x4_t{other[0], other[1], mine[0], mine[1]} : f32x4_t{mine[0], mine[1], other[0], other[1]});
+          }
+        }
+        continue;
+      }
+    }
 #pragma unroll
     for (int j = 0; j < NJ; ++j)
 #pragma unroll
@@ -299,6 +322,29 @@ __global__ void __launch_bounds__(256) delta_out_kernel(DeltaParams p) {
   }
 }
 
+// The same for V a multiple of 4: four values a lane, L lanes a head.
+template <typename T, int L>
+__global__ void __launch_bounds__(256) delta_out4_kernel(DeltaParams p) {
+  const int64_t i = (int64_t)blockIdx.x * (256 / L) + threadIdx.x / L;   // (row, head)
+  const int H = p.H, V = p.V, v = (threadIdx.x % L) * 4;
+  const bool in = i < (int64_t)p.B * p.T * H && v < V;
+  const int64_t m = in ? i / H : 0;
+  const int h = in ? (int)(i % H) : 0;
+  const bool live = in && !(p.lens && (int)(m % p.T) >= p.lens[m / p.T]);
+  f32x4_t x = {0.f, 0.f, 0.f, 0.f}, g = x, w = x;
+  if (live) {
+    x = ld4(p.o + i * V + v);
+    g = ld4(static_cast<const T*>(p.proj) + m * p.ldp + p.C + h * V + v);
+    w = ld4(p.norm_w + v);
+  }
+  const float ss = sum_lanes<L>(x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3]);
+  if (!in) return;
+  const float r = 1.f / sqrtf(ss / (float)V + p.eps);
+#pragma unroll
+  for (int j = 0; j < 4; ++j) x[j] *= r * w[j] * siluf_(g[j]);   // padding: zeros
+  st4(static_cast<T*>(p.y) + m * p.ldy + h * V + v, x);
+}
+
 // ---- one new token per sequence: a workgroup of NTH threads per (head, sequence)
 template <typename T, int NI, int NTH>
 __global__ void __launch_bounds__(NTH) delta_decode_kernel(DeltaParams p) {
@@ -431,7 +477,16 @@ static int run_scan(const DeltaParams& p, hipStream_t s) {
 template <typename T>
 static int run_out(const DeltaParams& p, hipStream_t s) {
   const int64_t n = (int64_t)p.B * p.T * p.H;
-  hipLaunchKernelGGL((delta_out_kernel<T>), dim3((unsigned)ceil_div64(n, 4)), dim3(256), 0, s, p);
+  const dim3 block(256);
+#define NXD_OUT4(L) hipLaunchKernelGGL((delta_out4_kernel<T, L>), dim3((unsigned)ceil_div64(n, 256 / L)), block, 0, s, p)
+  if (p.V % 4 || p.C % 4 || p.ldp % 4 || p.ldy % 4)
+    hipLaunchKernelGGL((delta_out_kernel<T>), dim3((unsigned)ceil_div64(n, 4)), block, 0, s, p);
+  else if (p.V <= 16) NXD_OUT4(4);
+  else if (p.V <= 32) NXD_OUT4(8);
+  else if (p.V <= 64) NXD_OUT4(16);
+  else if (p.V <= 128) NXD_OUT4(32);
+  else NXD_OUT4(64);
+#undef NXD_OUT4
   return hipGetLastError() == hipSuccess ? 0 : 1;
 }
 template <typename T>

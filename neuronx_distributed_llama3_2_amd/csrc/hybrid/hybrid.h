@@ -77,11 +77,19 @@ __device__ __forceinline__ float max64(float x) {
   return fmaxf(__uint_as_float(b[0]), __uint_as_float(b[1]));
 }
 template <int N>
-__device__ __forceinline__ float sum_lanes(float x) {   // each aligned group of N = 4, 8 or 16 lanes
+__device__ __forceinline__ float sum_lanes(float x) {   // each aligned group of N = 4, 8, 16, 32 or 64 lanes
   x = dpp_add<0xB1>(x);
   x = dpp_add<0x4E>(x);
   if (N >= 8) x = dpp_add<0x141>(x);
   if (N >= 16) x = dpp_add<0x140>(x);
+  if (N >= 32) {
+    auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+    x = __uint_as_float(a[0]) + __uint_as_float(a[1]);
+  }
+  if (N >= 64) {
+    auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(x), __float_as_uint(x), false, false);
+    x = __uint_as_float(b[0]) + __uint_as_float(b[1]);
+  }
   return x;
 }
 __device__ __forceinline__ float sum8(float x) {   // each aligned group of 8 lanes

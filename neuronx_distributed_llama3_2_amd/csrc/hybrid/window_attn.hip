@@ -77,6 +77,56 @@ __global__ void __launch_bounds__(256) attn_prep_kernel(WindowAttnParams p) {
   }
 }
 
+// The same for head sizes that are multiples of 4: four elements (two pairs) a lane, L lanes a head, so a
+// wave works on 64 / L heads at once.
+template <typename T, int L>
+__global__ void __launch_bounds__(256) attn_prep4_kernel(WindowAttnParams p) {
+  constexpr int HPB = 256 / L;   // heads at once
+  const int64_t m = blockIdx.x;
+  const int b = (int)(m / p.T), t = (int)(m % p.T);
+  const int len = p.lens ? min(p.lens[b], p.T) : p.T;
+  if (t >= len) return;
+  const int64_t ps = pos_of(p.pos, p.pos_stride, b) + t;
+  const int64_t pt = ps < p.max_pos ? ps : p.max_pos - 1;
+  const int slot = slot_of(p.slots, b, p.nslots);
+  const int entry = (int)(ps % p.cap);
+  const bool keep = t >= len - p.cap;   // a prompt longer than the ring: only its last entries
+  T* row = static_cast<T*>(p.buf) + m * p.ldb;
+  const int nq = p.H * p.maps, nk = p.G * p.maps, D = p.D, V = p.V, half = p.rot / 2;
+  const int d = (threadIdx.x % L) * 4;
+  const bool ok = d < D;
+  const float *cs = p.cos_t + pt * half, *sn = p.sin_t + pt * half;
+  float c2[2] = {1.f, 1.f}, s2[2] = {0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+    if (d / 2 + i < half) c2[i] = cs[d / 2 + i], s2[i] = sn[d / 2 + i];
+  const f32x4_t zero = {0.f, 0.f, 0.f, 0.f}, one = {1.f, 1.f, 1.f, 1.f};
+  for (int h0 = 0; h0 < nq + nk; h0 += HPB) {   // (uniform: the reduction needs every lane)
+    const int hd = h0 + threadIdx.x / L;
+    const bool in = ok && hd < nq + nk;
+    T* x = row + hd * D + d;
+    f32x4_t v = in ? ld4(x) : zero;
+    if (in && p.bias) v += ld4(p.bias + hd * D + d);
+    const f32x4_t w = in && p.qn_w ? ld4((hd < nq ? p.qn_w : p.kn_w) + d) : one;
+    const float ss = sum_lanes<L>(v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]);
+    if (!in) continue;
+    if (p.qn_w) v *= w * (1.f / sqrtf(ss / (float)D + p.eps));
+    const f32x4_t o = {v[0] * c2[0] - v[1] * s2[0], v[1] * c2[0] + v[0] * s2[0], v[2] * c2[1] - v[3] * s2[1],
+                       v[3] * c2[1] + v[2] * s2[1]};
+    st4(x, o);
+    if (hd >= nq && keep) st4(static_cast<T*>(p.kc) + (((int64_t)slot * nk + (hd - nq)) * p.cap + entry) * D + d, o);
+  }
+  const int c0 = (nq + nk) * D;
+  for (int i = threadIdx.x * 4; i < p.G * V; i += 1024) {
+    f32x4_t v = ld4(row + c0 + i);
+    if (p.bias) {
+      v += ld4(p.bias + c0 + i);
+      st4(row + c0 + i, v);
+    }
+    if (keep) st4(static_cast<T*>(p.vc) + (((int64_t)slot * p.G + i / V) * p.cap + entry) * V + i % V, v);
+  }
+}
+
 __device__ __forceinline__ float cap_score(float s, float scale, float cap) {
   s *= scale;
   return cap > 0.f ? cap * tanhf(s / cap) : s;
@@ -217,11 +267,22 @@ static int run_row(const WindowAttnParams& p, hipStream_t s) {
 
 }  // namespace hybrid
 
-int attn_prep_launch(bool f32, const WindowAttnParams& p, hipStream_t s) {
-  const dim3 grid((unsigned)(p.B * p.T));
-  if (f32) hipLaunchKernelGGL((hybrid::attn_prep_kernel<float>), grid, dim3(256), 0, s, p);
-  else hipLaunchKernelGGL((hybrid::attn_prep_kernel<uint16_t>), grid, dim3(256), 0, s, p);
+template <typename T>
+static int run_prep(const WindowAttnParams& p, hipStream_t s) {
+  using namespace hybrid;
+  const dim3 grid((unsigned)(p.B * p.T)), block(256);
+  if (p.D % 4 || p.V % 4 || p.ldb % 4 || reinterpret_cast<uintptr_t>(p.buf) % 16)
+    hipLaunchKernelGGL((attn_prep_kernel<T>), grid, block, 0, s, p);
+  else if (p.D <= 16) hipLaunchKernelGGL((attn_prep4_kernel<T, 4>), grid, block, 0, s, p);
+  else if (p.D <= 32) hipLaunchKernelGGL((attn_prep4_kernel<T, 8>), grid, block, 0, s, p);
+  else if (p.D <= 64) hipLaunchKernelGGL((attn_prep4_kernel<T, 16>), grid, block, 0, s, p);
+  else if (p.D <= 128) hipLaunchKernelGGL((attn_prep4_kernel<T, 32>), grid, block, 0, s, p);
+  else hipLaunchKernelGGL((attn_prep4_kernel<T, 64>), grid, block, 0, s, p);
   return hipGetLastError() == hipSuccess ? 0 : 1;
+}
+
+int attn_prep_launch(bool f32, const WindowAttnParams& p, hipStream_t s) {
+  return f32 ? run_prep<float>(p, s) : run_prep<uint16_t>(p, s);
 }
 
 int attn_prompt_d32_launch(const WindowAttnParams&, hipStream_t);
