@@ -299,6 +299,7 @@ void window_attn(Tensor buf, int64_t B, int64_t T, std::vector<int64_t> sizes, d
                  bool from_buf, bool fused) {
   auto p = attn_params(buf, B, T, sizes, pos, lens, slots, kc, vc);
   set_rule(p, scale, softcap, window, lam, out_scale, out_eps, buf, y);
+  TORCH_CHECK(from_buf || T <= p.cap, "window_attn: ", T, " new tokens do not fit a ring of ", p.cap);
   p.from_buf = from_buf ? 1 : 0;
   const bool f32 = buf.scalar_type() == at::kFloat;
   if (fused && !f32 && nxd::attn_prompt_supported(p)) {

@@ -31,7 +31,8 @@ struct WindowAttnParams {
   int64_t ldy;
   int from_buf;           // keys of this step's buffer (prompt from position 0) instead of the cache
   // split decode
-  int splits, tiles;      // workgroups per (sequence, head), 64-key tiles each
+  int share;              // query heads of a workgroup (of one key / value head)
+  int splits, tiles;      // workgroups per (sequence, heads), 64-key tiles each
   float* part;            // [B H, splits, maps (V + 2)] partial sums (splits > 1)
   int* tickets;           // [B H] arrivals, zero between launches (splits > 1)
 };

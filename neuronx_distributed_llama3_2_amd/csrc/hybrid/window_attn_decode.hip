@@ -264,18 +264,20 @@ __device__ __forceinline__ float dot8(const Raw<float>::eight& k, const float (&
   return s;
 }
 
-// LR lanes of 8 elements cover D
-template <typename T, int MAPS, int LR>
+// R query heads of one key / value head share the keys and values a workgroup reads.  LR lanes of 8
+// elements cover D.
+template <typename T, int MAPS, int LR, int R>
 __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
   constexpr int PARTS = 4 / MAPS, RPL = 64 / LR, NK = (64 / PARTS) / RPL;   // waves a map, keys a load, loads a wave
-  static_assert(NK >= 1, "whole loads");
+  constexpr int NJ = R * MAPS, SM = (NJ + 3) / 4;                           // rows of weights, of them a wave
+  static_assert(NK >= 1 && R <= 4, "whole loads, a wave a head at the end");
   typedef typename Raw<T>::four raw_t;
-  __shared__ __attribute__((aligned(16))) float q[MAPS][128], kn[MAPS][128], vn[256];
-  __shared__ __attribute__((aligned(16))) float sc[2][MAPS][64], pw[4][MAPS][64], acc[4][MAPS][256];
-  __shared__ float red[16];
+  __shared__ __attribute__((aligned(16))) float q[NJ][128], kn[MAPS][128], vn[256];
+  __shared__ __attribute__((aligned(16))) float sc[2][NJ][64], pw[NJ][64], acc[4][NJ][256];
+  __shared__ float fs[NJ], msum[NJ], lsum[NJ];
   __shared__ int arrival;
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int sp = blockIdx.x, h = blockIdx.y, b = blockIdx.z, rep = p.H / p.G, g = h / rep, D = p.D, V = p.V;
+  const int sp = blockIdx.x, h0 = blockIdx.y * R, b = blockIdx.z, rep = p.H / p.G, g = h0 / rep, D = p.D, V = p.V;
   const int slot = slot_of(p.slots, b, p.nslots);
   const int64_t ps = pos_of(p.pos, p.pos_stride, b);
   const int64_t pt = ps < p.max_pos ? ps : p.max_pos - 1;
@@ -312,17 +314,14 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
   if (first < n) {
     fetch_k(first);
     fetch_v(first);
-  }
-
-  if (first < n) {
     const int64_t qk0 = (int64_t)p.H * MAPS * D;
-    for (int job = w; job < (owner ? 2 * MAPS + 1 : MAPS); job += 4) {
-      if (job < MAPS) {
-        const int64_t o = ((int64_t)h * MAPS + job) * D;
+    for (int job = w; job < (owner ? NJ + MAPS + 1 : NJ); job += 4) {
+      if (job < NJ) {
+        const int64_t o = ((int64_t)h0 * MAPS + job) * D;
         prepare_head<T>(p, row + o, p.bias ? p.bias + o : nullptr, p.qn_w, pt, q[job]);
-      } else if (job < 2 * MAPS) {
-        const int64_t o = qk0 + ((int64_t)g * MAPS + job - MAPS) * D;
-        prepare_head<T>(p, row + o, p.bias ? p.bias + o : nullptr, p.kn_w, pt, kn[job - MAPS]);
+      } else if (job < NJ + MAPS) {
+        const int64_t o = qk0 + ((int64_t)g * MAPS + job - NJ) * D;
+        prepare_head<T>(p, row + o, p.bias ? p.bias + o : nullptr, p.kn_w, pt, kn[job - NJ]);
       } else {
         const int64_t o = qk0 + (int64_t)p.G * MAPS * D + (int64_t)g * V;
         for (int d = lane; d < V; d += 64) {
@@ -334,25 +333,30 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
     }
   }
   __syncthreads();
-  if (owner && h % rep == 0) {   // (the values are exact in the activation type)
+  if (owner && h0 % rep == 0) {   // (the values are exact in the activation type)
     const int e = entry(n - 1);
     for (int i = tid; i < MAPS * D; i += 256) st(kc + ((int64_t)(i / D) * p.cap + e) * D + i % D, kn[i / D][i % D]);
     for (int i = tid; i < V; i += 256) st(vc + (int64_t)e * V + i, vn[i]);
   }
 
-  float mx[MAPS], ls[MAPS];
-  f32x4_t a4[MAPS];
+  float q8[R][8], snew[R];   // this lane's piece of the queries; the new key's scores
 #pragma unroll
-  for (int i = 0; i < MAPS; ++i) mx[i] = -INFINITY, ls[i] = 0.f, a4[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  float q8[8];
+  for (int r = 0; r < R; ++r) {
+    snew[r] = 0.f;
 #pragma unroll
-  for (int i = 0; i < 8; ++i) q8[i] = dok ? q[c][dl + i] : 0.f;
-  float snew = 0.f;   // the new key's score
-  if (owner) {
+    for (int i = 0; i < 8; ++i) q8[r][i] = dok ? q[r * MAPS + c][dl + i] : 0.f;
+    if (owner) {
 #pragma unroll
-    for (int i = 0; i < 8; ++i) snew += dok ? kn[c][dl + i] * q8[i] : 0.f;
-    snew = sum_lanes<LR>(snew);
+      for (int i = 0; i < 8; ++i) snew[r] += dok ? kn[c][dl + i] * q8[r][i] : 0.f;
+      snew[r] = sum_lanes<LR>(snew[r]);
+    }
   }
+  float mx[SM], ls[SM];   // of weight rows w, w + 4
+  f32x4_t a4[NJ];
+#pragma unroll
+  for (int i = 0; i < SM; ++i) mx[i] = -INFINITY, ls[i] = 0.f;
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) a4[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   int flip = 0;
   for (int k0 = first; k0 < end; k0 += 64, flip ^= 1) {
     const int cnt = min(64, end - k0);
@@ -360,25 +364,33 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
       const int k = part * (64 / PARTS) + i * RPL + kl;
-      float s = sum_lanes<LR>(dot8(kr[i], q8));
-      if (has_new && k == cnt - 1) s = snew;
-      if (lane % LR == 0) sc[flip][c][k] = s;
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        float s = sum_lanes<LR>(dot8(kr[i], q8[r]));
+        if (has_new && k == cnt - 1) s = snew[r];
+        if (lane % LR == 0) sc[flip][r * MAPS + c][k] = s;
+      }
     }
     if (k0 + 64 < end) fetch_k(k0 + 64);
-    __syncthreads();   // (two score buffers: the next tile's scores do not wait for this one's readers)
+    lds_barrier();   // (two score buffers: the next tile's scores do not wait for this one's readers)
 #pragma unroll
-    for (int m = 0; m < MAPS; ++m) {
-      float s = sc[flip][m][lane] * p.scale;
-      if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
-      if (lane >= cnt) s = -INFINITY;
-      const float m2 = fmaxf(mx[m], max64(s));
-      const float f = mx[m] == -INFINITY ? 0.f : expf(mx[m] - m2), x = lane < cnt ? expf(s - m2) : 0.f;
-      mx[m] = m2;
-      ls[m] = ls[m] * f + sum64(x);
-      a4[m] *= f;
-      pw[w][m][lane] = x;
+    for (int i = 0; i < SM; ++i) {
+      const int j = w + 4 * i;
+      if (j < NJ) {
+        float s = sc[flip][j][lane] * p.scale;
+        if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
+        if (lane >= cnt) s = -INFINITY;
+        const float m2 = fmaxf(mx[i], max64(s));
+        const float f = mx[i] == -INFINITY ? 0.f : expf(mx[i] - m2), x = lane < cnt ? expf(s - m2) : 0.f;
+        mx[i] = m2;
+        ls[i] = ls[i] * f + sum64(x);
+        pw[j][lane] = x;
+        if (lane == 0) fs[j] = f;
+      }
     }
-    __builtin_amdgcn_wave_barrier();
+    lds_barrier();
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) a4[j] *= fs[j];
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       if (i * kpp < 16) {
@@ -386,49 +398,145 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
         f32x4_t x = widen(vr[i]);
         if (has_new && k >= cnt - 1) x = ld4(vn + col);   // (past the end: any finite value, its weight is zero)
 #pragma unroll
-        for (int m = 0; m < MAPS; ++m) a4[m] += x * pw[w][m][k];
+        for (int j = 0; j < NJ; ++j) a4[j] += x * pw[j][k];
       }
     }
     if (k0 + 64 < end) fetch_v(k0 + 64);
   }
 #pragma unroll
-  for (int m = 0; m < MAPS; ++m) {
+  for (int j = 0; j < NJ; ++j) {
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      for (int o = lpr; o < 64; o <<= 1) a4[m][i] += __shfl_xor(a4[m][i], o, 64);
-    if (ks == 0 && (lane % lpr) * 4 < V) st4(&acc[w][m][col], a4[m]);
+      for (int o = lpr; o < 64; o <<= 1) a4[j][i] += __shfl_xor(a4[j][i], o, 64);
+    if (ks == 0 && (lane % lpr) * 4 < V) st4(&acc[w][j][col], a4[j]);
+  }
+  if (lane == 0) {
+#pragma unroll
+    for (int i = 0; i < SM; ++i)
+      if (w + 4 * i < NJ) msum[w + 4 * i] = mx[i], lsum[w + 4 * i] = ls[i];
   }
   __syncthreads();
-  float a[MAPS];
+
+  // ---- wave r finishes head h0 + r: columns lane, lane + 64, ...
+  float l[MAPS], a[MAPS][4];
+  const int hd = b * (p.H / R) + blockIdx.y, stride = NJ * (V + 2);
+  if (p.splits > 1) {
+    float* part_ = p.part + ((int64_t)hd * p.splits + sp) * stride;
+    for (int i = tid; i < NJ * V; i += 256) {
+      const int j = i / V, v = i % V;
+      __hip_atomic_store(part_ + j * (V + 2) + 2 + v, acc[0][j][v] + acc[1][j][v] + acc[2][j][v] + acc[3][j][v], __ATOMIC_RELAXED,
+                         __HIP_MEMORY_SCOPE_AGENT);
+    }
+    if (tid < NJ) {
+      __hip_atomic_store(part_ + tid * (V + 2), msum[tid], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      __hip_atomic_store(part_ + tid * (V + 2) + 1, lsum[tid], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // every wave's stores have left before the ticket
+    __syncthreads();
+    if (tid == 0) arrival = __hip_atomic_fetch_add(p.tickets + hd, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    __syncthreads();
+    if (arrival != p.splits - 1) return;
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup");
+    if (tid == 0) __hip_atomic_store(p.tickets + hd, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    if (w >= R) return;
+    float m[MAPS];
 #pragma unroll
-  for (int m = 0; m < MAPS; ++m) a[m] = tid < V ? acc[0][m][tid] + acc[1][m][tid] + acc[2][m][tid] + acc[3][m][tid] : 0.f;
-  finish<T, MAPS>(p, b, h, sp, mx, ls, a, red, &arrival);
+    for (int k = 0; k < MAPS; ++k) {
+      m[k] = -INFINITY;
+      l[k] = 0.f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) a[k][i] = 0.f;
+    }
+    for (int s0 = 0; s0 < p.splits; s0 += 8) {   // eight splits' partial sums per round trip
+      float ms[MAPS][8], lp[MAPS][8], as[MAPS][8][4];
+#pragma unroll
+      for (int s = 0; s < 8; ++s)
+#pragma unroll
+        for (int k = 0; k < MAPS; ++k) {
+          const float* o = p.part + ((int64_t)hd * p.splits + min(s0 + s, p.splits - 1)) * stride + (w * MAPS + k) * (V + 2);
+          ms[k][s] = __hip_atomic_load(o, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+          lp[k][s] = __hip_atomic_load(o + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            as[k][s][i] = i == 0 || 64 * i < V ? __hip_atomic_load(o + 2 + min(lane + 64 * i, V - 1), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) : 0.f;
+        }
+#pragma unroll
+      for (int s = 0; s < 8; ++s)
+#pragma unroll
+        for (int k = 0; k < MAPS; ++k) {
+          if (s0 + s >= p.splits || ms[k][s] == -INFINITY) continue;   // (no split, or one past the visible keys)
+          const float m2 = fmaxf(m[k], ms[k][s]), f = m[k] == -INFINITY ? 0.f : expf(m[k] - m2), f2 = expf(ms[k][s] - m2);
+          l[k] = l[k] * f + lp[k][s] * f2;
+#pragma unroll
+          for (int i = 0; i < 4; ++i) a[k][i] = a[k][i] * f + as[k][s][i] * f2;
+          m[k] = m2;
+        }
+    }
+  } else {
+    if (w >= R) return;
+#pragma unroll
+    for (int k = 0; k < MAPS; ++k) {
+      const int j = w * MAPS + k;
+      l[k] = lsum[j];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int v = min(lane + 64 * i, V - 1);
+        a[k][i] = acc[0][j][v] + acc[1][j][v] + acc[2][j][v] + acc[3][j][v];
+      }
+    }
+  }
+  float o[4], ss = 0.f, sc_out = 1.f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    o[i] = a[0][i] / l[0];
+    if constexpr (MAPS == 2) o[i] -= p.lam * (a[MAPS - 1][i] / l[MAPS - 1]);
+    if (lane + 64 * i < V) ss += o[i] * o[i];
+  }
+  if constexpr (MAPS == 2) sc_out = p.out_scale / sqrtf(sum64(ss) / (float)V + p.out_eps);
+  T* y = static_cast<T*>(p.y) + (int64_t)b * p.ldy + (int64_t)(h0 + w) * V;
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (lane + 64 * i < V) st(y + lane + 64 * i, o[i] * sc_out);
+}
+
+template <typename T, int MAPS, int R>
+static void launch_decode(const WindowAttnParams& p, hipStream_t s) {
+  const dim3 grid((unsigned)p.splits, (unsigned)(p.H / R), (unsigned)p.B);
+  if (p.D <= 32) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 4, R>), grid, dim3(256), 0, s, p);
+  else if (p.D <= 64) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 8, R>), grid, dim3(256), 0, s, p);
+  else hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 16, R>), grid, dim3(256), 0, s, p);
 }
 
 template <typename T, int MAPS>
 static int run_decode(const WindowAttnParams& p, hipStream_t s) {
-  const dim3 grid((unsigned)p.splits, (unsigned)p.H, (unsigned)p.B);
-  if (p.tiles > 0 && p.D <= 32) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 4>), grid, dim3(256), 0, s, p);
-  else if (p.tiles > 0 && p.D <= 64) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 8>), grid, dim3(256), 0, s, p);
-  else if (p.tiles > 0) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 16>), grid, dim3(256), 0, s, p);
-  else hipLaunchKernelGGL((attn_decode_any_kernel<T, MAPS>), grid, dim3(256), 0, s, p);
+  if (p.tiles == 0)
+    hipLaunchKernelGGL((attn_decode_any_kernel<T, MAPS>), dim3((unsigned)p.splits, (unsigned)p.H, (unsigned)p.B), dim3(256), 0, s, p);
+  else if (p.share == 4) launch_decode<T, MAPS, 4>(p, s);
+  else if (p.share == 2) launch_decode<T, MAPS, 2>(p, s);
+  else launch_decode<T, MAPS, 1>(p, s);
   return hipGetLastError() == hipSuccess ? 0 : 1;
 }
 
 }  // namespace hybrid
 
-// workgroups per head and 64-key tiles each (0: the any-size kernel) for at most `seen` visible keys
+// heads a workgroup takes, workgroups per such group and 64-key tiles each (0: the any-size kernel) for at
+// most `seen` visible keys
 void attn_decode_plan(WindowAttnParams& p, int64_t seen) {
+  const int rep = p.H / p.G;
   if (p.D % 8 == 0 && p.V % 8 == 0 && p.D <= 128) {
-    // about 512 workgroups, but not more than 8 a head before each has 4 tiles: the merge has its price
-    // (16 heads, 1,024 visible keys, us: 1 sequence 8 / 16 workgroups a head 14.1 / 15.4; 8 sequences 1 / 2 /
-    // 4 / 8 of them 46 / 29 / 20 / 27)
-    const int64_t tiles = (seen + 63) / 64, heads = (int64_t)p.B * p.H, most = tiles / 4 > 8 ? tiles / 4 : (tiles < 8 ? tiles : 8);
-    int64_t splits = 512 / heads;
+    // heads share a workgroup's keys once there are enough workgroups without that (16 heads, 1,024 visible
+    // keys, us with 1 / 4 heads a workgroup: 1 sequence 13 / 20, 16 sequences 31 / 25, 32 sequences 49 / 33)
+    const int64_t all = (int64_t)p.B * p.H;
+    p.share = all >= 256 && rep % 4 == 0 ? 4 : (all >= 128 && rep % 2 == 0 ? 2 : 1);
+    // about 512 workgroups, but not more than 8 a group before each has 4 tiles: the merge has its price
+    const int64_t tiles = (seen + 63) / 64, groups = (int64_t)p.B * p.H / p.share;
+    const int64_t most = tiles / 4 > 8 ? tiles / 4 : (tiles < 8 ? tiles : 8);
+    int64_t splits = 512 / groups;
     splits = splits < 1 ? 1 : (splits > most ? most : splits);
     p.tiles = (int)((tiles + splits - 1) / splits);
     p.splits = (int)((tiles + p.tiles - 1) / p.tiles);
   } else {
+    p.share = 1;
     p.tiles = 0;
     p.splits = (int)((seen + 255) / 256);
   }

@@ -95,7 +95,7 @@ def window_attention(buf: torch.Tensor, B: int, T: int, sizes: AttnSizes, rule: 
                      lengths: Optional[torch.Tensor], slots: Optional[torch.Tensor], k_cache: torch.Tensor,
                      v_cache: torch.Tensor, prompt: bool, fused: bool = True) -> torch.Tensor:
     """Attention of the queries in buf (after attn_prep_): over the tokens of this step when they start
-    at position 0 (`prompt`), else over the cache.  Returns [B T, H V] (padding rows are zero).
+    at position 0 (`prompt`), else over the cache (a ring that wraps must hold window + T - 1 keys).  Returns [B T, H V] (padding rows are zero).
     fused: the matrix-core prompt kernel and the split decode kernel where the sizes allow (bf16)."""
     H, G, R, D, V = sizes.as_list()
     y = torch.empty((B * T, H * V), dtype=buf.dtype, device=buf.device)
@@ -105,8 +105,8 @@ def window_attention(buf: torch.Tensor, B: int, T: int, sizes: AttnSizes, rule: 
         return y
     y.zero_()
     cap = k_cache.shape[2]
-    if not prompt and rule.window > 0 and T > cap - rule.window + 1:
-        raise ValueError(f"{T} new tokens do not fit a ring of {cap} with a window of {rule.window}")
+    if not prompt and T > cap:
+        raise ValueError(f"{T} new tokens do not fit a ring of {cap}")
     for b in range(B):
         slot = int(slots[b]) if slots is not None else b
         p0 = int(positions.reshape(B, -1)[b, 0])

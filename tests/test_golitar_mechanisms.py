@@ -253,7 +253,8 @@ class Attn:
 
 ATTN = [  # H, G, maps, D, V, rot, window, softcap
     (4, 2, 2, 16, 24, 8, 37, 20.0), (2, 1, 2, 40, 64, 40, 64, 30.0), (3, 3, 2, 10, 6, 2, 1, 60.0),
-    (2, 2, 2, 72, 136, 64, 90, 50.0), (2, 1, 1, 48, 32, 16, 0, 0.0), (2, 1, 2, 64, 128, 0, 0, 30.0), (1, 1, 2, 128, 256, 2, 5, 0.0)]
+    (2, 2, 2, 72, 136, 64, 90, 50.0), (2, 1, 1, 48, 32, 16, 0, 0.0), (2, 1, 2, 64, 128, 0, 0, 30.0), (1, 1, 2, 128, 256, 2, 5, 0.0),
+    (8, 2, 2, 24, 40, 12, 70, 30.0), (4, 1, 1, 104, 72, 8, 0, 25.0), (12, 3, 2, 40, 160, 0, 100, 0.0)]
 
 
 @pytest.mark.parametrize("where", WHERE)
@@ -333,23 +334,46 @@ def test_first_tokens_see_only_what_is_there(where):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("visible", [63, 64, 65, 255, 257, 600, 2200])
-def test_split_decode(visible):
-    """Decoding over more than 256 visible keys (several workgroups per head and a merge), repeated: the
+@pytest.mark.parametrize("heads,vdim", [(2, 12), (4, 24)])   # any-size kernel; four heads a workgroup
+def test_split_decode(visible, heads, vdim):
+    """Decoding over many visible keys (several workgroups per head and a merge), repeated: the
     arrival counters are left at zero; a key that outweighs all others is far away."""
     where = ("cuda", torch.float32, 5e-5)
     T = visible + 40
-    a = Attn(where, 1, T, 2, 1, 2, 16, 12, 0, visible, 20.0, cap=visible + 15, scale=1.0, seed=8)
+    a = Attn(where, 1, T, heads, 1, 2, 16, vdim, 0, visible, 20.0, cap=visible + 15, scale=1.0, seed=8)
     a.bias.zero_()
     probe = rnd(16, seed=60)
+    k0 = heads * 32   # the first key column
     for i in range(T - 3, T):
         a.buf_o[0, i, :16] = probe
-        a.buf_o[0, i - visible + 1, 64:80] = probe * 1.5
+        a.buf_o[0, i - visible + 1, k0:k0 + 16] = probe * 1.5
     a.buf = a.buf_o.to(where[1]).to(where[0])
     a.buf_o = a.buf.double().cpu()
     want = a.oracle(0, T)
     a.step(0, T - 3, True)
     for t in range(T - 3, T):
         assert rel_err(a.step(t, 1, False, decode=True)[0], want[t:t + 1]) < where[2]
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("B,H,G", [(16, 8, 2), (40, 8, 2), (48, 6, 3)])
+def test_decode_shares_keys_between_heads(B, H, G):
+    """Enough sequences that several query heads of a key / value head share a workgroup, against the
+    one-wave-a-query kernel on the same cache; some sequences are much shorter than the window."""
+    where = ("cuda", torch.float32, 5e-5)
+    a = Attn(where, B, 150, H, G, 2, 24, 40, 8, 130, 20.0, cap=150, seed=12)
+    a.step(0, 149, True)
+    pos = torch.randint(0, 150, (B, 1), generator=torch.Generator().manual_seed(3)).cuda()
+    buf = a.buf[:, 149].contiguous()
+    prep = (a.bias.cuda(), a.qn.cuda(), a.kn.cuda(), 1e-5, a.cos.cuda(), a.sin.cuda(), pos)
+    kc, vc = a.kc.clone(), a.vc.clone()
+    got = ops.attn_decode(buf, a.sz, a.rule, *prep, a.slots, kc, vc, a.tickets)
+    row = buf.clone()
+    ops.attn_prep_(row, B, 1, a.sz, *prep, None, a.slots, a.kc, a.vc)
+    want = ops.window_attention(row, B, 1, a.sz, a.rule, pos, None, a.slots, a.kc, a.vc, False, False)
+    assert rel_err(got, want.cpu()) < 5e-5
+    assert rel_err(kc.flatten(0, 2), a.kc.flatten(0, 2).cpu()) < 1e-5 and torch.equal(vc, a.vc)
+    assert int(a.tickets.abs().sum()) == 0
 
 
 # ------------------------------------------------------------------ fused decode projections

@@ -328,3 +328,14 @@ def test_trace_run_needs_a_gpu(model_dirs, tmp_path):
     r = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", model_dirs["mixed"], "--out", str(tmp_path),
                         "--max-tokens", "8"], input="", capture_output=True, text=True, timeout=600, env=env)
     assert r.returncode != 0 and "GPU" in r.stderr
+
+
+def test_command_line(model_dirs, tmp_path, capsys):
+    sys.path.insert(0, os.path.join(ROOT, "examples", "inference"))
+    from llama3_2_runner import main
+
+    out = str(tmp_path / "traced")
+    main(["trace", "--model_path", model_dirs["mixed"], "--traced_path", out, "--max_prompt_length", "8", "--sequence_length", "14"],
+         runner_cls=GolitarRunner)
+    rows = main(["generate", "--traced_path", out, "--prompt_ids", ",".join(map(str, tokens(8, 211)))], runner_cls=GolitarRunner)
+    assert rows.shape == (1, 14) and rows[0, :8].tolist() == tokens(8, 211)
