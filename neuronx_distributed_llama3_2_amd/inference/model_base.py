@@ -156,6 +156,21 @@ class DecoderInferenceMixin:
         logits = self._gather_vocab(self._proj(self.lm_head, h))
         return (logits, h) if return_hidden else logits
 
+    def _forward_in_steps(self, input_ids, positions, seq_ids, last_index, return_hidden, lengths, logit_rows, step):
+        """forward_tokens over the cache, `step` new tokens at a time."""
+        B, T = input_ids.shape
+        out = []
+        for t in range(0, T, step):
+            n = (lengths - t).clamp(0, min(step, T - t)) if lengths is not None else None
+            out.append(self.forward_tokens(input_ids[:, t:t + step], positions[:, t:t + step], seq_ids,
+                                           return_hidden=True, lengths=n))
+        parts = [torch.cat([o[i] for o in out], 1) for i in range(2)]
+        if logit_rows is None and last_index is not None:
+            logit_rows = torch.arange(B, device=input_ids.device) * T + last_index
+        if logit_rows is not None:
+            parts = [p.reshape(B * T, -1)[logit_rows] for p in parts]
+        return tuple(parts) if return_hidden else parts[0]
+
     # ------------------------------------------------------------------ fused decode path
     def _fused_ffn_weights(self, layer):
         """(post-attention norm weight, fused gate/up [2I, H], down [H, I]) when the feed-forward

@@ -193,20 +193,6 @@ class GolitarInferenceModel(DecoderInferenceMixin, nn.Module):
         h = (u * torch.rsqrt(u.square().mean(-1, keepdim=True) + self.eps) * (1 + norm)).to(dt)
         return (logits, h) if logit_rows is not None else (logits.unsqueeze(1), h.unsqueeze(1))
 
-    def _forward_in_steps(self, input_ids, positions, seq_ids, last_index, return_hidden, lengths, logit_rows, step):
-        B, T = input_ids.shape
-        out = []
-        for t in range(0, T, step):
-            n = (lengths - t).clamp(0, min(step, T - t)) if lengths is not None else None
-            out.append(self.forward_tokens(input_ids[:, t:t + step], positions[:, t:t + step], seq_ids,
-                                           return_hidden=True, lengths=n))
-        parts = [torch.cat([o[i] for o in out], 1) for i in range(2)]
-        if logit_rows is None and last_index is not None:
-            logit_rows = torch.arange(B, device=input_ids.device) * T + last_index
-        if logit_rows is not None:
-            parts = [p.reshape(B * T, -1)[logit_rows] for p in parts]
-        return tuple(parts) if return_hidden else parts[0]
-
     def _ones(self, device) -> torch.Tensor:
         if getattr(self, "_ones_buf", None) is None or self._ones_buf.device != device:
             self._ones_buf = torch.ones(self.config.streams, dtype=torch.float32, device=device)

@@ -22,6 +22,7 @@ FAMILIES: Dict[str, Family] = {
     "mixtral": Family(".moe", "MixtralForCausalLMInference", "MixtralRunner"),
     "dbrx": Family(".moe", "DbrxForCausalLMInference", "DbrxRunner"),
     "golitar": Family(".golitar", "GolitarForCausalLMInference", "GolitarRunner", "_hybrid"),
+    "bezurax": Family(".bezurax", "BezuraxForCausalLMInference", "BezuraxRunner", "_hybrid"),
 }
 
 

@@ -6,3 +6,7 @@ from .differential_attention import DifferentialAttentionMixer, interleaved_rope
 from .gated_delta import GatedDeltaMixer  # noqa: F401
 from .hyper_connection import HyperConnection  # noqa: F401
 from .mlp import SquaredReluMLP  # noqa: F401
+from .channel_delta import ChannelDelta  # noqa: F401
+from .experts import RoutedExperts  # noqa: F401
+from .parallel_mixer import ParallelMixer  # noqa: F401
+from .pooled_attention import PooledAttention  # noqa: F401

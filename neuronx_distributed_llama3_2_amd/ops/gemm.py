@@ -47,13 +47,14 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias=None, out: torch.Tensor = None
     return y
 
 
-def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
-    """x [..., K] @ w[N, K]^T -> fp32 [..., N]: the accumulator unrounded (logits of 16-bit weights)."""
+def linear_f32(x: torch.Tensor, w: torch.Tensor, alpha: float = 1.0) -> torch.Tensor:
+    """alpha * x [..., K] @ w[N, K]^T -> fp32 [..., N]: the accumulator unrounded (logits of 16-bit weights)."""
     if _native(x, w) and x.stride(-1) == 1:
         y = torch.empty(x.shape[:-1] + (w.shape[0],), dtype=torch.float32, device=x.device)
-        gemm_ext().gemm(x.reshape(-1, x.shape[-1]), w.t(), y.view(-1, w.shape[0]), None, 1.0, 0.0)
+        gemm_ext().gemm(x.reshape(-1, x.shape[-1]), w.t(), y.view(-1, w.shape[0]), None, float(alpha), 0.0)
         return y
-    return torch.nn.functional.linear(x.float(), w.float())
+    y = torch.nn.functional.linear(x.float(), w.float())
+    return y if alpha == 1.0 else y.mul_(alpha)
 
 
 def matmul(a: torch.Tensor, b: torch.Tensor, out: torch.Tensor = None) -> torch.Tensor:
