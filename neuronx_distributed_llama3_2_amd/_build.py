@@ -26,8 +26,8 @@ BUILD_DIR = PKG_DIR.parent / "build" / "nxd_csrc"
 ARCH = os.environ.get("NXD_OFFLOAD_ARCH", "gfx950")
 EXT_SUFFIX = sysconfig.get_config_var("EXT_SUFFIX") or ".so"
 # `_C`: every kernel of csrc/*.hip.  `_hybrid`: the mechanisms of the hybrid decoders
-# (csrc/hybrid/: hyper-connections, gated delta rule, windowed / differential attention) and the GEMM
-# dispatch, a small module of its own, so that serving such a model compiles only what it runs.
+# (csrc/hybrid/: hyper-connections, delta rules, windowed / differential / pooled attention, routed experts) and the
+# dense and grouped GEMM dispatch, a small module of its own, so that serving such a model compiles only what it runs.
 TARGETS = ("_C", "_hybrid")
 
 
@@ -90,7 +90,8 @@ def _sources(target: str):
     """(kernel TUs, host TUs that include the torch headers) of one extension module."""
     if target == "_C":
         return sorted(CSRC.glob("*.hip")), sorted(CSRC.glob("*.cpp"))
-    return sorted((CSRC / "hybrid").glob("*.hip")), [*sorted((CSRC / "hybrid").glob("*.cpp")), CSRC / "gemm.cpp"]
+    shared = [CSRC / n for n in ("grouped_gemm.hip", "grouped_rowgemm.hip")]   # the experts' matrix products
+    return [*sorted((CSRC / "hybrid").glob("*.hip")), *shared], [*sorted((CSRC / "hybrid").glob("*.cpp")), CSRC / "gemm.cpp"]
 
 
 def lib_path(target: str) -> Path:

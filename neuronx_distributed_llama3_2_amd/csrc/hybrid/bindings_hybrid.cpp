@@ -1,15 +1,13 @@
 // Python bindings of the hybrid-decoder kernels (module `neuronx_distributed_llama3_2_amd._hybrid`).
 // Every entry point checks shapes, types and the kernels' size limits on the host before it launches
 // on the caller's current stream.
-#include <torch/extension.h>
-#include <ATen/hip/HIPContext.h>
-#include <hip/hip_runtime.h>
-
+#include "bindings_util.h"
 #include "delta_rule.h"
 #include "gemv_hyper.h"
 #include "window_attn.h"
 
-void register_gemm(pybind11::module& m);  // ../gemm.cpp
+void register_gemm(pybind11::module& m);      // ../gemm.cpp
+void register_parallel(pybind11::module& m);  // bindings_parallel.cpp
 
 namespace nxd {
 int hyper_step_launch(bool, float*, const void*, const int64_t*, int64_t, const void*, int64_t, const float*, const float*,
@@ -29,48 +27,12 @@ int attn_row_launch(bool, const WindowAttnParams&, hipStream_t);
 void attn_decode_plan(WindowAttnParams&, int64_t);
 int attn_decode_launch(bool, const WindowAttnParams&, hipStream_t);
 int gemv_hyper_launch(int, const GemvHyperParams&, hipStream_t);
+int pooled_prep_launch(bool, const WindowAttnParams&, hipStream_t);
 }  // namespace nxd
 
 namespace {
 
-using at::Tensor;
-using Opt = c10::optional<Tensor>;
-
-hipStream_t cur_stream() { return at::hip::getCurrentHIPStream().stream(); }
-void check_rc(int rc, const char* what) { TORCH_CHECK(rc == 0, what, " failed with code ", rc); }
-
-// activation tensors: bf16 or fp32, unit inner stride
-bool act_f32(const Tensor& t, const char* n) {
-  TORCH_CHECK(t.is_cuda() && t.dim() >= 2 && t.stride(-1) == 1, n, ": GPU tensor with a unit inner stride");
-  TORCH_CHECK(t.scalar_type() == at::kBFloat16 || t.scalar_type() == at::kFloat, n, ": bf16 or fp32");
-  return t.scalar_type() == at::kFloat;
-}
-void same_act(const Tensor& t, const Tensor& like, const char* n) {
-  act_f32(t, n);
-  TORCH_CHECK(t.scalar_type() == like.scalar_type(), n, ": activation type differs");
-}
-float* f32_ptr(const Tensor& t, int64_t numel, const char* n) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kFloat && t.is_contiguous() && t.numel() == numel, n,
-              ": contiguous fp32 of ", numel, " elements");
-  return t.data_ptr<float>();
-}
-float* f32_opt(const Opt& t, int64_t numel, const char* n) { return t.has_value() ? f32_ptr(*t, numel, n) : nullptr; }
-const int* i32_opt(const Opt& t, int64_t numel, const char* n) {
-  if (!t.has_value()) return nullptr;
-  TORCH_CHECK(t->is_cuda() && t->scalar_type() == at::kInt && t->is_contiguous() && t->numel() == numel, n,
-              ": contiguous int32 of ", numel, " elements");
-  return t->data_ptr<int>();
-}
-// first position of every sequence: int64 [B] or [B, T'] (column 0)
-const int64_t* pos_ptr(const Tensor& t, int64_t B, int64_t* stride) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kLong && t.dim() >= 1 && t.dim() <= 2 && t.size(0) == B,
-              "positions: int64 [B] or [B, T]");
-  *stride = B > 1 ? t.stride(0) : 0;
-  return t.data_ptr<int64_t>();
-}
-void check_align(const Tensor& t, const char* n) {
-  TORCH_CHECK(reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0, n, ": 16-byte alignment");
-}
+using namespace nxd::bind;
 
 void hyper_step(Tensor x, Opt embed, Opt ids, Opt y, Opt bias, Opt mix, Opt write, Opt read, Opt norm_w, double eps, Opt h,
                 Opt rows, bool store) {
@@ -254,6 +216,10 @@ nxd::WindowAttnParams attn_params(const Tensor& buf, int64_t B, int64_t T, const
   p.kc = kc.data_ptr();
   p.vc = vc.data_ptr();
   p.cap = (int)kc.size(2);
+  p.v_off = (p.H + p.G) * p.maps * p.D;
+  p.kbuf = static_cast<const char*>(p.buf) + (int64_t)p.H * p.maps * p.D * buf.element_size();
+  p.vbuf = static_cast<const char*>(p.buf) + (int64_t)p.v_off * buf.element_size();
+  p.ldk = p.ldv = p.ldb;
   return p;
 }
 
@@ -331,6 +297,129 @@ void attn_decode(Tensor buf, std::vector<int64_t> sizes, Opt bias, Opt qn_w, Opt
   check_rc(nxd::attn_decode_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "attn_decode");
 }
 
+// Pooled blocks.  sizes (H, G, D); buf columns q (H D) | k (G D, also the values); kn [B T, G D] normalised keys
+nxd::WindowAttnParams pooled_params(const Tensor& buf, const Opt& kn, int64_t B, int64_t T, const std::vector<int64_t>& sizes,
+                                    int64_t window, int64_t pool, const Tensor& pos, const Opt& lens, const Opt& slots,
+                                    const Tensor& kc, const Tensor& vc, const Tensor& pk, const Tensor& pv) {
+  const bool f32 = act_f32(buf, "buf");
+  same_act(kc, buf, "k cache");
+  same_act(vc, buf, "v cache");
+  same_act(pk, buf, "pooled k");
+  same_act(pv, buf, "pooled v");
+  TORCH_CHECK(sizes.size() == 3, "pooled attention: sizes (H, G, D)");
+  nxd::WindowAttnParams p{};
+  p.B = (int)B;
+  p.T = (int)T;
+  p.H = (int)sizes[0];
+  p.G = (int)sizes[1];
+  p.maps = 1;
+  p.D = p.V = (int)sizes[2];
+  TORCH_CHECK(B >= 1 && B <= 65535 && T >= 1 && B * T <= (1 << 30), "pooled attention: rows");
+  TORCH_CHECK(p.G >= 1 && p.H >= 1 && p.H <= 65535 && p.H % p.G == 0 && p.D >= 2 && p.D <= 256, "pooled attention: head layout, size up to 256");
+  TORCH_CHECK(buf.dim() == 2 && buf.size(0) == B * T && buf.size(1) >= (p.H + p.G) * p.D, "pooled attention: projection columns");
+  TORCH_CHECK(kc.dim() == 4 && kc.is_contiguous() && kc.size(1) == p.G && kc.size(3) == p.D && vc.is_contiguous() && vc.sizes() == kc.sizes(),
+              "pooled attention: caches [slots, G, cap, D]");
+  TORCH_CHECK(pk.dim() == 4 && pk.is_contiguous() && pk.size(0) == kc.size(0) && pk.size(1) == p.G && pk.size(3) == p.D &&
+                  pv.is_contiguous() && pv.sizes() == pk.sizes() && pk.size(2) >= 1 && pk.size(2) < (1 << 30),
+              "pooled attention: pooled caches [slots, G, blocks, D]");
+  TORCH_CHECK(kc.size(2) >= 1 && kc.size(2) < (1 << 30), "pooled attention: cache length");
+  TORCH_CHECK(slots.has_value() || B <= kc.size(0), "pooled attention: more sequences than slots");
+  TORCH_CHECK(window >= 1 && window < (1 << 30) && pool >= 1 && pool < (1 << 30), "pooled attention: window and block");
+  for (const Tensor* t : {&kc, &vc, &pk, &pv}) check_align(*t, "caches");
+  p.buf = buf.data_ptr();
+  p.ldb = buf.stride(0);
+  p.v_off = p.H * p.D;
+  p.vbuf = static_cast<const char*>(p.buf) + (int64_t)p.v_off * buf.element_size();
+  p.ldv = p.ldb;
+  if (kn.has_value()) {
+    same_act(*kn, buf, "kn");
+    TORCH_CHECK(kn->dim() == 2 && kn->size(0) == B * T && kn->size(1) == p.G * p.D, "pooled attention: kn [B T, G D]");
+    p.kbuf = kn->data_ptr();
+    p.ldk = kn->stride(0);
+  }
+  p.pos = pos_ptr(pos, B, &p.pos_stride);
+  p.lens = i32_opt(lens, B, "lens");
+  p.slots = i32_opt(slots, B, "slots");
+  p.nslots = (int)kc.size(0);
+  p.kc = kc.data_ptr();
+  p.vc = vc.data_ptr();
+  p.cap = (int)kc.size(2);
+  p.window = (int)window;
+  p.pool = (int)pool;
+  p.pcap = (int)pk.size(2);
+  p.pk = pk.data_ptr();
+  p.pv = pv.data_ptr();
+  p.norm_all = true;
+  (void)f32;
+  return p;
+}
+
+void set_pooled_norms(nxd::WindowAttnParams& p, const Tensor& qn_w, const Tensor& kn_w, double eps) {
+  p.qn_w = f32_ptr(qn_w, p.H * p.D, "q norm");
+  p.kn_w = f32_ptr(kn_w, p.G * p.D, "k norm");
+  check_align(qn_w, "q norm");
+  check_align(kn_w, "k norm");
+  p.eps = (float)eps;
+}
+
+void set_pooled_out(nxd::WindowAttnParams& p, double scale, const Tensor& buf, const Tensor& out, double out_scale) {
+  same_act(out, buf, "out");
+  TORCH_CHECK(out.dim() == 2 && out.size(0) == (int64_t)p.B * p.T && out.size(1) == p.H * p.D, "pooled attention: out [B T, H D]");
+  p.scale = (float)scale;
+  p.out_scale = (float)out_scale;
+  p.y = out.data_ptr();
+  p.ldy = out.stride(0);
+}
+
+void check_ring(const nxd::WindowAttnParams& p, bool prompt) {
+  // a ring that wraps must still hold what the first new token sees and the blocks the step completes
+  TORCH_CHECK(prompt || p.T <= p.cap, "pooled attention: ", p.T, " new tokens do not fit a ring of ", p.cap);
+}
+
+void pooled_prep(Tensor buf, Tensor kn, int64_t B, int64_t T, std::vector<int64_t> sizes, Tensor qn_w, Tensor kn_w, double eps,
+                 int64_t pool, Tensor pos, Opt lens, Opt slots, Tensor kc, Tensor vc, Tensor pk, Tensor pv, bool prompt) {
+  auto p = pooled_params(buf, kn, B, T, sizes, 1, pool, pos, lens, slots, kc, vc, pk, pv);
+  check_ring(p, prompt);
+  set_pooled_norms(p, qn_w, kn_w, eps);
+  p.from_buf = prompt ? 1 : 0;
+  check_rc(nxd::pooled_prep_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "pooled_prep");
+}
+
+void pooled_attn(Tensor buf, Tensor kn, int64_t B, int64_t T, std::vector<int64_t> sizes, double scale, int64_t window, int64_t pool,
+                 Tensor pos, Opt lens, Opt slots, Tensor kc, Tensor vc, Tensor pk, Tensor pv, Tensor out, double out_scale,
+                 bool prompt, bool fused) {
+  auto p = pooled_params(buf, kn, B, T, sizes, window, pool, pos, lens, slots, kc, vc, pk, pv);
+  check_ring(p, prompt);
+  set_pooled_out(p, scale, buf, out, out_scale);
+  p.from_buf = prompt ? 1 : 0;
+  const bool f32 = buf.scalar_type() == at::kFloat;
+  if (fused && !f32 && nxd::attn_prompt_supported(p)) {
+    check_rc(nxd::attn_prompt_launch(p, cur_stream()), "attn_prompt");
+    return;
+  }
+  check_rc(nxd::attn_row_launch(f32, p, cur_stream()), "pooled_attn");
+}
+
+void pooled_decode(Tensor buf, std::vector<int64_t> sizes, Tensor qn_w, Tensor kn_w, double eps, double scale, int64_t window,
+                   int64_t pool, Tensor pos, Opt slots, Tensor kc, Tensor vc, Tensor pk, Tensor pv, Tensor tickets, Tensor out,
+                   double out_scale) {
+  const int64_t B = buf.size(0);
+  auto p = pooled_params(buf, Opt(), B, 1, sizes, window, pool, pos, Opt(), slots, kc, vc, pk, pv);
+  set_pooled_norms(p, qn_w, kn_w, eps);
+  set_pooled_out(p, scale, buf, out, out_scale);
+  p.max_pos = 1 << 30;
+  nxd::attn_decode_plan(p, std::min(p.window, p.cap) + p.pcap);
+  TORCH_CHECK(tickets.is_cuda() && tickets.scalar_type() == at::kInt && tickets.is_contiguous() && tickets.numel() >= B * p.H,
+              "pooled_decode: int32 tickets, B H of them");
+  Tensor part;
+  if (p.splits > 1) {
+    part = at::empty({B * p.H * p.splits * (p.V + 2)}, buf.options().dtype(at::kFloat));
+    p.part = part.data_ptr<float>();
+    p.tickets = tickets.data_ptr<int>();
+  }
+  check_rc(nxd::attn_decode_launch(buf.scalar_type() == at::kFloat, p, cur_stream()), "pooled_decode");
+}
+
 // y = epi(x w^T), 1..4 rows of bf16; x bf16 [M, K], or u fp32 [M, K] normalised on the way in.  epi: 0 bf16,
 // 1 squared ReLU, 2 fp32 with cap, 3 into the streams (y unused, `un` receives the next sublayer's input)
 void gemv_hyper(int64_t epi, Opt x, Opt u, Opt norm_w, double eps, Tensor w, Opt y, double cap, Opt streams, Opt bias, Opt mix,
@@ -389,6 +478,7 @@ void gemv_hyper(int64_t epi, Opt x, Opt u, Opt norm_w, double eps, Tensor w, Opt
 
 PYBIND11_MODULE(_hybrid, m) {
   register_gemm(m);
+  register_parallel(m);
   namespace py = pybind11;
   m.def("hyper_step", &hyper_step, py::arg("x"), py::arg("embed") = py::none(), py::arg("ids") = py::none(),
         py::arg("y") = py::none(), py::arg("bias") = py::none(), py::arg("mix") = py::none(), py::arg("write") = py::none(),
@@ -406,6 +496,9 @@ PYBIND11_MODULE(_hybrid, m) {
         py::arg("softcap"), py::arg("window"), py::arg("lam"), py::arg("out_scale"), py::arg("out_eps"), py::arg("pos"),
         py::arg("lens"), py::arg("slots"), py::arg("kc"), py::arg("vc"), py::arg("y"), py::arg("from_buf"), py::arg("fused") = true);
   m.def("attn_decode", &attn_decode);
+  m.def("pooled_prep", &pooled_prep);
+  m.def("pooled_attn", &pooled_attn);
+  m.def("pooled_decode", &pooled_decode);
   m.def("gemv_hyper", &gemv_hyper, py::arg("epi"), py::arg("x") = py::none(), py::arg("u") = py::none(),
         py::arg("norm_w") = py::none(), py::arg("eps") = 0.0, py::arg("w"), py::arg("y") = py::none(), py::arg("cap") = 0.0,
         py::arg("streams") = py::none(), py::arg("bias") = py::none(), py::arg("mix") = py::none(),

@@ -1,5 +1,6 @@
 // Causal attention with a sliding window, score soft-capping and one or two maps per head
-// (differential attention), over a per-layer ring cache.
+// (differential attention), over a per-layer ring cache; optionally with one key and value for each block
+// of tokens before the window (one map, pooled_attn.hip).
 //
 //   attn_prep   : bias, per-head RMS norm of q / k, rotary turn of the pairs (2i, 2i + 1) of the first
 //                 `rot` dimensions, in place in the projection buffer; k and v also to the cache
@@ -140,10 +141,10 @@ struct KeySource {
   int mod;
   __device__ KeySource(const WindowAttnParams& p, int b, int g) {
     if (p.from_buf) {
-      const T* base = static_cast<const T*>(p.buf) + (int64_t)b * p.T * p.ldb;
-      k = base + (int64_t)(p.H + g) * p.maps * p.D;
-      v = base + (int64_t)(p.H + p.G) * p.maps * p.D + (int64_t)g * p.V;
-      ks = vs = p.ldb;
+      k = static_cast<const T*>(p.kbuf) + (int64_t)b * p.T * p.ldk + (int64_t)g * p.maps * p.D;
+      v = static_cast<const T*>(p.vbuf) + (int64_t)b * p.T * p.ldv + (int64_t)g * p.V;
+      ks = p.ldk;
+      vs = p.ldv;
       kmap = p.D;
       mod = 0x7fffffff;
     } else {
@@ -155,6 +156,16 @@ struct KeySource {
       kmap = (int64_t)p.cap * p.D;
       mod = p.cap;
     }
+  }
+  struct Pooled {};
+  __device__ KeySource(const WindowAttnParams& p, int b, int g, Pooled) {   // (one map)
+    const int64_t head = (int64_t)slot_of(p.slots, b, p.nslots) * p.G + g;
+    k = static_cast<const T*>(p.pk) + head * p.pcap * p.D;
+    v = static_cast<const T*>(p.pv) + head * p.pcap * p.V;
+    ks = p.D;
+    vs = p.V;
+    kmap = 0;
+    mod = 0x7fffffff;
   }
 };
 
@@ -204,7 +215,7 @@ __device__ __forceinline__ void attend(const WindowAttnParams& p, const KeySourc
 template <typename T, int MAPS, int VC>
 __device__ __forceinline__ void finish_head(const WindowAttnParams& p, int64_t m, int h, float (&a)[MAPS][VC]) {
   const int lane = threadIdx.x & 63, V = p.V;
-  float r = 1.f;
+  float r = p.out_scale;
   if constexpr (MAPS == 2) {
     float ss = 0.f;
 #pragma unroll
@@ -243,6 +254,10 @@ __global__ void __launch_bounds__(256) attn_row_kernel(WindowAttnParams p) {
   float acc[MAPS][VC] = {}, mx[MAPS], ls[MAPS];
 #pragma unroll
   for (int c = 0; c < MAPS; ++c) mx[c] = -INFINITY, ls[c] = 0.f;
+  if constexpr (MAPS == 1) {
+    if (p.pool > 0)
+      attend<T, MAPS, VC>(p, KeySource<T>(p, b, g, typename KeySource<T>::Pooled()), q, pw, 0, blocks_seen(p, ps), acc, mx, ls);
+  }
   attend<T, MAPS, VC>(p, KeySource<T>(p, b, g), q, pw, j0, ps + 1, acc, mx, ls);
 #pragma unroll
   for (int c = 0; c < MAPS; ++c)
@@ -294,7 +309,9 @@ int attn_prompt_d128_launch(const WindowAttnParams&, hipStream_t);
 // bf16 prompts on the matrix cores: 16-byte pieces of every head, head sizes the kernels are built for
 bool attn_prompt_supported(const WindowAttnParams& p) {
   return p.from_buf && p.T > 1 && p.D <= 128 && p.V <= 256 && p.D % 8 == 0 && p.V % 8 == 0 && p.ldb % 8 == 0 &&
-         p.ldy % 4 == 0 && reinterpret_cast<uintptr_t>(p.buf) % 16 == 0 && reinterpret_cast<uintptr_t>(p.y) % 16 == 0;
+         p.ldk % 8 == 0 && p.ldv % 8 == 0 && p.ldy % 4 == 0 && reinterpret_cast<uintptr_t>(p.buf) % 16 == 0 &&
+         reinterpret_cast<uintptr_t>(p.kbuf) % 16 == 0 && reinterpret_cast<uintptr_t>(p.vbuf) % 16 == 0 &&
+         reinterpret_cast<uintptr_t>(p.y) % 8 == 0;
 }
 int attn_prompt_launch(const WindowAttnParams& p, hipStream_t s) {
   if (p.D <= 32) return attn_prompt_d32_launch(p, s);

@@ -5,6 +5,9 @@
 // prepares key and value too (the group's first head also stores them in the cache), so nothing waits for
 // another launch.  With several workgroups a head the partial sums go to `part` and the last one to arrive
 // (a ticket in `tickets`, left at zero) merges them in order.
+//
+// POOL: the pooled blocks that the query sees are the first of its keys, the window's follow; the workgroup
+// that has a new key which ends a block writes the block's means (no query sees them before a later step).
 #include "window_attn.h"
 
 namespace nxd {
@@ -13,7 +16,7 @@ namespace hybrid {
 // bias, RMS norm, rotary turn of one head by one wave; out [D], rounded to the activation type
 template <typename T>
 __device__ __forceinline__ void prepare_head(const WindowAttnParams& p, const T* x, const float* bias, const float* nw,
-                                             int64_t pt, float* out) {
+                                             int64_t pt, float* out, float row_r = 0.f) {
   const int lane = threadIdx.x & 63, D = p.D, half = p.rot / 2;
   float u[2], w[2], ss = 0.f;
 #pragma unroll
@@ -23,7 +26,7 @@ __device__ __forceinline__ void prepare_head(const WindowAttnParams& p, const T*
     w[i] = d + 1 < D ? ld(x + d + 1) + (bias ? bias[d + 1] : 0.f) : 0.f;
     ss += u[i] * u[i] + w[i] * w[i];
   }
-  const float r = nw ? 1.f / sqrtf(sum64(ss) / (float)D + p.eps) : 1.f;
+  const float r = row_r > 0.f ? row_r : (nw ? 1.f / sqrtf(sum64(ss) / (float)D + p.eps) : 1.f);
 #pragma unroll
   for (int i = 0; i < 2; ++i) {
     const int pr = lane + 64 * i, d = 2 * pr;
@@ -47,6 +50,56 @@ __device__ __forceinline__ void prepare_head(const WindowAttnParams& p, const T*
       out[d + 1] = ld(&t);
     }
   }
+}
+
+// 1 / sqrt(mean of squares + eps) of n elements, by every wave for itself
+template <typename T>
+__device__ __forceinline__ float row_rms(const T* x, int n, float eps) {
+  const int lane = threadIdx.x & 63;
+  float ss = 0.f;
+  if (n % 4 == 0 && reinterpret_cast<uintptr_t>(x) % (4 * sizeof(T)) == 0) {
+#pragma unroll 4
+    for (int i = lane * 4; i < n; i += 256) {
+      const f32x4_t v = ld4(x + i);
+      ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+    }
+  } else {
+    for (int i = lane; i < n; i += 64) {
+      const float v = ld(x + i);
+      ss += v * v;
+    }
+  }
+  return 1.f / sqrtf(sum64(ss) / (float)n + eps);
+}
+
+// The means of the block that the new token (position ps, its key and value in LDS) ends, by 256 threads:
+// thread = element of the row and slice of the tokens.  red: at least 4 x 256 floats of LDS; every thread of
+// the workgroup calls it.
+template <typename T>
+__device__ __forceinline__ void pool_block(const WindowAttnParams& p, int slot, int g, int64_t ps, const float* kn, const float* vn,
+                                           float* red) {
+  const int tid = threadIdx.x, D = p.D;
+  const int width = D <= 64 ? 64 : (D <= 128 ? 128 : 256), slices = 256 / width, d = tid % width, sl = tid / width;
+  const int64_t head = (int64_t)slot * p.G + g, blk = ps / p.pool;
+  if (blk >= p.pcap) return;
+#pragma unroll
+  for (int which = 0; which < 2; ++which) {   // D == V
+    const T* src = static_cast<const T*>(which ? p.vc : p.kc) + head * p.cap * D;
+    const float* last = which ? vn : kn;
+    float a = 0.f;
+    if (d < D) {
+#pragma unroll 8
+      for (int64_t t = ps - p.pool + 1 + sl; t < ps; t += slices) a += ld(src + (t % p.cap) * D + d);
+    }
+    __syncthreads();
+    red[sl * 256 + d] = a;
+    __syncthreads();
+    if (sl == 0 && d < D) {
+      for (int i = 1; i < slices; ++i) a += red[i * 256 + d];
+      st(static_cast<T*>(which ? p.pv : p.pk) + (head * p.pcap + blk) * D + d, (a + last[d]) / (float)p.pool);
+    }
+  }
+  __syncthreads();
 }
 
 // A workgroup's sums over its keys (thread = value column): merged with the head's other workgroups if
@@ -98,7 +151,7 @@ __device__ __forceinline__ void finish(const WindowAttnParams& p, int b, int h, 
         }
     }
   }
-  float o = a[0] / l[0];
+  float o = a[0] / l[0] * (MAPS == 1 ? p.out_scale : 1.f);
   if constexpr (MAPS == 2) {
     o -= p.lam * (a[1] / l[1]);
     o *= p.out_scale / sqrtf(block_sum(tid < V ? o * o : 0.f, red) / (float)V + p.out_eps);
@@ -107,7 +160,7 @@ __device__ __forceinline__ void finish(const WindowAttnParams& p, int b, int h, 
 }
 
 // ---- any head sizes: 256 keys a workgroup, 64 a wave
-template <typename T, int MAPS>
+template <typename T, int MAPS, bool POOL>
 __global__ void __launch_bounds__(256) attn_decode_any_kernel(WindowAttnParams p) {
   __shared__ __attribute__((aligned(16))) float q[MAPS][256], kn[MAPS][256], vn[256];
   __shared__ __attribute__((aligned(16))) float pw[4][MAPS][64], acc[4][MAPS][256];
@@ -120,27 +173,36 @@ __global__ void __launch_bounds__(256) attn_decode_any_kernel(WindowAttnParams p
   const int64_t pt = ps < p.max_pos ? ps : p.max_pos - 1;
   int64_t j0 = p.window > 0 && ps - p.window + 1 > 0 ? ps - p.window + 1 : 0;
   if (ps - j0 >= p.cap) j0 = ps - p.cap + 1;            // the ring holds no more (a position beyond the cache)
-  const int n = (int)(ps - j0 + 1);                     // visible keys, the new one last
+  const int nb = POOL ? blocks_seen(p, ps) : 0;         // pooled blocks come first
+  const int n = nb + (int)(ps - j0 + 1);                // visible keys, the new one last
   const T* row = static_cast<const T*>(p.buf) + (int64_t)b * p.ldb;
   const T* kc = static_cast<const T*>(p.kc) + ((int64_t)slot * p.G + g) * MAPS * p.cap * D;
   const T* vc = static_cast<const T*>(p.vc) + ((int64_t)slot * p.G + g) * p.cap * V;
-  const int e0 = (int)(j0 % p.cap);                     // ring entry of key 0; key i is e0 + i, wrapped once
-  auto entry = [&](int i) { return e0 + i >= p.cap ? e0 + i - p.cap : e0 + i; };
+  const int e0 = (int)(j0 % p.cap);                     // ring entry of key nb; key nb + i is e0 + i, wrapped once
+  auto entry = [&](int i) { return e0 + i - nb >= p.cap ? e0 + i - nb - p.cap : e0 + i - nb; };
+  const T* pk = static_cast<const T*>(p.pk) + (POOL ? ((int64_t)slot * p.G + g) * p.pcap * D : 0);
+  const T* pv = static_cast<const T*>(p.pv) + (POOL ? ((int64_t)slot * p.G + g) * p.pcap * V : 0);
+  const bool ends = POOL && (ps + 1) % p.pool == 0;     // the new token ends a block
   const int first = sp * 256, last = min(n, first + 256) - 1;
   const bool owner = first < n && last == n - 1;        // this workgroup has the new key
 
   if (first < n) {
     const int64_t qk0 = (int64_t)p.H * MAPS * D;
+    float rq = 0.f, rk = 0.f;
+    if (POOL && p.norm_all) {
+      rq = row_rms(row, p.H * D, p.eps);
+      if (owner) rk = row_rms(row + qk0, p.G * D, p.eps);
+    }
     for (int job = w; job < (owner ? 2 * MAPS + 1 : MAPS); job += 4) {
       if (job < MAPS) {
         const int64_t c = ((int64_t)h * MAPS + job) * D;
-        prepare_head<T>(p, row + c, p.bias ? p.bias + c : nullptr, p.qn_w, pt, q[job]);
+        prepare_head<T>(p, row + c, p.bias ? p.bias + c : nullptr, p.norm_all ? p.qn_w + (int64_t)h * D : p.qn_w, pt, q[job], rq);
       } else if (job < 2 * MAPS) {
         const int m = job - MAPS;
         const int64_t c = qk0 + ((int64_t)g * MAPS + m) * D;
-        prepare_head<T>(p, row + c, p.bias ? p.bias + c : nullptr, p.kn_w, pt, kn[m]);
+        prepare_head<T>(p, row + c, p.bias ? p.bias + c : nullptr, p.norm_all ? p.kn_w + (int64_t)g * D : p.kn_w, pt, kn[m], rk);
       } else {
-        const int64_t c = qk0 + (int64_t)p.G * MAPS * D + (int64_t)g * V;
+        const int64_t c = p.v_off + (int64_t)g * V;
         for (int d = lane; d < V; d += 64) {
           T t;
           st(&t, ld(row + c + d) + (p.bias ? p.bias[c + d] : 0.f));
@@ -156,6 +218,7 @@ __global__ void __launch_bounds__(256) attn_decode_any_kernel(WindowAttnParams p
     T* vo = static_cast<T*>(p.vc) + ((int64_t)slot * p.G + g) * p.cap * V;
     for (int i = tid; i < MAPS * D; i += 256) st(ko + ((int64_t)(i / D) * p.cap + e) * D + i % D, kn[i / D][i % D]);
     for (int i = tid; i < V; i += 256) st(vo + (int64_t)e * V + i, vn[i]);
+    if (ends) pool_block<T>(p, slot, g, ps, kn[0], vn, &acc[0][0][0]);
   }
 
   // ---- this wave's 64 keys
@@ -166,13 +229,13 @@ __global__ void __launch_bounds__(256) attn_decode_any_kernel(WindowAttnParams p
   for (int i = lane; i < MAPS * V; i += 64) acc[w][i / V][i % V] = 0.f;
   if (cnt > 0) {
     const int key = k0 + min(lane, cnt - 1);
-    const int e = entry(key);
+    const int e = POOL && key < nb ? 0 : entry(key);
     // the new key's entry may hold an old key or the new one by now: its score comes from LDS
     const bool has_new = k0 + cnt == n;
 #pragma unroll
     for (int c = 0; c < MAPS; ++c) {
       float s;
-      const T* kr = kc + ((int64_t)c * p.cap + e) * D;
+      const T* kr = POOL && key < nb ? pk + (int64_t)key * D : kc + ((int64_t)c * p.cap + e) * D;
       s = 0.f;
       for (int d = 0; d < D; ++d) s += ld(kr + d) * q[c][d];
       if (has_new) {
@@ -194,7 +257,7 @@ __global__ void __launch_bounds__(256) attn_decode_any_kernel(WindowAttnParams p
       float a[MAPS] = {};
       for (int j = 0; j < cnt; ++j) {
         const int key2 = k0 + j;
-        const float x = key2 == n - 1 ? vn[d] : ld(vc + (int64_t)entry(key2) * V + d);
+        const float x = key2 == n - 1 ? vn[d] : (POOL && key2 < nb ? ld(pv + (int64_t)key2 * V + d) : ld(vc + (int64_t)entry(key2) * V + d));
 #pragma unroll
         for (int c = 0; c < MAPS; ++c) a[c] += pw[w][c][j] * x;
       }
@@ -266,7 +329,7 @@ __device__ __forceinline__ float dot8(const Raw<float>::eight& k, const float (&
 
 // R query heads of one key / value head share the keys and values a workgroup reads.  LR lanes of 8
 // elements cover D.
-template <typename T, int MAPS, int LR, int R>
+template <typename T, int MAPS, int LR, int R, bool POOL>
 __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
   constexpr int PARTS = 4 / MAPS, RPL = 64 / LR, NK = (64 / PARTS) / RPL;   // waves a map, keys a load, loads a wave
   constexpr int NJ = R * MAPS, SM = (NJ + 3) / 4;                           // rows of weights, of them a wave
@@ -283,9 +346,13 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
   const int64_t pt = ps < p.max_pos ? ps : p.max_pos - 1;
   int64_t j0 = p.window > 0 && ps - p.window + 1 > 0 ? ps - p.window + 1 : 0;
   if (ps - j0 >= p.cap) j0 = ps - p.cap + 1;            // the ring holds no more (a position beyond the cache)
-  const int n = (int)(ps - j0 + 1);                     // visible keys, the new one last
+  const int nb = POOL ? blocks_seen(p, ps) : 0;         // pooled blocks come first
+  const int n = nb + (int)(ps - j0 + 1);                // visible keys, the new one last
   const int e0 = (int)((uint32_t)j0 % (uint32_t)p.cap); // (positions are below 2^31)
-  auto entry = [&](int i) { return e0 + i >= p.cap ? e0 + i - p.cap : e0 + i; };
+  auto entry = [&](int i) { return e0 + i - nb >= p.cap ? e0 + i - nb - p.cap : e0 + i - nb; };
+  const T* pk = static_cast<const T*>(p.pk) + (POOL ? ((int64_t)slot * p.G + g) * p.pcap * D : 0);
+  const T* pv = static_cast<const T*>(p.pv) + (POOL ? ((int64_t)slot * p.G + g) * p.pcap * V : 0);
+  const bool ends = POOL && (ps + 1) % p.pool == 0;     // the new token ends a block
   const T* row = static_cast<const T*>(p.buf) + (int64_t)b * p.ldb;
   T* kc = static_cast<T*>(p.kc) + ((int64_t)slot * p.G + g) * MAPS * p.cap * D;
   T* vc = static_cast<T*>(p.vc) + ((int64_t)slot * p.G + g) * p.cap * V;
@@ -302,28 +369,38 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
   auto fetch_k = [&](int k0) {   // (keys past the end re-read the last)
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
-      const int e = entry(min(k0 + part * (64 / PARTS) + i * RPL + kl, n - 1));
-      kr[i] = *reinterpret_cast<const typename Raw<T>::eight*>(kc + ((int64_t)c * p.cap + e) * D + (dok ? dl : 0));
+      const int k = min(k0 + part * (64 / PARTS) + i * RPL + kl, n - 1);
+      const T* src = POOL && k < nb ? pk + (int64_t)k * D : kc + ((int64_t)c * p.cap + entry(k)) * D;
+      kr[i] = *reinterpret_cast<const typename Raw<T>::eight*>(src + (dok ? dl : 0));
     }
   };
   auto fetch_v = [&](int k0) {
 #pragma unroll
     for (int i = 0; i < 16; ++i)
-      if (i * kpp < 16) vr[i] = *reinterpret_cast<const raw_t*>(vc + (int64_t)entry(min(k0 + 16 * w + i * kpp + ks, n - 1)) * V + col);
+      if (i * kpp < 16) {
+        const int k = min(k0 + 16 * w + i * kpp + ks, n - 1);
+        vr[i] = *reinterpret_cast<const raw_t*>((POOL && k < nb ? pv + (int64_t)k * V : vc + (int64_t)entry(k) * V) + col);
+      }
   };
   if (first < n) {
     fetch_k(first);
     fetch_v(first);
     const int64_t qk0 = (int64_t)p.H * MAPS * D;
+    float rq = 0.f, rk = 0.f;
+    if (POOL && p.norm_all) {
+      rq = row_rms(row, p.H * D, p.eps);
+      if (owner) rk = row_rms(row + qk0, p.G * D, p.eps);
+    }
     for (int job = w; job < (owner ? NJ + MAPS + 1 : NJ); job += 4) {
       if (job < NJ) {
         const int64_t o = ((int64_t)h0 * MAPS + job) * D;
-        prepare_head<T>(p, row + o, p.bias ? p.bias + o : nullptr, p.qn_w, pt, q[job]);
+        prepare_head<T>(p, row + o, p.bias ? p.bias + o : nullptr, POOL && p.norm_all ? p.qn_w + o : p.qn_w, pt, q[job], rq);
       } else if (job < NJ + MAPS) {
         const int64_t o = qk0 + ((int64_t)g * MAPS + job - NJ) * D;
-        prepare_head<T>(p, row + o, p.bias ? p.bias + o : nullptr, p.kn_w, pt, kn[job - NJ]);
+        prepare_head<T>(p, row + o, p.bias ? p.bias + o : nullptr, POOL && p.norm_all ? p.kn_w + (int64_t)g * D : p.kn_w, pt,
+                        kn[job - NJ], rk);
       } else {
-        const int64_t o = qk0 + (int64_t)p.G * MAPS * D + (int64_t)g * V;
+        const int64_t o = p.v_off + (int64_t)g * V;
         for (int d = lane; d < V; d += 64) {
           T t;
           st(&t, ld(row + o + d) + (p.bias ? p.bias[o + d] : 0.f));
@@ -337,6 +414,7 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
     const int e = entry(n - 1);
     for (int i = tid; i < MAPS * D; i += 256) st(kc + ((int64_t)(i / D) * p.cap + e) * D + i % D, kn[i / D][i % D]);
     for (int i = tid; i < V; i += 256) st(vc + (int64_t)e * V + i, vn[i]);
+    if (ends) pool_block<T>(p, slot, g, ps, kn[0], vn, &acc[0][0][0]);
   }
 
   float q8[R][8], snew[R];   // this lane's piece of the queries; the new key's scores
@@ -485,7 +563,7 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
       }
     }
   }
-  float o[4], ss = 0.f, sc_out = 1.f;
+  float o[4], ss = 0.f, sc_out = p.out_scale;
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     o[i] = a[0][i] / l[0];
@@ -499,21 +577,21 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(WindowAttnParams p) {
     if (lane + 64 * i < V) st(y + lane + 64 * i, o[i] * sc_out);
 }
 
-template <typename T, int MAPS, int R>
+template <typename T, int MAPS, int R, bool POOL>
 static void launch_decode(const WindowAttnParams& p, hipStream_t s) {
   const dim3 grid((unsigned)p.splits, (unsigned)(p.H / R), (unsigned)p.B);
-  if (p.D <= 32) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 4, R>), grid, dim3(256), 0, s, p);
-  else if (p.D <= 64) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 8, R>), grid, dim3(256), 0, s, p);
-  else hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 16, R>), grid, dim3(256), 0, s, p);
+  if (p.D <= 32) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 4, R, POOL>), grid, dim3(256), 0, s, p);
+  else if (p.D <= 64) hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 8, R, POOL>), grid, dim3(256), 0, s, p);
+  else hipLaunchKernelGGL((attn_decode_kernel<T, MAPS, 16, R, POOL>), grid, dim3(256), 0, s, p);
 }
 
-template <typename T, int MAPS>
+template <typename T, int MAPS, bool POOL>
 static int run_decode(const WindowAttnParams& p, hipStream_t s) {
   if (p.tiles == 0)
-    hipLaunchKernelGGL((attn_decode_any_kernel<T, MAPS>), dim3((unsigned)p.splits, (unsigned)p.H, (unsigned)p.B), dim3(256), 0, s, p);
-  else if (p.share == 4) launch_decode<T, MAPS, 4>(p, s);
-  else if (p.share == 2) launch_decode<T, MAPS, 2>(p, s);
-  else launch_decode<T, MAPS, 1>(p, s);
+    hipLaunchKernelGGL((attn_decode_any_kernel<T, MAPS, POOL>), dim3((unsigned)p.splits, (unsigned)p.H, (unsigned)p.B), dim3(256), 0, s, p);
+  else if (p.share == 4) launch_decode<T, MAPS, 4, POOL>(p, s);
+  else if (p.share == 2) launch_decode<T, MAPS, 2, POOL>(p, s);
+  else launch_decode<T, MAPS, 1, POOL>(p, s);
   return hipGetLastError() == hipSuccess ? 0 : 1;
 }
 
@@ -543,8 +621,10 @@ void attn_decode_plan(WindowAttnParams& p, int64_t seen) {
 }
 
 int attn_decode_launch(bool f32, const WindowAttnParams& p, hipStream_t s) {
-  if (p.maps == 2) return f32 ? hybrid::run_decode<float, 2>(p, s) : hybrid::run_decode<uint16_t, 2>(p, s);
-  return f32 ? hybrid::run_decode<float, 1>(p, s) : hybrid::run_decode<uint16_t, 1>(p, s);
+  using namespace hybrid;
+  if (p.pool > 0) return p.maps != 1 ? -1 : (f32 ? run_decode<float, 1, true>(p, s) : run_decode<uint16_t, 1, true>(p, s));
+  if (p.maps == 2) return f32 ? run_decode<float, 2, false>(p, s) : run_decode<uint16_t, 2, false>(p, s);
+  return f32 ? run_decode<float, 1, false>(p, s) : run_decode<uint16_t, 1, false>(p, s);
 }
 
 }  // namespace nxd

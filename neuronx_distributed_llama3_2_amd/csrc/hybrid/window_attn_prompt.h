@@ -12,6 +12,8 @@
 //     lane-local plus one cross-half exchange and P^T is the B operand of O^T += V^T P^T directly;
 //   * with a score cap of at most 40 the maximum is known in advance, exp(cap tanh(x) - cap) is
 //     computed as exp(-2 cap / (exp(2 x) + 1)) and there is no running maximum to follow;
+//   * POOL (one map): the tiles of the pooled blocks that some row sees come first, read from the pooled
+//     cache, in the same softmax;
 //   * at the end the second map's waves hand their rows to the first's through LDS: the difference, its
 //     RMS over the head and the output scale are applied there in fp32.
 #pragma once
@@ -43,7 +45,7 @@ __device__ __forceinline__ void tr_wait(short4_t (&v)[N]) {
 
 // KS 16-wide steps of the (padded) query size, NDB 32-wide blocks of the (padded) value size; FIXED: the
 // scores' maximum is the cap (0 < softcap <= 40), else a running maximum is kept
-template <int KS, int NDB, int MAPS, bool FIXED>
+template <int KS, int NDB, int MAPS, bool FIXED, bool POOL = false>
 __global__ void __launch_bounds__(256 * MAPS, 2) attn_prompt_kernel(WindowAttnParams p) {
   constexpr int BN = 64, DP = KS * 16, VP = NDB * 32, NT = 256 * MAPS;
   constexpr int KROW = DP * 2 + 16, VROW = VP * 2 + 16;         // bytes of an LDS row
@@ -67,8 +69,11 @@ __global__ void __launch_bounds__(256 * MAPS, 2) attn_prompt_kernel(WindowAttnPa
   }
   const uint16_t* base = static_cast<const uint16_t*>(p.buf) + (int64_t)b * p.T * p.ldb;
   const uint16_t* qrow = base + (int64_t)min(my_q, p.T - 1) * p.ldb + ((int64_t)h * MAPS + c) * p.D;
-  const uint16_t* kb = base + (int64_t)(p.H + g) * MAPS * p.D;
-  const uint16_t* vb = base + (int64_t)(p.H + p.G) * MAPS * p.D + (int64_t)g * p.V;
+  const uint16_t* kb = static_cast<const uint16_t*>(p.kbuf) + (int64_t)b * p.T * p.ldk + (int64_t)g * MAPS * p.D;
+  const uint16_t* vb = static_cast<const uint16_t*>(p.vbuf) + (int64_t)b * p.T * p.ldv + (int64_t)g * p.V;
+  const int64_t phead = POOL ? (int64_t)slot_of(p.slots, b, p.nslots) * p.G + g : 0;
+  const uint16_t* pkb = static_cast<const uint16_t*>(p.pk) + phead * p.pcap * p.D;
+  const uint16_t* pvb = static_cast<const uint16_t*>(p.pv) + phead * p.pcap * p.V;
 
   bf16x8_t qf[KS];
 #pragma unroll
@@ -81,24 +86,30 @@ __global__ void __launch_bounds__(256 * MAPS, 2) attn_prompt_kernel(WindowAttnPa
 
   const int kend = min(len, qb0 + 128);
   const int kbeg = p.window > 0 ? max(0, qb0 - p.window + 1) / BN * BN : 0;
+  const int pend = POOL ? blocks_seen(p, kend - 1) : 0;                    // pooled blocks some row of the workgroup sees
+  const int my_blocks = POOL ? blocks_seen(p, my_q) : 0;
+  const int first_blocks = POOL ? blocks_seen(p, q0) : 0, last_blocks = POOL ? blocks_seen(p, q0 + 31) : 0;   // of the wave
   const int wave_lo = p.window > 0 ? q0 - p.window + 1 : 0, wave_hi = q0 + 31;   // keys some row may see
 
   // staging registers of the next tile
   u32x4_t kst[NK], vst[NV];
-  auto fetch = [&](int k0) {
+  auto fetch = [&](int k0, bool pooled) {
+    const uint16_t *ksrc = POOL && pooled ? pkb : kb, *vsrc = POOL && pooled ? pvb : vb;
+    const int64_t lk = POOL && pooled ? p.D : p.ldk, lv = POOL && pooled ? p.V : p.ldv;
+    const int last = (POOL && pooled ? pend : len) - 1;
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
       const int e = tid + NT * i, ch = e % KCH, row = (e / KCH) % BN, m = e / (KCH * BN);
       kst[i] = u32x4_t{0u, 0u, 0u, 0u};
       if (m < MAPS && ch * 8 < p.D)
-        kst[i] = *reinterpret_cast<const u32x4_t*>(kb + (int64_t)min(k0 + row, len - 1) * p.ldb + m * p.D + ch * 8);
+        kst[i] = *reinterpret_cast<const u32x4_t*>(ksrc + (int64_t)min(k0 + row, last) * lk + m * p.D + ch * 8);
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int e = tid + NT * i, ch = e % VCH, row = e / VCH;
       vst[i] = u32x4_t{0u, 0u, 0u, 0u};
       if (row < BN && ch * 8 < p.V)
-        vst[i] = *reinterpret_cast<const u32x4_t*>(vb + (int64_t)min(k0 + row, len - 1) * p.ldb + ch * 8);
+        vst[i] = *reinterpret_cast<const u32x4_t*>(vsrc + (int64_t)min(k0 + row, last) * lv + ch * 8);
     }
   };
   auto stash = [&](int buf) {
@@ -129,17 +140,22 @@ __global__ void __launch_bounds__(256 * MAPS, 2) attn_prompt_kernel(WindowAttnPa
   const int gi = lane & 15, tq = gi >> 2, tp = gi & 3, grp = lane >> 4;
   const uint32_t vlane = lds_addr(smem) + MAPS * KTILE + (uint32_t)((4 * hh + tq) * VROW + (16 * (grp & 1) + 4 * tp) * 2);
 
-  fetch(kbeg);
+  bool pooled = pend > 0;   // tiles of pooled blocks first
+  int k0 = pooled ? 0 : kbeg;
+  fetch(k0, pooled);
   stash(0);
   __syncthreads();
   int buf = 0;
-  for (int k0 = kbeg; k0 < kend; k0 += BN, buf ^= 1) {
-    const bool more = k0 + BN < kend;
-    if (more) fetch(k0 + BN);
-    if (k0 <= wave_hi && k0 + BN - 1 >= wave_lo) {
+  for (;; buf ^= 1) {
+    const bool nextp = POOL && pooled && k0 + BN < pend;
+    const int knext = POOL && pooled && !nextp ? kbeg : k0 + BN;
+    const bool more = nextp || knext < kend;
+    if (more) fetch(knext, nextp);
+    if (POOL && pooled ? k0 < last_blocks : (k0 <= wave_hi && k0 + BN - 1 >= wave_lo)) {
       const char* kl = smem + buf * BUF + c * KTILE;
       const uint32_t va = vlane + buf * BUF;
-      const bool edge = k0 + BN - 1 > q0 || (p.window > 0 && k0 < q0 + 31 - p.window + 1);
+      const bool edge = POOL && pooled ? k0 + BN > first_blocks
+                                       : k0 + BN - 1 > q0 || (p.window > 0 && k0 < q0 + 31 - p.window + 1);
       f32x16_t s[2];
       s[0] = f32x16_t{0};
       s[1] = f32x16_t{0};
@@ -162,8 +178,8 @@ __global__ void __launch_bounds__(256 * MAPS, 2) attn_prompt_kernel(WindowAttnPa
       };
       issue(0, vt[0]);
       // element e of s[j] is key k0 + 32 j + (e & 3) + 8 (e >> 2) + 4 hh
-      const int hi = my_q - k0 - 4 * hh;                                              // seen: offset <= hi
-      const int lo = p.window > 0 ? my_q - p.window + 1 - k0 - 4 * hh : -0x40000000;  //       offset >= lo
+      const int hi = (POOL && pooled ? my_blocks - 1 : my_q) - k0 - 4 * hh;           // seen: offset <= hi
+      const int lo = p.window > 0 && !(POOL && pooled) ? my_q - p.window + 1 - k0 - 4 * hh : -0x40000000;  // and >= lo
       float sum = 0.f;
       bf16x8_t pf[4];
       if constexpr (FIXED) {
@@ -249,16 +265,20 @@ __global__ void __launch_bounds__(256 * MAPS, 2) attn_prompt_kernel(WindowAttnPa
         }
       }
     }
-    if (more) stash(buf ^ 1);
+    if (!more) break;
+    stash(buf ^ 1);
     lds_barrier();
+    k0 = knext;
+    pooled = nextp;
   }
 
   const bool live = my_q < len;
   const float inv = live && ls > 0.f ? 1.f / ls : 0.f;
 #pragma unroll
   for (int db = 0; db < NDB; ++db) acc[db] *= inv;
-  float sc = 1.f;
+  float sc = p.out_scale;
   if constexpr (MAPS == 2) {
+    __syncthreads();   // (the tiles' last readers are done)
     float* xch = reinterpret_cast<float*>(smem) + w * (NDB * 16 * 64) + lane;   // [wave][element][lane]
     if (c == 1) {
 #pragma unroll
@@ -291,18 +311,25 @@ __global__ void __launch_bounds__(256 * MAPS, 2) attn_prompt_kernel(WindowAttnPa
     }
 }
 
-template <int KS, int NDB, int MAPS, bool FIXED>
+template <int KS, int NDB, int MAPS, bool FIXED, bool POOL = false>
 int attn_prompt_run(const WindowAttnParams& p, hipStream_t s) {
   constexpr size_t tiles = 2 * (size_t)64 * (MAPS * (KS * 32 + 16) + NDB * 64 + 16);
   constexpr size_t xch = MAPS == 2 ? (size_t)4 * NDB * 16 * 64 * 4 : 0;
   constexpr size_t lds = tiles > xch ? tiles : xch;
   static_assert(lds <= 160 * 1024, "LDS of a compute unit");
-  static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_prompt_kernel<KS, NDB, MAPS, FIXED>),
+  static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_prompt_kernel<KS, NDB, MAPS, FIXED, POOL>),
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
   if (attr != hipSuccess) return 2;
   const int64_t grid = (int64_t)((p.T + 127) / 128) * p.B * p.H;
-  hipLaunchKernelGGL((attn_prompt_kernel<KS, NDB, MAPS, FIXED>), dim3((unsigned)grid), dim3(256 * MAPS), lds, s, p);
+  hipLaunchKernelGGL((attn_prompt_kernel<KS, NDB, MAPS, FIXED, POOL>), dim3((unsigned)grid), dim3(256 * MAPS), lds, s, p);
   return hipGetLastError() == hipSuccess ? 0 : 1;
+}
+
+// pooled blocks: values are as wide as keys
+template <int KS>
+int attn_prompt_pooled(const WindowAttnParams& p, hipStream_t s) {
+  if (p.maps != 1 || p.V > KS * 16) return -1;
+  return attn_prompt_run<KS, (KS * 16 + 31) / 32, 1, false, true>(p, s);
 }
 
 template <int KS, int MAPS, bool FIXED>

@@ -3,6 +3,7 @@
 
 namespace nxd {
 int attn_prompt_d128_launch(const WindowAttnParams& p, hipStream_t s) {
+  if (p.pool > 0) return hybrid::attn_prompt_pooled<8>(p, s);
   if (p.maps == 1) return hybrid::attn_prompt_by_v<8, 1, false>(p, s);
   return p.softcap > 0.f && p.softcap <= 40.f ? hybrid::attn_prompt_by_v<8, 2, true>(p, s)
                                               : hybrid::attn_prompt_by_v<8, 2, false>(p, s);

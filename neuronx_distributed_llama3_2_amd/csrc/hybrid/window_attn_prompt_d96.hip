@@ -3,6 +3,7 @@
 
 namespace nxd {
 int attn_prompt_d96_launch(const WindowAttnParams& p, hipStream_t s) {
+  if (p.pool > 0) return hybrid::attn_prompt_pooled<6>(p, s);
   if (p.maps == 1) return hybrid::attn_prompt_by_v<6, 1, false>(p, s);
   return p.softcap > 0.f && p.softcap <= 40.f ? hybrid::attn_prompt_by_v<6, 2, true>(p, s)
                                               : hybrid::attn_prompt_by_v<6, 2, false>(p, s);
