@@ -11,7 +11,7 @@ on a side stream), global batch 32 by default (the 1F1B bubble is (P-1)/(M+P-1) 
     python -m torch.distributed.run --nnodes=1 --nproc-per-node N --master-addr 127.0.0.1 \
         --master-port P bench.py --gpus N --steps K --warmup W
 
-`--serve golitar | llama` measures serving instead (prefill and decode tokens/s of one GPU).
+`--serve bezurax | golitar | llama` measures serving instead (prefill and decode tokens/s of one GPU).
 
 Without a launcher (no WORLD_SIZE in the environment) and N > 1, bench.py starts the N rank
 processes itself (child processes, before any HIP call) and waits for them.
@@ -75,7 +75,7 @@ def parse():
     ap.add_argument("--no-sp", action="store_true")
     ap.add_argument("--ckpt", default=None, help="activation checkpointing: None | full | selective")
     ap.add_argument("--lr", type=float, default=1e-5, help="AdamW learning rate (tests raise it so the loss moves)")
-    ap.add_argument("--serve", choices=["golitar", "llama"], default=None,
+    ap.add_argument("--serve", choices=["bezurax", "golitar", "llama"], default=None,
                     help="instead of the training step: prefill and decode throughput of this model family at layer "
                          "sizes of a real model, one GPU (inference/serve_bench.py; --steps timed repetitions)")
     ap.add_argument("--serve-size", action="append", choices=["2k", "4k"], default=None, help="default: both")

@@ -4,7 +4,9 @@ context encoding and token generation through the application's own captured gra
 
 The Golitar sizes are built to equal the Llama ones: the same width, depth and vocabulary, the same
 parameters in the feed-forward (two matrices instead of three), three gated-delta layers to one
-differential-attention layer."""
+differential-attention layer.  The Bezurax sizes have the same width, depth and vocabulary, heads as
+Golitar's in both mixers of every layer, and the feed-forward parameters that a token uses equal to
+Llama's (half of them in the shared expert, half in 4 of 32 routed ones)."""
 
 from __future__ import annotations
 
@@ -15,7 +17,7 @@ import torch
 
 from .config import InferenceConfig
 
-FAMILIES = ("golitar", "llama")
+FAMILIES = ("bezurax", "golitar", "llama")
 SIZES = ("2k", "4k")
 # (sequences, tokens) of a prompt batch; sequences of a decode batch
 PREFILL = [(1, 8192), (4, 2048), (1, 2048)]
@@ -37,6 +39,18 @@ def golitar_config(size: str) -> dict:
             "width": width, "vocab": 128256, "streams": 4, "norm": {"eps": 1e-5}, "logit_softcap": 30.0}
 
 
+def bezurax_config(size: str) -> dict:
+    """config.json of the benchmark model of this size."""
+    width, layers, ff, heads, kv, rank = {"2k": (2048, 16, 1024, 16, 4, 64), "4k": (4096, 8, 1792, 32, 8, 96)}[size]
+    mlp = {"kind": "moe", "expert": {"ff": ff, "limit": 7.0}, "shared": {"ff": 4 * ff, "limit": 7.0},
+           "router": {"experts": 32, "top": 4, "groups": {"count": 4, "keep": 2}, "scale": 2.5}}
+    mixer = {"left": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                      "mask": {"size": 1024, "pool": 16}},
+             "left_scale": 0.7, "right": {"heads": heads, "dim": 128, "rank": rank}, "right_scale": 0.7}
+    return {"architecture": "Bezurax", "layers": [{"type": "parallel", "mixer": mixer, "mlp": mlp}] * layers,
+            "width": width, "vocab": 128256, "norm": {"eps": 1e-5, "groups": 8}, "logit_scale": 1.0}
+
+
 def build(family: str, size: str, batch: int, max_len: int, context: int):
     icfg = InferenceConfig(batch_size=batch, seq_len=max_len, max_context_length=context, decode_graph_steps=8)
     torch.manual_seed(0)
@@ -45,6 +59,11 @@ def build(family: str, size: str, batch: int, max_len: int, context: int):
         from .golitar import GolitarForCausalLMInference
 
         return GolitarForCausalLMInference(GolitarConfig(golitar_config(size)), icfg)
+    if family == "bezurax":
+        from ..models.bezurax import BezuraxConfig
+        from .bezurax import BezuraxForCausalLMInference
+
+        return BezuraxForCausalLMInference(BezuraxConfig(bezurax_config(size)), icfg)
     from ..models.llama.modeling_llama import llama_config
     from .generation import LlamaForCausalLMInference
 

@@ -376,6 +376,20 @@ def test_pooled_attention(where, H, G, D, window, pool):
         assert all(bool((a.cache[n][0] == 7.0).all()) for n in ("k", "v", "pk", "pv"))   # nobody's slot
 
 
+def one_key_matches(a, at):
+    """Only token `at`'s key has the component that all queries consist of: every other score is exactly zero,
+    in 16 bits as well, whatever the values are."""
+    H, G, D = a.sz.as_list()
+    a.qn.fill_(1.0)
+    a.kn.fill_(1.0)
+    a.buf_o[0, :, :H * D] = 0
+    a.buf_o[0, :, :H * D:D] = 1.0
+    a.buf_o[0, :, H * D::D] = 0
+    a.buf_o[0, at, H * D:(H + G) * D] = 0
+    a.buf_o[0, at, H * D:(H + G) * D:D] = 3.0
+    a.round()
+
+
 @pytest.mark.parametrize("where", WHERE)
 @pytest.mark.parametrize("window,pool", [(1, 2), (5, 5), (63, 8), (64, 7), (65, 1), (30, 50)])
 def test_window_and_block_edges(where, window, pool):
@@ -383,15 +397,8 @@ def test_window_and_block_edges(where, window, pool):
     until its block has left, then through the block's mean.  Prompts, portions and decoding; a window or a
     block one token off would change the output completely."""
     T, D, at = 190, 16, 41
-    a = Attn(where, 1, T, 1, 1, D, window, pool, scale=3.0 * max(1, pool) / 4, seed=5)
-    a.qn.fill_(1.0)
-    a.kn.fill_(1.0)
-    probe = rnd(D, seed=50)
-    a.buf_o[0, :, :D] = probe + rnd(T, D, seed=51, std=0.05)
-    others = a.buf_o[0, :, D:2 * D]
-    others -= (others @ probe)[:, None] * probe / (probe @ probe)   # at right angles to every query
-    a.buf_o[0, at, D:2 * D] = probe * 3
-    a.round()
+    a = Attn(where, 1, T, 1, 1, D, window, pool, scale=0.75 * pool, seed=5)
+    one_key_matches(a, at)
     want, tol = a.oracle(0, T), a.tol()
     edge = at + window                                           # the first query that has lost the token
     seen = (at // pool + 1) * pool - 1 + window                  # the first that sees its block
@@ -432,19 +439,11 @@ def test_first_tokens_see_only_what_is_there(where):
 def test_far_block_in_long_decoding(where):
     """The only matching key is hundreds of tokens back, in one of very many blocks."""
     T, D = 700, 24
-    a = Attn(where, 1, T, 2, 1, D, 10, 4, scale=9.0, seed=7)
-    a.qn.fill_(1.0)
-    a.kn.fill_(1.0)
-    probe = rnd(2 * D, seed=50)
-    probe[D:] = probe[:D]
-    a.buf_o[0, :, :2 * D] = probe
-    k = a.buf_o[0, :, 2 * D:3 * D]
-    k -= (k @ probe[:D])[:, None] * probe[:D] / (probe[:D] @ probe[:D])
-    a.buf_o[0, 13, 2 * D:3 * D] = probe[:D] * 4
-    a.round()
+    a = Attn(where, 1, T, 2, 1, D, 10, 4, scale=2.5, seed=7)
+    one_key_matches(a, 13)
     want = a.oracle(0, T)
     away = a.buf_o.clone()
-    a.buf_o[0, 13, 2 * D:3 * D] *= -1
+    a.buf_o[0, 13] *= -1
     assert rel_err(a.oracle(0, T)[-3:], want[-3:]) > 0.2   # the far key is what decides
     a.buf_o = away
     a.step(0, T - 4, True)
