@@ -423,7 +423,7 @@ void pooled_decode(Tensor buf, std::vector<int64_t> sizes, Tensor qn_w, Tensor k
 // y = epi(x w^T), 1..4 rows of bf16; x bf16 [M, K], or u fp32 [M, K] normalised on the way in.  epi: 0 bf16,
 // 1 squared ReLU, 2 fp32 with cap, 3 into the streams (y unused, `un` receives the next sublayer's input)
 void gemv_hyper(int64_t epi, Opt x, Opt u, Opt norm_w, double eps, Tensor w, Opt y, double cap, Opt streams, Opt bias, Opt mix,
-                Opt write, Opt read, Opt un) {
+                Opt write, Opt read, Opt un, double alpha) {
   nxd::GemvHyperParams p{};
   TORCH_CHECK(epi >= 0 && epi <= 3, "gemv_hyper: epi 0..3");
   TORCH_CHECK(x.has_value() != u.has_value() && u.has_value() == norm_w.has_value(), "gemv_hyper: x, or u with norm_w");
@@ -442,6 +442,7 @@ void gemv_hyper(int64_t epi, Opt x, Opt u, Opt norm_w, double eps, Tensor w, Opt
   p.ldw = w.stride(0);
   p.eps = (float)eps;
   p.cap = (float)cap;
+  p.alpha = (float)alpha;
   if (x.has_value()) {
     TORCH_CHECK(x->scalar_type() == at::kBFloat16 && x->stride(0) % 8 == 0, "gemv_hyper: x bf16, rows 16-byte aligned");
     p.x = static_cast<const uint16_t*>(x->data_ptr());
@@ -502,5 +503,5 @@ PYBIND11_MODULE(_hybrid, m) {
   m.def("gemv_hyper", &gemv_hyper, py::arg("epi"), py::arg("x") = py::none(), py::arg("u") = py::none(),
         py::arg("norm_w") = py::none(), py::arg("eps") = 0.0, py::arg("w"), py::arg("y") = py::none(), py::arg("cap") = 0.0,
         py::arg("streams") = py::none(), py::arg("bias") = py::none(), py::arg("mix") = py::none(),
-        py::arg("write") = py::none(), py::arg("read") = py::none(), py::arg("un") = py::none());
+        py::arg("write") = py::none(), py::arg("read") = py::none(), py::arg("un") = py::none(), py::arg("alpha") = 1.0);
 }

@@ -14,6 +14,7 @@ int moe_route_chunk();
 int moe_route_launch(const RouterParams&, hipStream_t);
 int clamped_glu_launch(bool, const GluParams&, bool, hipStream_t);
 int gather_rows_launch(const void*, const int*, void*, int64_t, int64_t, int64_t, hipStream_t);
+int experts_few_launch(const RouterParams&, const ExpertFewParams&, hipStream_t);
 int expert_rows_launch(bool, const ExpertRowsParams&, hipStream_t);
 int grouped_gemm_launch(int, const void*, const void*, void*, const int*, int, int, int, int, int, hipStream_t);
 int grouped_rowgemm_launch(int, const void*, const void*, void*, const int*, int, int, int, int, hipStream_t);
@@ -69,11 +70,16 @@ void residual_norms(Tensor x, Opt embed, Opt ids, std::vector<Tensor> adds, Opt 
     act(*pairs, "pairs");
     TORCH_CHECK(pairs->dim() == 2 && pairs->is_contiguous() && pairs->size(1) == p.W && pairs->size(0) >= 1 && pairs->size(0) < (1LL << 31),
                 "residual_norms: pairs [P, W]");
-    TORCH_CHECK(inverse.has_value() && inverse->dim() == 2 && inverse->size(0) == p.M, "residual_norms: inverse [M, k]");
     p.pairs = pairs->data_ptr();
     p.npairs = (int)pairs->size(0);
-    p.k = (int)inverse->size(1);
-    p.inverse = i32_opt(inverse, p.M * p.k, "inverse");
+    if (inverse.has_value()) {
+      TORCH_CHECK(inverse->dim() == 2 && inverse->size(0) == p.M, "residual_norms: inverse [M, k]");
+      p.k = (int)inverse->size(1);
+      p.inverse = i32_opt(inverse, p.M * p.k, "inverse");
+    } else {   // row m k + j belongs to row m
+      TORCH_CHECK(p.npairs % p.M == 0, "residual_norms: as many pairs for every row");
+      p.k = (int)(p.npairs / p.M);
+    }
   }
   for (size_t i = 0; i < norms.size(); ++i) {
     act(hs[i], "h");
@@ -135,31 +141,37 @@ void channel_delta(Tensor proj, int64_t B, int64_t T, std::vector<int64_t> sizes
   p.nch = (int)((T + C - 1) / C);
   TORCH_CHECK(p.nch <= 65535, "channel_delta: tokens of one step");
   const int64_t cells = B * p.nch * p.H;
-  Tensor buf = at::empty({cells * (2 * C * p.DP + 3 * p.DP * p.DP)}, proj.options().dtype(at::kFloat));
-  p.cq = buf.data_ptr<float>();
-  p.co = p.cq + cells * C * p.DP;
-  p.ct = p.co + cells * C * p.DP;
-  p.cm = p.ct + cells * p.DP * p.DP;
-  p.cs = p.cm + cells * p.DP * p.DP;
+  const int64_t piece = cells * C * p.DP;
+  Tensor buf = at::empty({6 * piece + cells * p.DP * (p.DP + 1)}, proj.options().dtype(at::kFloat));
+  float* at = buf.data_ptr<float>();
+  for (float** q : {&p.cq, &p.co, &p.cw, &p.cy, &p.cb, &p.ck}) *q = at, at += piece;
+  p.cs = at;
+  p.ce = at + cells * p.DP * p.DP;
   check_rc(nxd::channel_delta_chunk_launch(f32, p, cur_stream()), "channel_delta_chunk");
 }
 
 int* i32_new(const Tensor& t, int64_t numel, const char* n) { return const_cast<int*>(i32_opt(t, numel, n)); }
 
-// rule (experts, top, groups, keep)
-nxd::RouterParams router_params(const Tensor& logits, const std::vector<int64_t>& rule, double scale) {
+// rule (experts, top, groups, keep): the rule alone
+nxd::RouterParams rule_params(const std::vector<int64_t>& rule, double scale, int64_t M) {
   TORCH_CHECK(rule.size() == 4, "router: rule (experts, top, groups, keep)");
-  TORCH_CHECK(logits.is_cuda() && logits.dim() == 2 && logits.scalar_type() == at::kFloat && logits.stride(1) == 1, "router: fp32 logits [M, E]");
   nxd::RouterParams p{};
-  p.M = logits.size(0);
+  p.M = M;
   p.E = (int)rule[0];
   p.top = (int)rule[1];
   p.groups = (int)rule[2];
   p.keep = (int)rule[3];
-  TORCH_CHECK(p.M >= 1 && p.E >= 1 && p.E <= 1024 && logits.size(1) >= p.E, "router: up to 1024 experts");
+  TORCH_CHECK(p.M >= 1 && p.E >= 1 && p.E <= 1024, "router: up to 1024 experts");
   TORCH_CHECK(p.groups >= 1 && p.E % p.groups == 0 && p.keep >= 1 && p.keep <= p.groups, "router: equal groups");
   TORCH_CHECK(p.top >= 1 && p.top <= 64 && p.top <= p.keep * (p.E / p.groups) && p.M * p.top < (1LL << 31), "router: up to 64 choices");
   p.scale = (float)scale;
+  return p;
+}
+
+nxd::RouterParams router_params(const Tensor& logits, const std::vector<int64_t>& rule, double scale) {
+  TORCH_CHECK(logits.is_cuda() && logits.dim() == 2 && logits.scalar_type() == at::kFloat && logits.stride(1) == 1, "router: fp32 logits [M, E]");
+  auto p = rule_params(rule, scale, logits.size(0));
+  TORCH_CHECK(logits.size(1) >= p.E, "router: logits of every expert");
   p.logits = logits.data_ptr<float>();
   p.ldl = logits.stride(0);
   return p;
@@ -252,6 +264,51 @@ void expert_rows(Tensor x, Tensor w, Tensor offs, Opt token, Tensor y) {
   check_rc(nxd::expert_rows_launch(f32, p, cur_stream()), "expert_rows");
 }
 
+// y [M (top + shared), W]: outputs of a token's experts, weighted, then its shared expert's
+void experts_few(Tensor h, Tensor router, std::vector<int64_t> rule, double scale, Tensor up, Tensor down, double limit, Opt sup,
+                 Opt sdown, double slimit, Tensor y) {
+  auto bf = [](const Tensor& t, int64_t d, const char* n) {
+    TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kBFloat16 && t.dim() == d && t.is_contiguous(), "experts_few: ", n, ": contiguous bf16");
+    check_align(t, n);
+    return static_cast<uint16_t*>(t.data_ptr());
+  };
+  nxd::ExpertFewParams p{};
+  p.h = bf(h, 2, "h");
+  const auto r = rule_params(rule, scale, h.size(0));
+  p.M = (int)h.size(0);
+  p.W = (int)h.size(1);
+  p.ldh = h.stride(0);
+  p.E = r.E;
+  p.top = r.top;
+  p.router = bf(router, 2, "router");
+  p.up = bf(up, 3, "up");
+  p.down = bf(down, 3, "down");
+  p.F = (int)down.size(2);
+  p.shared = sup.has_value() ? 1 : 0;
+  TORCH_CHECK(sup.has_value() == sdown.has_value(), "experts_few: both matrices of the shared expert");
+  if (p.shared) {
+    p.sup = bf(*sup, 2, "shared up");
+    p.sdown = bf(*sdown, 2, "shared down");
+    p.FS = (int)sdown->size(1);
+    TORCH_CHECK(sup->size(0) == 2 * p.FS && sup->size(1) == p.W && sdown->size(0) == p.W, "experts_few: shared expert's shapes");
+  }
+  TORCH_CHECK(p.M <= 64 && p.W % 8 == 0 && p.F % 8 == 0 && p.FS % 8 == 0 && p.F >= 8 && p.W >= 8, "experts_few: up to 64 tokens, sizes multiples of 8");
+  TORCH_CHECK(router.size(0) >= p.E + p.shared && router.size(1) == p.W, "experts_few: router [>= E + shared, W]");
+  TORCH_CHECK(up.size(0) == p.E && up.size(1) == 2 * p.F && up.size(2) == p.W && down.size(0) == p.E && down.size(1) == p.W, "experts_few: experts' shapes");
+  const int64_t slots = p.top + p.shared;
+  p.y = bf(y, 2, "y");
+  TORCH_CHECK(y.size(0) == p.M * slots && y.size(1) == p.W, "experts_few: y [M (top + shared), W]");
+  p.limit = (float)limit;
+  p.slimit = (float)slimit;
+  Tensor index = at::empty({p.M, p.top}, h.options().dtype(at::kInt)), score = at::empty({p.M, slots}, h.options().dtype(at::kFloat));
+  Tensor a = at::empty({(int64_t)p.M * p.top * p.F + (int64_t)p.M * p.FS}, h.options());
+  p.index = index.data_ptr<int>();
+  p.score = score.data_ptr<float>();
+  p.a = static_cast<uint16_t*>(a.data_ptr());
+  p.sa = p.a + (int64_t)p.M * p.top * p.F;
+  check_rc(nxd::experts_few_launch(r, p, cur_stream()), "experts_few");
+}
+
 }  // namespace
 
 void register_parallel(pybind11::module& m) {
@@ -262,4 +319,5 @@ void register_parallel(pybind11::module& m) {
   m.def("gather_rows", &gather_rows);
   m.def("grouped_linear", &grouped_linear);
   m.def("expert_rows", &expert_rows);
+  m.def("experts_few", &experts_few);
 }

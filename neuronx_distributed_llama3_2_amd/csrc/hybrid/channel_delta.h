@@ -22,8 +22,8 @@ struct ChannelDeltaParams {
   int64_t ldy;
   // chunks (channel_delta_chunk.hip), a cell = (sequence, chunk, head)
   int nch;
-  float *cq, *co;            // Q [cells, C DP], O [cells, C DP]
-  float *ct, *cm, *cs;       // T, M, S [cells, DP DP]
+  float *cq, *co, *cw, *cy, *cb, *ck;   // Q, O', W, Y, E B^T, E K^T [cells, C DP]
+  float *cs, *ce;            // S_0 [cells, DP DP], E [cells, DP]
 };
 
 namespace hybrid {

@@ -6,12 +6,13 @@
 // The removals' read-outs z_t = u_t^T S_(t-1) of all tokens solve (A = strictly lower parts)
 //   (I - A_ub) Z = U S_0 + A_uk V,     A_ub = U B^T, A_uk = U K^T
 // which is linear in the state S_0 the chunk starts from: Z = W S_0 + Y.  With the lower parts (diagonal
-// included) A_rb = R B^T, A_rk = R K^T and E = diag(e^(L_C)) everything else is linear in S_0 as well:
-//   O   = Q S_0 + O',   Q = R + A_rb W,        O' = A_rb Y + A_rk V
-//   S_1 = T S_0 + M,    T = E (I + B^T W),     M  = E (B^T Y + K^T V)
+// included) A_rb = R B^T, A_rk = R K^T and E = diag(e^(L_C)):
+//   O   = Q S_0 + O',            Q = R + A_rb W,  O' = A_rb Y + A_rk V
+//   S_1 = E S_0 + (E B^T) Z + (E K^T) V
 //
-//   prepare : Q, O', T, M of every (sequence, chunk, head) in parallel
-//   scan    : S <- T S + M, the chunks of a head one after another for 16 columns of the state
+//   prepare : Q, O', W, Y, E B^T, E K^T of every (sequence, chunk, head) in parallel
+//   scan    : Z and the next state, the chunks of a head one after another for 16 columns of the state; a
+//             wave has 16 rows of it, so W S_0 is summed over the waves, and nothing else is exchanged
 //   output  : O = Q S_0 + O', the head norm and the gate
 //
 // A log decay lies in (-e^(-1/2), 0), so e^(-L) stays below e^39 in a chunk of 64 and every product of a
@@ -40,17 +41,46 @@ __device__ __forceinline__ float pow2(double x) {
 
 constexpr int RANK_TILE = 64;
 
+// 8 neighbouring elements of a row, all of them there and 16-byte aligned (`wide`) or not
+template <typename T>
+struct Raw8;
+template <>
+struct Raw8<uint16_t> {
+  u32x4_t v;
+  __device__ void load(const uint16_t* p) { v = *reinterpret_cast<const u32x4_t*>(p); }
+  __device__ void zero() { v = u32x4_t{0u, 0u, 0u, 0u}; }
+  __device__ void get(float (&f)[8]) const { unpack8(v, f); }
+};
+template <>
+struct Raw8<float> {
+  f32x4_t a, b;
+  __device__ void load(const float* p) { a = ld4(p), b = ld4(p + 4); }
+  __device__ void zero() { a = b = f32x4_t{0.f, 0.f, 0.f, 0.f}; }
+  __device__ void get(float (&f)[8]) const {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) f[i] = a[i], f[4 + i] = b[i];
+  }
+};
+
+// LDS of the prepare kernel (floats): U, later the four products (with the rank tile before both); then R, B, K
+template <int NB, int CB>
+constexpr int first_region() {
+  constexpr int C = CB * 16, u = C * (NB * 16 + 4), a = 4 * C * C, r = C * (RANK_TILE + 4);
+  return u > a ? (u > r ? u : r) : (a > r ? a : r);
+}
+
 // NB = DP / 16 blocks of the head's channels, CB = C / 16 of the chunk's tokens.  One workgroup of 8 waves
 // a cell.
 template <typename T, int NB, int CB>
-__global__ void __launch_bounds__(512) cdelta_prepare_kernel(ChannelDeltaParams p) {
-  constexpr int DP = NB * 16, C = CB * 16, KS = DP + 4, AS = C + 4;   // LDS row strides (floats)
+__global__ void __launch_bounds__(512, CB == 2 ? 4 : 2) cdelta_prepare_kernel(ChannelDeltaParams p) {
+  constexpr int DP = NB * 16, C = CB * 16, KS = DP + 4;               // row stride of U, R, B, K
   constexpr int JW = (2 * NB + 7) / 8, HB = CB / 2, RS = RANK_TILE + 4;
   constexpr int LPT = 512 / C;                                        // lanes a token
-  static_assert(C * RS <= 4 * C * AS, "the rank tile fits where the products go");
+  constexpr int PJ = CB * (CB + 1) / 2 * 4, PW = (PJ + 7) / 8;        // blocks of the products, of them a wave
+  static_assert(C * DP / 8 <= 512, "a thread has 8 elements of a row");
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  float *us = sm, *rs = us + C * KS, *bs = rs + C * KS, *ks = bs + C * KS;   // [C][KS]
-  float* am = ks + C * KS;                                                   // A_ub, A_uk, A_rb, A_rk: [C][AS] each
+  float *us = sm, *rs = us + first_region<NB, CB>(), *bs = rs + C * KS, *ks = bs + C * KS;   // [C][KS]
+  float* am = us;   // A_ub, A_uk, A_rb, A_rk: [C][C] each, 16-byte pieces of a row swapped by its number
   __shared__ float rn[C], ec[DP];
   __shared__ double tot[2][DP];
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lq = lane >> 4;
@@ -62,26 +92,31 @@ __global__ void __launch_bounds__(512) cdelta_prepare_kernel(ChannelDeltaParams 
   const int64_t cell = ((int64_t)b * p.nch + ch) * H + h;
   const T* head = static_cast<const T*>(p.proj) + m0 * p.ldp + h * D;
   const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
+  // columns of V this wave solves for, and of U
+  const int tv = w, tw = w >= NB ? w - NB : w + 8 - NB;
+  const bool has_v = tv < NB && tv * 16 < D, has_w = tw < NB;
 
-  {   // ---- lengths of the keys
-    const int t = tid / LPT, j = tid % LPT;
-    float ss = 0.f;
-    if (t < n) {
-      const T* k = head + (int64_t)t * p.ldp + HD;
-      if (D % 4 == 0 && p.ldp % 4 == 0 && reinterpret_cast<uintptr_t>(p.proj) % 16 == 0) {
-        for (int d = 4 * j; d < D; d += 4 * LPT) {
-          const f32x4_t v = ld4(k + d);
-          ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
-        }
-      } else {
-        for (int d = j; d < D; d += LPT) {
-          const float v = ld(k + d);
-          ss += v * v;
-        }
+  // ---- what comes from memory is on its way first: r, k, removal (8 elements a thread), v (this wave's columns)
+  const bool wide = D % 8 == 0 && p.ldp % 8 == 0 && reinterpret_cast<uintptr_t>(p.proj) % 16 == 0;
+  const int rt = tid / (DP / 8), rc = tid % (DP / 8) * 8;
+  Raw8<T> raw[3];
+#pragma unroll
+  for (int j = 0; j < 3; ++j) raw[j].zero();
+  if (wide && rt < n && rc < D) {
+#pragma unroll
+    for (int j = 0; j < 3; ++j) raw[j].load(head + (int64_t)rt * p.ldp + (j == 0 ? 0 : (j == 1 ? HD : 4 * HD)) + rc);
+  }
+  f32x4_t v[CB];
+#pragma unroll
+  for (int bk = 0; bk < CB; ++bk) {
+    v[bk] = zero;
+    if (has_v) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 16 * bk + 4 * lq + i, col = tv * 16 + lr;
+        if (t < n && col < D) v[bk][i] = ld(head + (int64_t)t * p.ldp + 2 * HD + col);
       }
     }
-    ss = sum_lanes<LPT>(ss);
-    if (j == 0) rn[t] = 1.f / sqrtf(ss + 1e-6f);
   }
 
   // ---- log decays: W2 tanh(low), tokens x channels.  job = (channel block, half of the tokens)
@@ -90,12 +125,35 @@ __global__ void __launch_bounds__(512) cdelta_prepare_kernel(ChannelDeltaParams 
   for (int j = 0; j < JW; ++j)
 #pragma unroll
     for (int i = 0; i < HB; ++i) lw[j][i] = zero;
-  float* tl = am;   // [C][RS]
+  float* tl = us;   // [C][RS]
   for (int r0 = 0; r0 < N; r0 += RANK_TILE) {
-    __syncthreads();
+    if (r0 > 0) __syncthreads();
     for (int i = tid; i < C * RANK_TILE; i += 512) {
       const int t = i / RANK_TILE, k = i % RANK_TILE;
       tl[t * RS + k] = t < n && r0 + k < N ? tanhf_(ld(head + (int64_t)t * p.ldp + 5 * HD - h * D + r0 + k)) : 0.f;
+    }
+    if (r0 == 0) {
+      if (wide) {
+        if (rt < C) {
+#pragma unroll
+          for (int j = 0; j < 3; ++j) {
+            float f[8];
+            raw[j].get(f);
+            float* o = (j == 0 ? rs : (j == 1 ? ks : bs)) + rt * KS + rc;
+            st4(o, f32x4_t{f[0], f[1], f[2], f[3]});
+            st4(o + 4, f32x4_t{f[4], f[5], f[6], f[7]});
+          }
+        }
+      } else {
+        for (int i = tid; i < C * DP; i += 512) {
+          const int t = i / DP, c = i % DP;
+          const bool in = t < n && c < D;
+          const T* x = head + (int64_t)t * p.ldp + c;
+          rs[t * KS + c] = in ? ld(x) : 0.f;
+          ks[t * KS + c] = in ? ld(x + HD) : 0.f;
+          bs[t * KS + c] = in ? ld(x + 4 * HD) : 0.f;
+        }
+      }
     }
     __syncthreads();
     const int steps = (min(N - r0, RANK_TILE) + 15) / 16;
@@ -106,18 +164,30 @@ __global__ void __launch_bounds__(512) cdelta_prepare_kernel(ChannelDeltaParams 
       const int c = (job % NB) * 16 + lr, half = job / NB;
       const T* wr = static_cast<const T*>(p.w2) + (int64_t)(h * D + min(c, D - 1)) * N + r0;
       for (int s = 0; s < steps; ++s) {
-        f32x4_t f;
+        const int k = 16 * s + 4 * lq;
+        f32x4_t f = zero;
+        if (N % 4 == 0) {
+          if (r0 + k < N) f = ld4(wr + k);
+        } else {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int k = 16 * s + 4 * lq + i;
-          f[i] = r0 + k < N ? ld(wr + k) : 0.f;
+          for (int i = 0; i < 4; ++i) f[i] = r0 + k + i < N ? ld(wr + k + i) : 0.f;
         }
 #pragma unroll
-        for (int i = 0; i < HB; ++i) lw[j][i] = mma4(ld4(tl + (16 * (half * HB + i) + lr) * RS + 16 * s + 4 * lq), f, lw[j][i]);
+        for (int i = 0; i < HB; ++i) lw[j][i] = mma4(ld4(tl + (16 * (half * HB + i) + lr) * RS + k), f, lw[j][i]);
       }
     }
   }
-  // their running sums: of a half's tokens, then over both halves
+  {   // lengths of the keys
+    const int t = tid / LPT, j = tid % LPT;
+    float ss = 0.f;
+    for (int d = 4 * j; d < DP; d += 4 * LPT) {
+      const f32x4_t x = ld4(ks + t * KS + d);
+      ss += x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+    }
+    ss = sum_lanes<LPT>(ss);
+    if (j == 0) rn[t] = 1.f / sqrtf(ss + 1e-6f);
+  }
+  // the decays' running sums: of a half's tokens, then over both halves
   double base[JW][HB];   // sum before the lane's four tokens of a block
 #pragma unroll
   for (int j = 0; j < JW; ++j) {
@@ -144,8 +214,11 @@ __global__ void __launch_bounds__(512) cdelta_prepare_kernel(ChannelDeltaParams 
     }
     if (lq == 0) tot[half][c] = run;
   }
-  __syncthreads();
-  if (tid < DP) ec[tid] = pow2(tot[0][tid] + tot[1][tid]);
+  __syncthreads();   // (the rank tile's last readers are done as well)
+  if (tid < DP) {
+    ec[tid] = pow2(tot[0][tid] + tot[1][tid]);
+    p.ce[cell * DP + tid] = ec[tid];
+  }
 #pragma unroll
   for (int j = 0; j < JW; ++j) {
     const int job = w + 8 * j;
@@ -156,52 +229,56 @@ __global__ void __launch_bounds__(512) cdelta_prepare_kernel(ChannelDeltaParams 
 #pragma unroll
     for (int i = 0; i < HB; ++i) {
       double L = before + base[j][i];
-      float kk[4], aa[4], rr[4];
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int t = 16 * (half * HB + i) + 4 * lq + e;
-        const bool in = t < n && c < D;
-        const T* x = head + (int64_t)min(t, n - 1) * p.ldp + min(c, D - 1);
-        kk[e] = in ? ld(x + HD) : 0.f;
-        aa[e] = ld(x + 4 * HD);
-        rr[e] = in ? ld(x) : 0.f;
-      }
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int t = 16 * (half * HB + i) + 4 * lq + e, o = t * KS + c;
-        const float u = kk[e] * rn[t], a = 1.f / (1.f + expf(-(aa[e] + ab)));
+        const float k = ks[o], u = k * rn[t], a = 1.f / (1.f + expf(-(bs[o] + ab)));
         us[o] = u * pow2(L);
         L += (double)lw[j][i][e];
         const float inv = pow2(-L);
-        rs[o] = rr[e] * pow2(L);
+        rs[o] *= pow2(L);
         bs[o] = -a * u * inv;
-        ks[o] = kk[e] * inv;
+        ks[o] = k * inv;
       }
     }
   }
   __syncthreads();
 
-  // ---- the lower blocks of the four products
-  for (int job = w; job < CB * (CB + 1) / 2; job += 8) {
-    int bi = 0, bj = job;
-    while (bj > bi) bj -= ++bi;   // (0,0) (1,0) (1,1) (2,0) ...
-    f32x4_t ub = zero, uk = zero, rb = zero, rk = zero;
+  // ---- the lower blocks of the four products; the columns of U this wave solves for, before they go
+  auto piece = [&](int m, int row, int ch16) { return am + (m * C + row) * C + 4 * (ch16 ^ (row & (C / 4 - 1))); };
+  f32x4_t prod[PW], uw[CB];
 #pragma unroll
-    for (int kb = 0; kb < NB; ++kb) {
+  for (int j = 0; j < PW; ++j) {
+    const int job = w + 8 * j;
+    prod[j] = zero;
+    if (job >= PJ) continue;
+    int bi = 0, bj = job >> 2;
+    while (bj > bi) bj -= ++bi;   // (0,0) (1,0) (1,1) (2,0) ...
+    const float *ra = (job & 2) ? rs : us, *rb = (job & 1) ? ks : bs;
+    f32x4_t x0 = zero, x1 = zero;
+#pragma unroll
+    for (int kb = 0; kb < NB; kb += 2) {   // NB is even
       const int ro = (16 * bi + lr) * KS + 16 * kb + 4 * lq, co = (16 * bj + lr) * KS + 16 * kb + 4 * lq;
-      const f32x4_t fu = ld4(us + ro), fr = ld4(rs + ro), fb = ld4(bs + co), fk = ld4(ks + co);
-      ub = mma4(fu, fb, ub);
-      uk = mma4(fu, fk, uk);
-      rb = mma4(fr, fb, rb);
-      rk = mma4(fr, fk, rk);
+      x0 = mma4(ld4(ra + ro), ld4(rb + co), x0);
+      x1 = mma4(ld4(ra + ro + 16), ld4(rb + co + 16), x1);
     }
+    prod[j] = x0 + x1;
+  }
+#pragma unroll
+  for (int bi = 0; bi < CB; ++bi)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) uw[bi][i] = has_w ? us[(16 * bi + 4 * lq + i) * KS + tw * 16 + lr] : 0.f;
+  __syncthreads();
+#pragma unroll
+  for (int j = 0; j < PW; ++j) {
+    const int job = w + 8 * j, m = job & 3;
+    if (job >= PJ) continue;
+    int bi = 0, bj = job >> 2;
+    while (bj > bi) bj -= ++bi;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int row = 16 * bi + 4 * lq + i, col = 16 * bj + lr, o = row * AS + col;
-      am[o] = col < row ? ub[i] : 0.f;
-      am[C * AS + o] = col < row ? uk[i] : 0.f;
-      am[2 * C * AS + o] = col <= row ? rb[i] : 0.f;
-      am[3 * C * AS + o] = col <= row ? rk[i] : 0.f;
+      const int row = 16 * bi + 4 * lq + i, col = 16 * bj + lr;
+      piece(m, row, col >> 2)[col & 3] = col < row || (m >= 2 && col == row) ? prod[j][i] : 0.f;
     }
   }
   __syncthreads();
@@ -209,114 +286,89 @@ __global__ void __launch_bounds__(512) cdelta_prepare_kernel(ChannelDeltaParams 
   // ---- the diagonal blocks of I - A_ub, inverted in place by substitution: column lr
   if (w < CB) {
     float x[16];
-    float* a = am + (16 * w) * AS + 16 * w;
+    auto at = [&](int i, int j) { return piece(0, 16 * w + i, 4 * w + (j >> 2)) + (j & 3); };
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       float s = i == lr ? 1.f : 0.f;
 #pragma unroll
-      for (int j = 0; j < i; ++j) s += a[i * AS + j] * x[j];
+      for (int j = 0; j < i; ++j) s += *at(i, j) * x[j];
       x[i] = s;
     }
     __builtin_amdgcn_wave_barrier();
     if (lq == 0) {
 #pragma unroll
-      for (int i = 0; i < 16; ++i) a[i * AS + lr] = x[i];
+      for (int i = 0; i < 16; ++i) *at(i, lr) = x[i];
     }
+  }
+  // ---- E B^T and E K^T, A operands of the scan
+  for (int job = w; job < NB * CB; job += 8) {
+    const int cb = job / CB, bk = job % CB;
+    const float e = ec[16 * cb + lr];
+    f32x4_t fb, fk;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int o = (16 * bk + 4 * lq + i) * KS + 16 * cb + lr;
+      fb[i] = bs[o] * e;
+      fk[i] = ks[o] * e;
+    }
+    st4(p.cb + ((cell * NB + cb) * CB + bk) * 256 + lane * 4, fb);
+    st4(p.ck + ((cell * NB + cb) * CB + bk) * 256 + lane * 4, fk);
   }
   __syncthreads();
 
-  // ---- 16 columns of Y (from V) or W (from U) at a time, and what follows from them
-  auto frag = [&](int m, int bi, int bk) { return ld4(am + m * (C * AS) + (16 * bi + lr) * AS + 16 * bk + 4 * lq); };
-  for (int tile = w; tile < 2 * NB; tile += 8) {
-    const bool isv = tile < NB;
-    const int col = (isv ? tile : tile - NB) * 16 + lr, cb0 = isv ? tile : tile - NB;
-    if (isv && cb0 * 16 >= D) continue;
-    f32x4_t y[CB], v[CB];
-    if (isv) {
-#pragma unroll
-      for (int bk = 0; bk < CB; ++bk)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int t = 16 * bk + 4 * lq + i;
-          v[bk][i] = t < n && col < D ? ld(head + (int64_t)t * p.ldp + 2 * HD + col) : 0.f;
-        }
-    }
+  // ---- 16 columns of Y (from V) and of W (from U), and the outputs' parts
+  auto frag = [&](int m, int bi, int bk) { return ld4(piece(m, 16 * bi + lr, 4 * bk + lq)); };
+  if (has_v) {
+    f32x4_t y[CB];
 #pragma unroll
     for (int bi = 0; bi < CB; ++bi) {
       f32x4_t r = zero;
-      if (isv) {
 #pragma unroll
-        for (int bk = 0; bk <= bi; ++bk) r = mma4(frag(1, bi, bk), v[bk], r);
-      } else {
-#pragma unroll
-        for (int i = 0; i < 4; ++i) r[i] = us[(16 * bi + 4 * lq + i) * KS + col];
-      }
+      for (int bk = 0; bk <= bi; ++bk) r = mma4(frag(1, bi, bk), v[bk], r);
 #pragma unroll
       for (int bk = 0; bk < bi; ++bk) r = mma4(frag(0, bi, bk), y[bk], r);
       y[bi] = mma4(frag(0, bi, bi), r, zero);
+      st4(p.cy + ((cell * NB + tv) * CB + bi) * 256 + lane * 4, y[bi]);
     }
-    if (isv) {
 #pragma unroll
-      for (int bi = 0; bi < CB; ++bi) {
-        f32x4_t o = zero, o2 = zero;
+    for (int bi = 0; bi < CB; ++bi) {
+      f32x4_t o = zero, o2 = zero;
 #pragma unroll
-        for (int bk = 0; bk <= bi; ++bk) {
-          o = mma4(frag(2, bi, bk), y[bk], o);
-          o2 = mma4(frag(3, bi, bk), v[bk], o2);
-        }
-        st4(p.co + ((cell * NB + cb0) * CB + bi) * 256 + lane * 4, o + o2);
+      for (int bk = 0; bk <= bi; ++bk) {
+        o = mma4(frag(2, bi, bk), y[bk], o);
+        o2 = mma4(frag(3, bi, bk), v[bk], o2);
       }
+      st4(p.co + ((cell * NB + tv) * CB + bi) * 256 + lane * 4, o + o2);
+    }
+  }
+  if (has_w) {
+    f32x4_t y[CB];
 #pragma unroll
-      for (int cb = 0; cb < NB; ++cb) {
-        f32x4_t m = zero, m2 = zero;
+    for (int bi = 0; bi < CB; ++bi) {
+      f32x4_t r = uw[bi];
 #pragma unroll
-        for (int bk = 0; bk < CB; ++bk) {
-          f32x4_t fb, fk;
+      for (int bk = 0; bk < bi; ++bk) r = mma4(frag(0, bi, bk), y[bk], r);
+      y[bi] = mma4(frag(0, bi, bi), r, zero);
+      // W as an A operand: its transpose is what these registers are
+      float* o = p.cw + ((cell * NB + tw) * CB + bi) * 256 + (lr >> 2) * 64 + (lr & 3);
 #pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            const int o = (16 * bk + 4 * lq + i) * KS + 16 * cb + lr;
-            fb[i] = bs[o];
-            fk[i] = ks[o];
-          }
-          m = mma4(fb, y[bk], m);
-          m2 = mma4(fk, v[bk], m2);
-        }
-        m += m2;
+      for (int i = 0; i < 4; ++i) o[(4 * lq + i) * 4] = y[bi][i];
+    }
 #pragma unroll
-        for (int i = 0; i < 4; ++i) m[i] *= ec[16 * cb + 4 * lq + i];
-        st4(p.cm + ((cell * NB + cb0) * NB + cb) * 256 + lane * 4, m);
-      }
-    } else {   // (transposed products: A operands of what reads them)
+    for (int bi = 0; bi < CB; ++bi) {   // (a transposed product: an A operand of what reads it)
+      f32x4_t q = ld4(rs + (16 * bi + lr) * KS + 16 * tw + 4 * lq);
 #pragma unroll
-      for (int bi = 0; bi < CB; ++bi) {
-        f32x4_t q = ld4(rs + (16 * bi + lr) * KS + 16 * cb0 + 4 * lq);
-#pragma unroll
-        for (int bk = 0; bk <= bi; ++bk) q = mma4(y[bk], frag(2, bi, bk), q);
-        st4(p.cq + ((cell * CB + bi) * NB + cb0) * 256 + lane * 4, q);
-      }
-#pragma unroll
-      for (int cb = 0; cb < NB; ++cb) {
-        f32x4_t t = zero;
-#pragma unroll
-        for (int bk = 0; bk < CB; ++bk) {
-          f32x4_t fb;
-#pragma unroll
-          for (int i = 0; i < 4; ++i) fb[i] = bs[(16 * bk + 4 * lq + i) * KS + 16 * cb + lr];
-          t = mma4(y[bk], fb, t);
-        }
-#pragma unroll
-        for (int i = 0; i < 4; ++i) t[i] = (t[i] + (16 * cb + lr == 16 * cb0 + 4 * lq + i ? 1.f : 0.f)) * ec[16 * cb + lr];
-        st4(p.ct + ((cell * NB + cb) * NB + cb0) * 256 + lane * 4, t);
-      }
+      for (int bk = 0; bk <= bi; ++bk) q = mma4(y[bk], frag(2, bi, bk), q);
+      st4(p.cq + ((cell * CB + bi) * NB + tw) * 256 + lane * 4, q);
     }
   }
 }
 
-// 16 columns of one head's state, a wave for 16 rows.  T and M are fetched four chunks ahead.
-template <int NB, int CB>
+// 16 columns of one head's state, a wave for 16 rows.  A chunk's operands are fetched AHEAD chunks before.
+template <typename T, int NB, int CB>
 __global__ void __launch_bounds__(NB * 64) cdelta_scan_kernel(ChannelDeltaParams p) {
-  constexpr int DP = NB * 16, C = CB * 16, AHEAD = 4;
-  __shared__ __attribute__((aligned(16))) f32x4_t ss[2][NB][64];
+  constexpr int DP = NB * 16, C = CB * 16, AHEAD = CB == 2 ? 4 : 2, RB = (CB + NB - 1) / NB;   // blocks of Z a wave sums
+  __shared__ __attribute__((aligned(16))) f32x4_t part[NB][CB][64], zs[CB][64];
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lq = lane >> 4;
   const int bh = blockIdx.x % (p.B * p.H), vt = blockIdx.x / (p.B * p.H);   // a head's columns on one XCD
   const int b = bh / p.H, h = bh % p.H, H = p.H, D = p.D, v = vt * 16 + lr;
@@ -325,49 +377,80 @@ __global__ void __launch_bounds__(NB * 64) cdelta_scan_kernel(ChannelDeltaParams
   const int slot = slot_of(p.slots, b, p.nslots);
   const int64_t p0 = pos_of(p.pos, p.pos_stride, b);
   float* state = p.state + (((int64_t)slot * H + h) * D + min(v, D - 1)) * DP + w * 16 + 4 * lq;
-  f32x4_t S = {0.f, 0.f, 0.f, 0.f};
+  const T* vals = static_cast<const T*>(p.proj) + (int64_t)b * p.T * p.ldp + 2 * H * D + h * D + min(v, D - 1);
+  const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
+  f32x4_t S = zero;
   if (p0 > 0 && v < D) S = ld4(state);
   const int nch = (len + C - 1) / C;
+  const int64_t NC = (int64_t)NB * CB * 256;   // floats of a cell's operand
   struct Ops {
-    f32x4_t t[NB], m;
+    f32x4_t w[CB], b[CB], k[CB], y[RB];
+    T v[CB][4];
+    float e[4];
   };
   Ops set[AHEAD];
   auto fetch = [&](int c, Ops& o) {   // (past the last chunk the last one is read again)
-    const int64_t cell = ((int64_t)b * p.nch + min(c, nch - 1)) * H + h;
-    const float* t = p.ct + (cell * NB + w) * (NB * 256) + lane * 4;
+    c = min(c, nch - 1);
+    const int64_t cell = ((int64_t)b * p.nch + c) * H + h, at = cell * NC + (int64_t)w * CB * 256 + lane * 4;
 #pragma unroll
-    for (int kb = 0; kb < NB; ++kb) o.t[kb] = ld4(t + kb * 256);
-    o.m = ld4(p.cm + ((cell * NB + vt) * NB + w) * 256 + lane * 4);
+    for (int i = 0; i < CB; ++i) {
+      o.w[i] = ld4(p.cw + at + i * 256);
+      o.b[i] = ld4(p.cb + at + i * 256);
+      o.k[i] = ld4(p.ck + at + i * 256);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) o.v[i][j] = vals[(int64_t)min(c * C + 16 * i + 4 * lq + j, len - 1) * p.ldp];
+    }
+#pragma unroll
+    for (int i = 0; i < RB; ++i)
+      if (w + NB * i < CB) o.y[i] = ld4(p.cy + cell * NC + ((int64_t)vt * CB + w + NB * i) * 256 + lane * 4);
+    const f32x4_t e = ld4(p.ce + cell * DP + w * 16 + 4 * lq);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o.e[j] = e[j];
   };
 #pragma unroll
   for (int i = 0; i < AHEAD; ++i) fetch(i, set[i]);
-  auto chunk = [&](int c, Ops& o, int flip) {
+  auto chunk = [&](int c, Ops& o) {
     const int64_t cell = ((int64_t)b * p.nch + c) * H + h;
-    ss[flip][w][lane] = S;
+#pragma unroll
+    for (int i = 0; i < CB; ++i) part[w][i][lane] = mma4(o.w[i], S, zero);
     st4(p.cs + ((cell * NB + vt) * NB + w) * 256 + lane * 4, S);
-    lds_barrier();
-    f32x4_t s[NB], a0 = o.m, a1 = {0.f, 0.f, 0.f, 0.f};
+    f32x4_t n0, n1 = zero;
 #pragma unroll
-    for (int kb = 0; kb < NB; ++kb) s[kb] = ss[flip][kb][lane];
+    for (int j = 0; j < 4; ++j) n0[j] = S[j] * o.e[j];
 #pragma unroll
-    for (int kb = 0; kb < NB; kb += 2) {   // NB is even
+    for (int i = 0; i < CB; ++i) {   // (needs nothing of the other waves)
+      f32x4_t x;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        a0 = __builtin_amdgcn_mfma_f32_16x16x4f32(o.t[kb][i], s[kb][i], a0, 0, 0, 0);
-        a1 = __builtin_amdgcn_mfma_f32_16x16x4f32(o.t[kb + 1][i], s[kb + 1][i], a1, 0, 0, 0);
-      }
+      for (int j = 0; j < 4; ++j) x[j] = c * C + 16 * i + 4 * lq + j < len && v < D ? ld(&o.v[i][j]) : 0.f;
+      n1 = mma4(o.k[i], x, n1);
     }
-    S = a0 + a1;
+    lds_barrier();
+#pragma unroll
+    for (int i = 0; i < RB; ++i) {
+      const int blk = w + NB * i;
+      if (blk >= CB) continue;
+      f32x4_t z = o.y[i];
+#pragma unroll
+      for (int j = 0; j < NB; ++j) z += part[j][blk][lane];
+      zs[blk][lane] = z;
+    }
+    lds_barrier();
+#pragma unroll
+    for (int i = 0; i < CB; ++i) {
+      if (i & 1) n1 = mma4(o.b[i], zs[i][lane], n1);
+      else n0 = mma4(o.b[i], zs[i][lane], n0);
+    }
+    S = n0 + n1;
     fetch(c + AHEAD, o);
   };
   int c = 0;
   for (; c + AHEAD <= nch; c += AHEAD) {
 #pragma unroll
-    for (int i = 0; i < AHEAD; ++i) chunk(c + i, set[i], i & 1);
+    for (int i = 0; i < AHEAD; ++i) chunk(c + i, set[i]);
   }
 #pragma unroll
   for (int i = 0; i < AHEAD; ++i)
-    if (c + i < nch) chunk(c + i, set[i], i & 1);
+    if (c + i < nch) chunk(c + i, set[i]);
   if (v < D) st4(state, S);
 }
 
@@ -423,7 +506,7 @@ __global__ void __launch_bounds__(CB * 64) cdelta_output_kernel(ChannelDeltaPara
 template <typename T, int NB, int CB>
 static int run_chunk(const ChannelDeltaParams& p, hipStream_t s) {
   constexpr int C = CB * 16;
-  constexpr size_t lds = (size_t)4 * C * (NB * 16 + 4 + C + 4) * 4;
+  constexpr size_t lds = (size_t)(first_region<NB, CB>() + 3 * C * (NB * 16 + 4)) * 4;
   static_assert(lds <= 152 * 1024, "LDS of a compute unit");
   static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&cdelta_prepare_kernel<T, NB, CB>),
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
@@ -431,7 +514,7 @@ static int run_chunk(const ChannelDeltaParams& p, hipStream_t s) {
   const dim3 grid((unsigned)p.H, (unsigned)p.nch, (unsigned)p.B);
   hipLaunchKernelGGL((cdelta_prepare_kernel<T, NB, CB>), grid, dim3(512), lds, s, p);
   if (hipGetLastError() != hipSuccess) return 1;
-  hipLaunchKernelGGL((cdelta_scan_kernel<NB, CB>), dim3((unsigned)(ceil_div(p.D, 16) * p.B * p.H)), dim3(NB * 64), 0, s, p);
+  hipLaunchKernelGGL((cdelta_scan_kernel<T, NB, CB>), dim3((unsigned)(ceil_div(p.D, 16) * p.B * p.H)), dim3(NB * 64), 0, s, p);
   if (hipGetLastError() != hipSuccess) return 1;
   hipLaunchKernelGGL((cdelta_output_kernel<T, NB, CB>), grid, dim3(CB * 64), 0, s, p);
   return hipGetLastError() == hipSuccess ? 0 : 1;

@@ -1,4 +1,4 @@
-// Parameters of the routed-expert kernels (csrc/hybrid/moe_route.hip, expert_rows.hip).
+// Parameters of the routed-expert kernels (csrc/hybrid/moe_route.hip, expert_decode.hip).
 #pragma once
 #include "hybrid.h"
 
@@ -43,6 +43,20 @@ struct ExpertRowsParams {
   int E, N, K;
   int64_t P;
   void* y;                 // [P, N]
+};
+
+// a few tokens (expert_decode.hip)
+struct ExpertFewParams {
+  int M, E, top, shared;   // shared: 1 with a shared expert (else 0)
+  int W, F, FS;            // width, feed-forward sizes
+  const uint16_t* h;       // [M, ldh]
+  int64_t ldh;
+  const uint16_t *router, *up, *down, *sup, *sdown;   // [E + shared, W], [E, 2 F, W], [E, W, F], [2 FS, W], [W, FS]
+  float limit, slimit;
+  int* index;              // [M, top]
+  float* score;            // [M, top + shared]
+  uint16_t *a, *sa;        // [M top, F], [M, FS]
+  uint16_t* y;             // [M (top + shared), W]
 };
 
 namespace hybrid {

@@ -15,7 +15,7 @@ struct GemvHyperParams {
   int M, N, K;
   void* y;                // [M, N]
   int64_t ldy;
-  float cap;
+  float alpha, cap;       // fp32 outputs: cap tanh(alpha y / cap), or alpha y
   // HYPER
   float* streams;         // [M, S, N]
   int S;

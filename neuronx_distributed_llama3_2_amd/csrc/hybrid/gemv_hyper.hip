@@ -1,7 +1,7 @@
 // Decode projections (1 to 4 rows) of hyper-connected decoders, with the element-wise work around them:
 //
 //   NORM prologue : x = rms_normalise(u) (1 + norm_w) from the fp32 sublayer input u [M, K]
-//   epilogues     : store (bf16) | squared ReLU (bf16) | fp32 with an optional cap tanh(y / cap)
+//   epilogues     : store (bf16) | squared ReLU (bf16) | fp32 with a factor and an optional cap
 //                   | HYPER: y + bias goes straight into the residual streams, x_t = sum_s mix[s][t] x_s +
 //                   write[t] y, and u = sum_t read[t] x_t of the next sublayer comes out -- a column of
 //                   the streams belongs to the one wave that owns the weight row, so it is updated in place
@@ -36,6 +36,7 @@ __device__ __forceinline__ void emit(const GemvHyperParams& p, int m, int n, flo
     const float r = fmaxf(v, 0.f);
     static_cast<uint16_t*>(p.y)[(int64_t)m * p.ldy + n] = f2bf(r * r);
   } else if (EPI == F32CAP) {
+    v *= p.alpha;
     static_cast<float*>(p.y)[(int64_t)m * p.ldy + n] = p.cap > 0.f ? p.cap * tanhf(v / p.cap) : v;
   } else {
     v = bf2f(f2bf(v)) + (p.bias ? p.bias[n] : 0.f);   // the projection's output is a bf16 activation

@@ -14,7 +14,7 @@ struct GroupNormParams {
   const void* add[2];      // [M, ld_add] (nullable)
   int64_t ld_add[2];
   const void* pairs;       // [npairs, W] (nullable)
-  const int* inverse;      // [M, k]
+  const int* inverse;      // [M, k] (nullable: row m k + j)
   int npairs, k;
   const float* w[2];       // [W]
   void* h[2];              // [R, ldh] (nullable)

@@ -1,7 +1,7 @@
 // The step between two layers whose sublayers read one fp32 residual side by side:
 //
 //   x <- x (or an embedding row) + outputs of the last layer (up to two rows, and k rows of expert outputs
-//        found through `inverse`)
+//        found through `inverse`, or in order)
 //   h_n = x / sqrt(mean over each of `groups` equal parts of x^2 + eps) * w_n      (one or two weights)
 //
 // One workgroup a row, the row in registers, 4 elements a lane and step (1 for sizes that are no multiple).
@@ -72,7 +72,7 @@ __global__ void __launch_bounds__(256) residual_norms_kernel(GroupNormParams p) 
   }
   if (p.pairs) {
     for (int k = 0; k < p.k; ++k) {
-      const int row = min(max(p.inverse[m * p.k + k], 0), p.npairs - 1);
+      const int row = p.inverse ? min(max(p.inverse[m * p.k + k], 0), p.npairs - 1) : (int)(m * p.k + k);
       const T* s = static_cast<const T*>(p.pairs) + (int64_t)row * W;
 #pragma unroll
       for (int i = 0; i < NV; ++i) {

@@ -2,8 +2,8 @@
 //
 //   moe_choose : scores, groups, the chosen experts and their weights of a chunk of tokens (a wave a token),
 //                and the chunk's count of every expert
-//   moe_place  : where every (token, choice) pair goes when pairs are sorted by expert (stable), from the
-//                counts of all chunks
+//   moe_scan   : where every chunk's pairs of every expert start when pairs are sorted by expert
+//   moe_place  : where every (token, choice) pair goes (stable)
 //
 // and what runs around the experts' matrix products: the gather of token rows and the clamped gated
 // activation with the pair's weight.
@@ -39,34 +39,58 @@ __global__ void __launch_bounds__(ROUTE_WAVES * 64) moe_choose_kernel(RouterPara
   for (int e = tid; e < E; e += ROUTE_WAVES * 64) p.counts[(int64_t)blockIdx.x * E + e] = count[e];
 }
 
+// counts[chunk][e] -> the chunk's first row of expert e; offs.  One workgroup, a wave an expert at a time
+__global__ void __launch_bounds__(1024) moe_scan_kernel(RouterParams p) {
+  extern __shared__ int total[];   // [E + 1]
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, E = p.E;
+  for (int e = w; e < E; e += 16) {
+    int run = 0;
+    for (int c0 = 0; c0 < p.chunks; c0 += 64) {
+      const int c = c0 + lane, n = c < p.chunks ? p.counts[(int64_t)c * E + e] : 0;
+      int x = n;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const int y = __shfl_up(x, o, 64);
+        if (lane >= o) x += y;
+      }
+      if (c < p.chunks) p.counts[(int64_t)c * E + e] = run + x - n;
+      run += __shfl(x, 63, 64);
+    }
+    if (lane == 0) total[e] = run;
+  }
+  __syncthreads();
+  if (w == 0) {
+    int run = 0;
+    for (int e0 = 0; e0 < E; e0 += 64) {
+      const int e = e0 + lane, n = e < E ? total[e] : 0;
+      int x = n;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const int y = __shfl_up(x, o, 64);
+        if (lane >= o) x += y;
+      }
+      if (e < E) p.offs[e] = run + x - n;
+      run += __shfl(x, 63, 64);
+    }
+    if (lane == 0) p.offs[E] = run;
+  }
+}
+
+// a thread a (token, choice) pair of the chunk
 __global__ void __launch_bounds__(256) moe_place_kernel(RouterParams p) {
-  extern __shared__ __attribute__((aligned(16))) int ism[];   // E totals, then the chunk's experts
-  int *total = ism, *ex = ism + p.E;
+  extern __shared__ __attribute__((aligned(16))) int ex[];   // the chunk's experts
   const int tid = threadIdx.x, ch = blockIdx.x, E = p.E, top = p.top;
   const int64_t i0 = (int64_t)ch * ROUTE_TOKENS * top;
   const int n = (int)min((int64_t)ROUTE_TOKENS * top, p.M * top - i0);
   for (int i = tid; i < n; i += 256) ex[i] = p.index[i0 + i];
-  for (int e = tid; e < E; e += 256) {
-    int t = 0;
-    for (int c = 0; c < p.chunks; ++c) t += p.counts[(int64_t)c * E + e];
-    total[e] = t;
-  }
   __syncthreads();
-  for (int e = tid; e < E; e += 256) {
-    int at = 0;
-    for (int j = 0; j < e; ++j) at += total[j];
-    if (ch == 0) {
-      p.offs[e] = at;
-      if (e == E - 1) p.offs[E] = at + total[e];
-    }
-    for (int c = 0; c < ch; ++c) at += p.counts[(int64_t)c * E + e];
-    for (int i = 0; i < n; ++i) {
-      if (ex[i] != e) continue;
-      p.token[at] = (int)((i0 + i) / top);
-      p.weight[at] = p.score[i0 + i];
-      p.inverse[i0 + i] = at;
-      ++at;
-    }
+  for (int i = tid; i < n; i += 256) {
+    const int e = ex[i];
+    int at = p.offs[e] + p.counts[(int64_t)ch * E + e];
+    for (int j = 0; j < i; ++j) at += ex[j] == e;
+    p.token[at] = (int)((i0 + i) / top);
+    p.weight[at] = p.score[i0 + i];
+    p.inverse[i0 + i] = at;
   }
 }
 
@@ -135,7 +159,8 @@ int moe_route_launch(const RouterParams& p, hipStream_t s) {
                                                      hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024);
   if (attr != hipSuccess) return 2;
   hipLaunchKernelGGL(moe_choose_kernel, dim3((unsigned)p.chunks), dim3(ROUTE_WAVES * 64), lds, s, p);
-  hipLaunchKernelGGL(moe_place_kernel, dim3((unsigned)p.chunks), dim3(256), (size_t)(p.E + ROUTE_TOKENS * p.top) * 4, s, p);
+  hipLaunchKernelGGL(moe_scan_kernel, dim3(1), dim3(1024), (size_t)(p.E + 1) * 4, s, p);
+  hipLaunchKernelGGL(moe_place_kernel, dim3((unsigned)p.chunks), dim3(256), (size_t)ROUTE_TOKENS * p.top * 4, s, p);
   return hipGetLastError() == hipSuccess ? 0 : 1;
 }
 

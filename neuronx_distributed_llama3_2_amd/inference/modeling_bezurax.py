@@ -18,7 +18,7 @@ import torch.nn as nn
 from .. import ops
 from ..models.bezurax import BezuraxConfig
 from ..modules.hybrid import ChannelDelta, ParallelMixer, PooledAttention, RoutedExperts, StepContext
-from ..modules.hybrid.context import small
+from ..modules.hybrid.context import few_rows, small
 from ..ops.experts import RouterRule
 from ..ops.gemm import linear_f32
 from ..parallel_layers.parallel_state import get_tensor_model_parallel_size
@@ -131,10 +131,14 @@ class BezuraxInferenceModel(DecoderInferenceMixin, nn.Module):
             y = layer.mixer(hs[0], self.kv_cache[i], ctx)
             last = dict(adds=[y])
             if layer.mlp is not None:
-                m = layer.mlp(hs[1])
+                m = layer.mlp(hs[1], ctx.fused)
                 last = dict(m, adds=[y, *m["adds"]])
         h = ops.residual_norms(x, [self.model.norm.weight], rows=logit_rows, store=False, **norm, **last)[0]
-        logits = linear_f32(h, self.lm_head.weight, self.config.logit_scale)
+        w, scale = self.lm_head.weight, self.config.logit_scale
+        if ctx.fused and few_rows(h, w):
+            logits = ops.decode_linear(w, h, epilogue="f32", alpha=scale)
+        else:
+            logits = linear_f32(h, w, scale)
         if logit_rows is None:
             logits, h = logits.view(B, T, -1), h.view(B, T, -1)
         return (logits, h) if return_hidden else logits

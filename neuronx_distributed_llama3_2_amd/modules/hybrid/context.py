@@ -31,9 +31,23 @@ def padded_rows(n: int) -> int:
     return (n + ROW_ALIGN - 1) // ROW_ALIGN * ROW_ALIGN
 
 
-def linear(x: torch.Tensor, mod: torch.nn.Module) -> torch.Tensor:
-    """x [M, K] @ mod.weight^T, through the module's packed copy when the layout pass chose it."""
+# rows up to which a projection streams its weights (csrc/hybrid/gemv_hyper.hip)
+FEW_ROWS = 4
+
+
+def few_rows(x: torch.Tensor, w: torch.Tensor) -> bool:
+    return x.is_cuda and x.shape[0] <= FEW_ROWS and x.dtype == w.dtype == torch.bfloat16 and w.shape[1] % 8 == 0 and \
+        x.is_contiguous()
+
+
+def linear(x: torch.Tensor, mod: torch.nn.Module, fused: bool = False) -> torch.Tensor:
+    """x [M, K] @ mod.weight^T: through the module's packed copy when the layout pass chose it; fused: a few
+    rows by the decode kernel."""
+    from ... import ops
     from ...trace.weight_layout import packed_linear
+
+    if fused and few_rows(x, mod.weight):
+        return ops.decode_linear(mod.weight, x)
 
     return packed_linear(mod, x, mod.weight)
 

@@ -35,9 +35,13 @@ class RoutedExperts(nn.Module):
         self.gate_up.normal_(0.0, self.gate_up.shape[2] ** -0.5)
         self.down.normal_(0.0, self.down.shape[2] ** -0.5)
 
-    def forward(self, h: torch.Tensor) -> Dict[str, object]:
+    def forward(self, h: torch.Tensor, fused: bool = True) -> Dict[str, object]:
         """What ops.residual_norms adds to the residual: the outputs of (token, choice) pairs, weighted,
-        where each is, and the shared expert's output."""
+        where each is, and the shared expert's output.  fused: a few tokens take the unsorted kernels."""
+        shared = (self.shared_up.weight, self.shared_down.weight) if self.shared_up is not None else (None, None)
+        if fused and ops.experts_few_supported(h, self.gate_up, self.down, *shared):
+            return dict(pairs=ops.experts_few(h, self.router.weight, self.rule, self.gate_up, self.down, self.limit, *shared,
+                                              self.shared_limit), adds=[])
         logits = linear_f32(h, self.router.weight)
         r = ops.route(logits, self.rule)
         a = ops.clamped_glu(ops.expert_linear_rows(h, self.gate_up, r.offs, r.token), self.limit, r.weight)

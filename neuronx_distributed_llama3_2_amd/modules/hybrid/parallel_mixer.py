@@ -52,4 +52,4 @@ class ParallelMixer(nn.Module):
         return out
 
     def forward(self, h: torch.Tensor, cache: Dict[str, torch.Tensor], ctx: StepContext) -> torch.Tensor:
-        return linear(self.core(linear(h, self.in_proj), cache, ctx), self.o_proj)
+        return linear(self.core(linear(h, self.in_proj, ctx.fused), cache, ctx), self.o_proj, ctx.fused)

@@ -8,7 +8,8 @@ from .cross_entropy import parallel_cross_entropy_reference, vocab_parallel_cros
 from .decode import argmax_rows, decode_attention, greedy_advance_, kv_cache_write, topk_sample  # noqa: F401
 from .delta_rule import DeltaSizes, delta_rule  # noqa: F401
 from .embedding import vocab_parallel_embedding  # noqa: F401
-from .experts import RouterRule, Routing, clamped_glu, expert_linear_rows, route  # noqa: F401
+from .experts import (RouterRule, Routing, clamped_glu, expert_linear_rows, experts_few, experts_few_supported,  # noqa: F401
+                      route)
 from .group_norm import residual_norms  # noqa: F401
 from .grouped_gemm import (grouped_linear, grouped_linear_reference, moe_dispatch, moe_permutation,  # noqa: F401
                            moe_unpermute_combine)

@@ -1,4 +1,4 @@
-"""Routed experts of inference decoders (csrc/hybrid/moe_route.hip, expert_rows.hip and the grouped GEMMs):
+"""Routed experts of inference decoders (csrc/hybrid/moe_route.hip, expert_decode.hip and the grouped GEMMs):
 sigmoid router with groups of experts, clamped gated activation, all on the device without a host sync."""
 
 from __future__ import annotations
@@ -98,4 +98,26 @@ def expert_linear_rows(x: torch.Tensor, w: torch.Tensor, offs: torch.Tensor, tok
     b = offs.tolist()
     for e in range(E):
         y[b[e]:b[e + 1]] = torch.nn.functional.linear(xs[b[e]:b[e + 1]], w[e])
+    return y
+
+
+# tokens up to which the experts run unsorted (csrc/hybrid/expert_decode.hip)
+FEW_TOKENS = 64
+
+
+def experts_few_supported(h: torch.Tensor, *weights: Optional[torch.Tensor]) -> bool:
+    return use_native(h) and h.shape[0] <= FEW_TOKENS and h.dtype == torch.bfloat16 and \
+        all(w is None or w.dtype == torch.bfloat16 and w.shape[-1] % 8 == 0 for w in weights)
+
+
+def experts_few(h: torch.Tensor, router: torch.Tensor, rule: RouterRule, gate_up: torch.Tensor, down: torch.Tensor, limit: float,
+                shared_up: Optional[torch.Tensor] = None, shared_down: Optional[torch.Tensor] = None,
+                shared_limit: float = 0.0) -> torch.Tensor:
+    """A whole routed feed-forward for a few tokens (GPU, bf16) in three launches.  router [>= E (+ 1), W]: the
+    experts' rows, then the shared expert's gate.  Returns [M (top + 1), W]: for each token its experts'
+    weighted outputs and then its shared expert's; their sum is the feed-forward's output."""
+    slots = rule.top + (0 if shared_up is None else 1)
+    y = torch.empty((h.shape[0] * slots, h.shape[1]), dtype=h.dtype, device=h.device)
+    hybrid_ext().experts_few(h, router, rule.as_list(), rule.scale, gate_up, down, float(limit), shared_up, shared_down,
+                             float(shared_limit), y)
     return y

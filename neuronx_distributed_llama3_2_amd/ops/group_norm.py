@@ -21,7 +21,7 @@ def residual_norms(x: torch.Tensor, norms: Sequence[torch.Tensor], eps: float, g
       h_n = x / sqrt(mean of x^2 over each of `groups` equal parts + eps) * norms[n]
 
     for at most two adds and two norms (fp32 [W]).  pairs [P, W], inverse int32 [M, k]: outputs of
-    (token, choice) pairs and where each is.  rows [R] (int64): only these rows, read-only (store=False).
+    (token, choice) pairs and where each is (None: in order, P / M for each row).  rows [R] (int64): only these rows, read-only (store=False).
     Returns the normalised rows in `dtype` (that of the adds / embed)."""
     M, W = x.shape
     src = embed if embed is not None else (adds[0] if adds else pairs)
@@ -39,7 +39,7 @@ def residual_norms(x: torch.Tensor, norms: Sequence[torch.Tensor], eps: float, g
     for a in adds:
         y = y + a.float()
     if pairs is not None:
-        y = y + pairs[inverse.long()].float().sum(1)
+        y = y + (pairs[inverse.long()] if inverse is not None else pairs.view(M, -1, W)).float().sum(1)
     if store:
         x.copy_(y)
     if rows is not None:

@@ -75,13 +75,14 @@ _EPI = {"store": 0, "relu2": 1, "f32": 2, "streams": 3}
 
 
 def decode_linear(w: torch.Tensor, x: Optional[torch.Tensor] = None, u: Optional[torch.Tensor] = None,
-                  norm_w: Optional[torch.Tensor] = None, eps: float = 0.0, epilogue: str = "store", cap: float = 0.0):
+                  norm_w: Optional[torch.Tensor] = None, eps: float = 0.0, epilogue: str = "store", cap: float = 0.0,
+                  alpha: float = 1.0):
     """epilogue(x w^T) for a few rows in one launch (csrc/hybrid/gemv_hyper.hip, GPU, bf16 weights): x
     bf16 [M, K], or u fp32 [M, K], normalised as hyper_step does on the way in.  "store": bf16, "relu2":
-    bf16 squared ReLU, "f32": fp32, with cap > 0 cap tanh(y / cap)."""
+    bf16 squared ReLU, "f32": fp32 alpha y, with cap > 0 cap tanh(alpha y / cap)."""
     M = (x if x is not None else u).shape[0]
     y = torch.empty((M, w.shape[0]), dtype=torch.float32 if epilogue == "f32" else torch.bfloat16, device=w.device)
-    hybrid_ext().gemv_hyper(_EPI[epilogue], x, u, norm_w, float(eps), w, y, float(cap))
+    hybrid_ext().gemv_hyper(_EPI[epilogue], x, u, norm_w, float(eps), w, y, float(cap), alpha=float(alpha))
     return y
 
 

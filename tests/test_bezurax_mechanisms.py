@@ -122,7 +122,7 @@ def test_clamped_activation(where, F):
 
 @pytest.mark.parametrize("where", WHERE)
 @pytest.mark.parametrize("E,N,K", [(5, 24, 40), (3, 17, 9), (4, 136, 64), (7, 64, 256)])
-@pytest.mark.parametrize("M", [2, 60, 700])
+@pytest.mark.parametrize("M", [2, 60, 2500])
 def test_expert_products(where, E, N, K, M):
     w, w_o = act(rnd(E, N, K) * K ** -0.5, where)
     x, x_o = act(rnd(M, K, seed=1), where)
@@ -170,16 +170,34 @@ MOES = [(48, 6, 2, 24, 1.2, 1.7, 3, 2, 40, 0.8), (64, 8, 4, 32, 0.6, 2.0, 2, 1, 
 
 @pytest.mark.parametrize("where", WHERE)
 @pytest.mark.parametrize("case", MOES)
-@pytest.mark.parametrize("M", [1, 4, 90])
+@pytest.mark.parametrize("M", [1, 4, 17, 33, 64, 90])
 def test_routed_experts(where, case, M):
-    """The whole feed-forward, as it reaches the residual."""
+    """The whole feed-forward, as it reaches the residual, for a few tokens (unsorted kernels) and many."""
     mod, cfg, sd = experts_module(where, *case)
     W = case[0]
     h, h_o = act(rnd(M, W, seed=5), where)
-    x = torch.zeros((M, W), dtype=torch.float32, device=where[0])
-    # the residual sum takes what the feed-forward returns
-    ops.residual_norms(x, [torch.ones(W, device=where[0])], 1e-5, 1, dtype=where[1], **mod(h))
-    assert rel_err(x, O.moe(h_o, cfg, sd, "")) < (where[2] if where[1] == torch.float32 else 4e-2)
+    want = O.moe(h_o, cfg, sd, "")
+    for fused in (True, False):
+        x = torch.zeros((M, W), dtype=torch.float32, device=where[0])
+        # the residual sum takes what the feed-forward returns
+        ops.residual_norms(x, [torch.ones(W, device=where[0])], 1e-5, 1, dtype=where[1], **mod(h, fused))
+        assert rel_err(x, want) < (where[2] if where[1] == torch.float32 else 4e-2), fused
+
+
+@pytest.mark.parametrize("where", WHERE[:2])
+def test_few_tokens_of_many_experts(where):
+    """More pairs than experts, one expert that every token uses, experts nobody uses."""
+    E, M, W, dt, dev = 8, 64, 64, torch.bfloat16 if where[0] == "cuda" else torch.float32, where[0]
+    mod, cfg, sd = experts_module((dev, dt, 0), W, E, 3, 16, 1.0, 1.0, 1, 1, 8, 1.0)
+    h, h_o = act(rnd(M, W, seed=5), (dev, dt))
+    h_o[:, 0] = 4.0
+    for e, v in enumerate((9.0, -9.0, 0.0, 0.0, -9.0, 0.5, 0.0, 1.0)):   # expert 0 always, 1 and 4 never
+        sd["router"][e, 0] = v
+    h = h_o.to(dt).to(dev)
+    mod.router.weight.data[:E] = sd["router"].to(dt)
+    x = torch.zeros((M, W), dtype=torch.float32, device=dev)
+    ops.residual_norms(x, [torch.ones(W, device=dev)], 1e-5, 1, dtype=dt, **mod(h))
+    assert rel_err(x, O.moe(h_o, cfg, sd, "")) < (2e-5 if dev == "cpu" else 4e-2)
 
 
 # ------------------------------------------------------------------ generalised delta rule
@@ -484,6 +502,14 @@ def test_decode_shares_keys_between_heads(B, H, G):
     for n in ("k", "v", "pk", "pv"):
         assert rel_err(other[n].flatten(0, 2), a.cache[n].flatten(0, 2).cpu()) < 1e-5
     assert int(other["tickets"].abs().sum()) == 0
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("M", [1, 3, 4])
+def test_scaled_logits_of_a_few_rows(M):
+    w, x = (rnd(77, 48) * 48 ** -0.5).bfloat16(), rnd(M, 48, seed=1).bfloat16()
+    y = ops.decode_linear(w.cuda(), x.cuda(), epilogue="f32", alpha=0.3)
+    assert rel_err(y, x.double() @ w.double().T * 0.3) < 1e-4
 
 
 # ------------------------------------------------------------------ both side by side
