@@ -142,9 +142,9 @@ void channel_delta(Tensor proj, int64_t B, int64_t T, std::vector<int64_t> sizes
   TORCH_CHECK(p.nch <= 65535, "channel_delta: tokens of one step");
   const int64_t cells = B * p.nch * p.H;
   const int64_t piece = cells * C * p.DP;
-  Tensor buf = at::empty({6 * piece + cells * p.DP * (p.DP + 1)}, proj.options().dtype(at::kFloat));
+  Tensor buf = at::empty({7 * piece + cells * p.DP * (p.DP + 1)}, proj.options().dtype(at::kFloat));
   float* at = buf.data_ptr<float>();
-  for (float** q : {&p.cq, &p.co, &p.cw, &p.cy, &p.cb, &p.ck}) *q = at, at += piece;
+  for (float** q : {&p.cq, &p.co, &p.cw, &p.cy, &p.cb, &p.ck, &p.cv}) *q = at, at += piece;
   p.cs = at;
   p.ce = at + cells * p.DP * p.DP;
   check_rc(nxd::channel_delta_chunk_launch(f32, p, cur_stream()), "channel_delta_chunk");

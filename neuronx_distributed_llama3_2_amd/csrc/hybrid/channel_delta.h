@@ -22,7 +22,7 @@ struct ChannelDeltaParams {
   int64_t ldy;
   // chunks (channel_delta_chunk.hip), a cell = (sequence, chunk, head)
   int nch;
-  float *cq, *co, *cw, *cy, *cb, *ck;   // Q, O', W, Y, E B^T, E K^T [cells, C DP]
+  float *cq, *co, *cw, *cy, *cb, *ck, *cv;   // Q, O', W, Y, E B^T, E K^T, V [cells, C DP]
   float *cs, *ce;            // S_0 [cells, DP DP], E [cells, DP]
 };
 

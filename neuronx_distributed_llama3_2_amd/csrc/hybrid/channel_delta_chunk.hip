@@ -10,9 +10,10 @@
 //   O   = Q S_0 + O',            Q = R + A_rb W,  O' = A_rb Y + A_rk V
 //   S_1 = E S_0 + (E B^T) Z + (E K^T) V
 //
-//   prepare : Q, O', W, Y, E B^T, E K^T of every (sequence, chunk, head) in parallel
+//   prepare : Q, O', W, Y, E B^T, E K^T, V of every (sequence, chunk, head) in parallel
 //   scan    : Z and the next state, the chunks of a head one after another for 16 columns of the state; a
-//             wave has 16 rows of it, so W S_0 is summed over the waves, and nothing else is exchanged
+//             wave has 16 rows of it, so W S_0 is summed over the waves (by waves of their own, while the others
+//             multiply K^T V), and nothing else is exchanged
 //   output  : O = Q S_0 + O', the head norm and the gate
 //
 // A log decay lies in (-e^(-1/2), 0), so e^(-L) stays below e^39 in a chunk of 64 and every product of a
@@ -33,10 +34,28 @@ __device__ __forceinline__ f32x4_t mma4(const f32x4_t& a, const f32x4_t& b, f32x
   for (int i = 0; i < 4; ++i) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[i], b[i], c, 0, 0, 0);
   return c;
 }
+// N products, their steps interleaved (a step waits for the one before it in its own chain)
+template <int N, typename A, typename B>
+__device__ __forceinline__ void mma4_interleaved(A a, B b, f32x4_t (&c)[N]) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int n = 0; n < N; ++n) c[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(a(n)[i], b(n)[i], c[n], 0, 0, 0);
+}
 // 2^x for a sum x kept in fp64
 __device__ __forceinline__ float pow2(double x) {
   const double n = rint(x);
   return ldexpf(__builtin_amdgcn_exp2f((float)(x - n)), (int)n);
+}
+
+// a uniform base and a lane's offset in bytes: one address register a lane (the base is kept apart from the
+// offset by hand, or the loop gets a 64-bit address a lane for every load)
+template <typename V, typename P>
+__device__ __forceinline__ V at(const P* base, uint32_t bytes) {
+  typedef const __attribute__((address_space(1))) char* global_t;
+  global_t g = (global_t)(const char*)base;
+  asm("" : "+s"(g));
+  return *(const __attribute__((address_space(1))) V*)(g + bytes);
 }
 
 constexpr int RANK_TILE = 64;
@@ -96,7 +115,7 @@ __global__ void __launch_bounds__(512, CB == 2 ? 4 : 2) cdelta_prepare_kernel(Ch
   const int tv = w, tw = w >= NB ? w - NB : w + 8 - NB;
   const bool has_v = tv < NB && tv * 16 < D, has_w = tw < NB;
 
-  // ---- what comes from memory is on its way first: r, k, removal (8 elements a thread), v (this wave's columns)
+  // ---- r, k, removal are on their way first: 8 elements a thread
   const bool wide = D % 8 == 0 && p.ldp % 8 == 0 && reinterpret_cast<uintptr_t>(p.proj) % 16 == 0;
   const int rt = tid / (DP / 8), rc = tid % (DP / 8) * 8;
   Raw8<T> raw[3];
@@ -105,18 +124,6 @@ __global__ void __launch_bounds__(512, CB == 2 ? 4 : 2) cdelta_prepare_kernel(Ch
   if (wide && rt < n && rc < D) {
 #pragma unroll
     for (int j = 0; j < 3; ++j) raw[j].load(head + (int64_t)rt * p.ldp + (j == 0 ? 0 : (j == 1 ? HD : 4 * HD)) + rc);
-  }
-  f32x4_t v[CB];
-#pragma unroll
-  for (int bk = 0; bk < CB; ++bk) {
-    v[bk] = zero;
-    if (has_v) {
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = 16 * bk + 4 * lq + i, col = tv * 16 + lr;
-        if (t < n && col < D) v[bk][i] = ld(head + (int64_t)t * p.ldp + 2 * HD + col);
-      }
-    }
   }
 
   // ---- log decays: W2 tanh(low), tokens x channels.  job = (channel block, half of the tokens)
@@ -244,8 +251,20 @@ __global__ void __launch_bounds__(512, CB == 2 ? 4 : 2) cdelta_prepare_kernel(Ch
   }
   __syncthreads();
 
-  // ---- the lower blocks of the four products; the columns of U this wave solves for, before they go
+  // ---- the lower blocks of the four products; this wave's columns of V, and of U before they go
   auto piece = [&](int m, int row, int ch16) { return am + (m * C + row) * C + 4 * (ch16 ^ (row & (C / 4 - 1))); };
+  f32x4_t v[CB];
+#pragma unroll
+  for (int bk = 0; bk < CB; ++bk) {
+    v[bk] = zero;
+    if (has_v) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 16 * bk + 4 * lq + i, col = tv * 16 + lr;
+        if (t < n && col < D) v[bk][i] = ld(head + (int64_t)t * p.ldp + 2 * HD + col);
+      }
+    }
+  }
   f32x4_t prod[PW], uw[CB];
 #pragma unroll
   for (int j = 0; j < PW; ++j) {
@@ -286,18 +305,18 @@ __global__ void __launch_bounds__(512, CB == 2 ? 4 : 2) cdelta_prepare_kernel(Ch
   // ---- the diagonal blocks of I - A_ub, inverted in place by substitution: column lr
   if (w < CB) {
     float x[16];
-    auto at = [&](int i, int j) { return piece(0, 16 * w + i, 4 * w + (j >> 2)) + (j & 3); };
+    auto el = [&](int i, int j) { return piece(0, 16 * w + i, 4 * w + (j >> 2)) + (j & 3); };
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       float s = i == lr ? 1.f : 0.f;
 #pragma unroll
-      for (int j = 0; j < i; ++j) s += *at(i, j) * x[j];
+      for (int j = 0; j < i; ++j) s += *el(i, j) * x[j];
       x[i] = s;
     }
     __builtin_amdgcn_wave_barrier();
     if (lq == 0) {
 #pragma unroll
-      for (int i = 0; i < 16; ++i) *at(i, lr) = x[i];
+      for (int i = 0; i < 16; ++i) *el(i, lr) = x[i];
     }
   }
   // ---- E B^T and E K^T, A operands of the scan
@@ -322,6 +341,7 @@ __global__ void __launch_bounds__(512, CB == 2 ? 4 : 2) cdelta_prepare_kernel(Ch
     f32x4_t y[CB];
 #pragma unroll
     for (int bi = 0; bi < CB; ++bi) {
+      st4(p.cv + ((cell * NB + tv) * CB + bi) * 256 + lane * 4, v[bi]);
       f32x4_t r = zero;
 #pragma unroll
       for (int bk = 0; bk <= bi; ++bk) r = mma4(frag(1, bi, bk), v[bk], r);
@@ -364,84 +384,102 @@ __global__ void __launch_bounds__(512, CB == 2 ? 4 : 2) cdelta_prepare_kernel(Ch
   }
 }
 
-// 16 columns of one head's state, a wave for 16 rows.  A chunk's operands are fetched AHEAD chunks before.
-template <typename T, int NB, int CB>
-__global__ void __launch_bounds__(NB * 64) cdelta_scan_kernel(ChannelDeltaParams p) {
-  constexpr int DP = NB * 16, C = CB * 16, AHEAD = CB == 2 ? 4 : 2, RB = (CB + NB - 1) / NB;   // blocks of Z a wave sums
+// 16 columns of one head's state: a wave for 16 rows of it, and a wave for 16 tokens that sums the waves' parts
+// of W S_0.  A chunk's operands are fetched AHEAD chunks before.
+template <int NB, int CB>
+__global__ void __launch_bounds__((NB + CB) * 64) cdelta_scan_kernel(ChannelDeltaParams p) {
+  constexpr int DP = NB * 16, C = CB * 16, AHEAD = CB == 2 ? 3 : 2;
   __shared__ __attribute__((aligned(16))) f32x4_t part[NB][CB][64], zs[CB][64];
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6), lr = lane & 15, lq = lane >> 4;
   const int bh = blockIdx.x % (p.B * p.H), vt = blockIdx.x / (p.B * p.H);   // a head's columns on one XCD
   const int b = bh / p.H, h = bh % p.H, H = p.H, D = p.D, v = vt * 16 + lr;
   const int len = p.lens ? min(p.lens[b], p.T) : p.T;
   if (len <= 0) return;
+  const int nch = (len + C - 1) / C;
+  const int64_t NC = (int64_t)NB * CB * 256;   // floats of a cell's operand
+  const uint32_t l16 = lane * 16;
+  auto cell_of = [&](int c) { return ((int64_t)b * p.nch + min(c, nch - 1)) * H + h; };   // (past the end the last is read again)
+  if (w >= NB) {
+    const int blk = w - NB;
+    const float* y = p.cy + (vt * CB + blk) * 256;
+    f32x4_t set[AHEAD];
+#pragma unroll
+    for (int i = 0; i < AHEAD; ++i) set[i] = at<f32x4_t>(y + cell_of(i) * NC, l16);
+    auto chunk = [&](int c, f32x4_t& o) {
+      lds_barrier();
+      f32x4_t z = part[0][blk][lane];
+#pragma unroll
+      for (int j = 1; j < NB; ++j) z += part[j][blk][lane];
+      zs[blk][lane] = z + o;
+      __builtin_amdgcn_sched_barrier(0);   // a load ahead of the old value's last use would need a register of its own,
+      o = at<f32x4_t>(y + cell_of(c + AHEAD) * NC, l16);   // and a copy that waits for it
+      lds_barrier();
+    };
+    int c = 0;
+    for (; c + AHEAD <= nch; c += AHEAD) {
+#pragma unroll
+      for (int i = 0; i < AHEAD; ++i) chunk(c + i, set[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < AHEAD; ++i)
+      if (c + i < nch) chunk(c + i, set[i]);
+    return;
+  }
   const int slot = slot_of(p.slots, b, p.nslots);
   const int64_t p0 = pos_of(p.pos, p.pos_stride, b);
   float* state = p.state + (((int64_t)slot * H + h) * D + min(v, D - 1)) * DP + w * 16 + 4 * lq;
-  const T* vals = static_cast<const T*>(p.proj) + (int64_t)b * p.T * p.ldp + 2 * H * D + h * D + min(v, D - 1);
   const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
   f32x4_t S = zero;
   if (p0 > 0 && v < D) S = ld4(state);
-  const int nch = (len + C - 1) / C;
-  const int64_t NC = (int64_t)NB * CB * 256;   // floats of a cell's operand
   struct Ops {
-    f32x4_t w[CB], b[CB], k[CB], y[RB];
-    T v[CB][4];
-    float e[4];
+    f32x4_t w[CB], k[CB], v[CB], b[CB], e;
   };
   Ops set[AHEAD];
-  auto fetch = [&](int c, Ops& o) {   // (past the last chunk the last one is read again)
-    c = min(c, nch - 1);
-    const int64_t cell = ((int64_t)b * p.nch + c) * H + h, at = cell * NC + (int64_t)w * CB * 256 + lane * 4;
+  auto fetch_first = [&](int c, Ops& o) {
+    const int64_t cell = cell_of(c), first = cell * NC + w * CB * 256;   // (uniform)
 #pragma unroll
     for (int i = 0; i < CB; ++i) {
-      o.w[i] = ld4(p.cw + at + i * 256);
-      o.b[i] = ld4(p.cb + at + i * 256);
-      o.k[i] = ld4(p.ck + at + i * 256);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) o.v[i][j] = vals[(int64_t)min(c * C + 16 * i + 4 * lq + j, len - 1) * p.ldp];
+      o.w[i] = at<f32x4_t>(p.cw + first + i * 256, l16);
+      o.k[i] = at<f32x4_t>(p.ck + first + i * 256, l16);
+      o.v[i] = at<f32x4_t>(p.cv + cell * NC + (vt * CB + i) * 256, l16);
     }
+    o.e = at<f32x4_t>(p.ce + cell * DP + w * 16, lq * 16);
+  };
+  auto fetch_last = [&](int c, Ops& o) {
+    const float* src = p.cb + cell_of(c) * NC + w * CB * 256;
 #pragma unroll
-    for (int i = 0; i < RB; ++i)
-      if (w + NB * i < CB) o.y[i] = ld4(p.cy + cell * NC + ((int64_t)vt * CB + w + NB * i) * 256 + lane * 4);
-    const f32x4_t e = ld4(p.ce + cell * DP + w * 16 + 4 * lq);
-#pragma unroll
-    for (int j = 0; j < 4; ++j) o.e[j] = e[j];
+    for (int i = 0; i < CB; ++i) o.b[i] = at<f32x4_t>(src + i * 256, l16);
   };
 #pragma unroll
-  for (int i = 0; i < AHEAD; ++i) fetch(i, set[i]);
+  for (int i = 0; i < AHEAD; ++i) {
+    fetch_first(i, set[i]);
+    fetch_last(i, set[i]);
+  }
   auto chunk = [&](int c, Ops& o) {
-    const int64_t cell = ((int64_t)b * p.nch + c) * H + h;
+    f32x4_t z[CB];
 #pragma unroll
-    for (int i = 0; i < CB; ++i) part[w][i][lane] = mma4(o.w[i], S, zero);
-    st4(p.cs + ((cell * NB + vt) * NB + w) * 256 + lane * 4, S);
-    f32x4_t n0, n1 = zero;
+    for (int i = 0; i < CB; ++i) z[i] = zero;
+    mma4_interleaved<CB>([&](int i) { return o.w[i]; }, [&](int) { return S; }, z);
 #pragma unroll
-    for (int j = 0; j < 4; ++j) n0[j] = S[j] * o.e[j];
-#pragma unroll
-    for (int i = 0; i < CB; ++i) {   // (needs nothing of the other waves)
-      f32x4_t x;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) x[j] = c * C + 16 * i + 4 * lq + j < len && v < D ? ld(&o.v[i][j]) : 0.f;
-      n1 = mma4(o.k[i], x, n1);
-    }
+    for (int i = 0; i < CB; ++i) part[w][i][lane] = z[i];
+    *reinterpret_cast<f32x4_t*>(reinterpret_cast<char*>(p.cs + ((cell_of(c) * NB + vt) * NB + w) * 256) + l16) = S;
     lds_barrier();
+    z[0] = S * o.e;   // while the parts are summed: E S_0 + (E K^T) V
 #pragma unroll
-    for (int i = 0; i < RB; ++i) {
-      const int blk = w + NB * i;
-      if (blk >= CB) continue;
-      f32x4_t z = o.y[i];
-#pragma unroll
-      for (int j = 0; j < NB; ++j) z += part[j][blk][lane];
-      zs[blk][lane] = z;
-    }
+    for (int i = 1; i < CB; ++i) z[i] = zero;
+    mma4_interleaved<CB>([&](int i) { return o.k[i]; }, [&](int i) { return o.v[i]; }, z);
+    __builtin_amdgcn_sched_barrier(0);   // (as above)
+    fetch_first(c + AHEAD, o);
     lds_barrier();
+    f32x4_t x[CB];
 #pragma unroll
-    for (int i = 0; i < CB; ++i) {
-      if (i & 1) n1 = mma4(o.b[i], zs[i][lane], n1);
-      else n0 = mma4(o.b[i], zs[i][lane], n0);
-    }
-    S = n0 + n1;
-    fetch(c + AHEAD, o);
+    for (int i = 0; i < CB; ++i) x[i] = zs[i][lane];
+    mma4_interleaved<CB>([&](int i) { return o.b[i]; }, [&](int i) { return x[i]; }, z);
+    __builtin_amdgcn_sched_barrier(0);
+    fetch_last(c + AHEAD, o);
+    S = z[0];
+#pragma unroll
+    for (int i = 1; i < CB; ++i) S += z[i];
   };
   int c = 0;
   for (; c + AHEAD <= nch; c += AHEAD) {
@@ -514,7 +552,7 @@ static int run_chunk(const ChannelDeltaParams& p, hipStream_t s) {
   const dim3 grid((unsigned)p.H, (unsigned)p.nch, (unsigned)p.B);
   hipLaunchKernelGGL((cdelta_prepare_kernel<T, NB, CB>), grid, dim3(512), lds, s, p);
   if (hipGetLastError() != hipSuccess) return 1;
-  hipLaunchKernelGGL((cdelta_scan_kernel<T, NB, CB>), dim3((unsigned)(ceil_div(p.D, 16) * p.B * p.H)), dim3(NB * 64), 0, s, p);
+  hipLaunchKernelGGL((cdelta_scan_kernel<NB, CB>), dim3((unsigned)(ceil_div(p.D, 16) * p.B * p.H)), dim3((NB + CB) * 64), 0, s, p);
   if (hipGetLastError() != hipSuccess) return 1;
   hipLaunchKernelGGL((cdelta_output_kernel<T, NB, CB>), grid, dim3(CB * 64), 0, s, p);
   return hipGetLastError() == hipSuccess ? 0 : 1;
