@@ -15,6 +15,7 @@ int moe_route_launch(const RouterParams&, hipStream_t);
 int clamped_glu_launch(bool, const GluParams&, bool, hipStream_t);
 int gather_rows_launch(const void*, const int*, void*, int64_t, int64_t, int64_t, hipStream_t);
 int experts_few_launch(const RouterParams&, const ExpertFewParams&, hipStream_t);
+int linear_few_launch(const LinearFewParams&, hipStream_t);
 int expert_rows_launch(bool, const ExpertRowsParams&, hipStream_t);
 int grouped_gemm_launch(int, const void*, const void*, void*, const int*, int, int, int, int, int, hipStream_t);
 int grouped_rowgemm_launch(int, const void*, const void*, void*, const int*, int, int, int, int, hipStream_t);
@@ -266,7 +267,7 @@ void expert_rows(Tensor x, Tensor w, Tensor offs, Opt token, Tensor y) {
 
 // y [M (top + shared), W]: outputs of a token's experts, weighted, then its shared expert's
 void experts_few(Tensor h, Tensor router, std::vector<int64_t> rule, double scale, Tensor up, Tensor down, double limit, Opt sup,
-                 Opt sdown, double slimit, Tensor y) {
+                 Opt sdown, double slimit, Opt gate, Tensor y) {
   auto bf = [](const Tensor& t, int64_t d, const char* n) {
     TORCH_CHECK(t.is_cuda() && t.scalar_type() == at::kBFloat16 && t.dim() == d && t.is_contiguous(), "experts_few: ", n, ": contiguous bf16");
     check_align(t, n);
@@ -292,8 +293,10 @@ void experts_few(Tensor h, Tensor router, std::vector<int64_t> rule, double scal
     p.FS = (int)sdown->size(1);
     TORCH_CHECK(sup->size(0) == 2 * p.FS && sup->size(1) == p.W && sdown->size(0) == p.W, "experts_few: shared expert's shapes");
   }
-  TORCH_CHECK(p.M <= 64 && p.W % 8 == 0 && p.F % 8 == 0 && p.FS % 8 == 0 && p.F >= 8 && p.W >= 8, "experts_few: up to 64 tokens, sizes multiples of 8");
-  TORCH_CHECK(router.size(0) >= p.E + p.shared && router.size(1) == p.W, "experts_few: router [>= E + shared, W]");
+  TORCH_CHECK(p.M <= 64 && p.W % 8 == 0 && p.F % 8 == 0 && p.FS % 8 == 0 && p.F >= 8 && p.W >= 8 && p.W < (1 << 24) && (int64_t)p.M * p.top * p.F < (1LL << 31) && p.FS < (1 << 24), "experts_few: up to 64 tokens, sizes multiples of 8");
+  TORCH_CHECK(!(p.shared && gate.has_value()) && (!p.shared || p.M <= 16), "experts_few: the shared expert here (up to 16 tokens), or its gate");
+  p.gate = f32_opt(gate, p.M, "gate");
+  TORCH_CHECK(router.size(0) >= p.E + (p.shared || p.gate ? 1 : 0) && router.size(1) == p.W, "experts_few: router [>= E + shared, W]");
   TORCH_CHECK(up.size(0) == p.E && up.size(1) == 2 * p.F && up.size(2) == p.W && down.size(0) == p.E && down.size(1) == p.W, "experts_few: experts' shapes");
   const int64_t slots = p.top + p.shared;
   p.y = bf(y, 2, "y");
@@ -309,6 +312,27 @@ void experts_few(Tensor h, Tensor router, std::vector<int64_t> rule, double scal
   check_rc(nxd::experts_few_launch(r, p, cur_stream()), "experts_few");
 }
 
+// y [M, N] = x [M, K] w^T, up to 16 rows
+void linear_few(Tensor x, Tensor w, Tensor y) {
+  for (const Tensor* t : {&x, &w, &y})
+    TORCH_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16 && t->dim() == 2 && t->stride(1) == 1, "linear_few: bf16 matrices");
+  nxd::LinearFewParams p{};
+  p.M = (int)x.size(0);
+  p.K = (int)x.size(1);
+  p.N = (int)w.size(0);
+  TORCH_CHECK(p.M >= 1 && p.M <= 16 && p.K >= 8 && p.K % 8 == 0 && p.N >= 1 && x.stride(0) < (1 << 24), "linear_few: 1..16 rows, K a multiple of 8");
+  TORCH_CHECK(w.is_contiguous() && w.size(1) == p.K && y.size(0) == p.M && y.size(1) == p.N && x.stride(0) % 8 == 0, "linear_few: shapes");
+  check_align(x, "x");
+  check_align(w, "w");
+  check_align(y, "y");
+  p.x = static_cast<const uint16_t*>(x.data_ptr());
+  p.ldx = x.stride(0);
+  p.w = static_cast<const uint16_t*>(w.data_ptr());
+  p.y = static_cast<uint16_t*>(y.data_ptr());
+  p.ldy = y.stride(0);
+  check_rc(nxd::linear_few_launch(p, cur_stream()), "linear_few");
+}
+
 }  // namespace
 
 void register_parallel(pybind11::module& m) {
@@ -320,4 +344,5 @@ void register_parallel(pybind11::module& m) {
   m.def("grouped_linear", &grouped_linear);
   m.def("expert_rows", &expert_rows);
   m.def("experts_few", &experts_few);
+  m.def("linear_few", &linear_few);
 }

@@ -46,6 +46,15 @@ struct ExpertRowsParams {
 };
 
 // a few tokens (expert_decode.hip)
+struct LinearFewParams {
+  int M, N, K;
+  const uint16_t* x;       // [M, ldx]
+  int64_t ldx;
+  const uint16_t* w;       // [N, K]
+  uint16_t* y;             // [M, ldy]
+  int64_t ldy;
+};
+
 struct ExpertFewParams {
   int M, E, top, shared;   // shared: 1 with a shared expert (else 0)
   int W, F, FS;            // width, feed-forward sizes
@@ -55,6 +64,7 @@ struct ExpertFewParams {
   float limit, slimit;
   int* index;              // [M, top]
   float* score;            // [M, top + shared]
+  float* gate;             // [M] the shared expert's gate, for a caller that runs it (nullable)
   uint16_t *a, *sa;        // [M top, F], [M, FS]
   uint16_t* y;             // [M (top + shared), W]
 };

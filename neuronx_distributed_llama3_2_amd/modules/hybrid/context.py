@@ -31,24 +31,23 @@ def padded_rows(n: int) -> int:
     return (n + ROW_ALIGN - 1) // ROW_ALIGN * ROW_ALIGN
 
 
-# rows up to which a projection streams its weights (csrc/hybrid/gemv_hyper.hip)
-FEW_ROWS = 4
+# rows up to which a projection is a dot product a wave (csrc/hybrid/gemv_hyper.hip), and up to which it is
+# 16 weight rows a workgroup (csrc/hybrid/expert_decode.hip)
+FEW_ROWS, SOME_ROWS = 2, 16
 
 
-def few_rows(x: torch.Tensor, w: torch.Tensor) -> bool:
-    return x.is_cuda and x.shape[0] <= FEW_ROWS and x.dtype == w.dtype == torch.bfloat16 and w.shape[1] % 8 == 0 and \
-        x.is_contiguous()
+def few_rows(x: torch.Tensor, w: torch.Tensor, limit: int = FEW_ROWS) -> bool:
+    return x.is_cuda and x.shape[0] <= limit and x.dtype == w.dtype == torch.bfloat16 and w.shape[1] % 8 == 0 and x.is_contiguous()
 
 
 def linear(x: torch.Tensor, mod: torch.nn.Module, fused: bool = False) -> torch.Tensor:
     """x [M, K] @ mod.weight^T: through the module's packed copy when the layout pass chose it; fused: a few
-    rows by the decode kernel."""
+    rows by the kernels that stream the weights."""
     from ... import ops
     from ...trace.weight_layout import packed_linear
 
-    if fused and few_rows(x, mod.weight):
-        return ops.decode_linear(mod.weight, x)
-
+    if fused and few_rows(x, mod.weight, SOME_ROWS):
+        return ops.decode_linear(mod.weight, x) if x.shape[0] <= FEW_ROWS else ops.linear_few(x, mod.weight)
     return packed_linear(mod, x, mod.weight)
 
 

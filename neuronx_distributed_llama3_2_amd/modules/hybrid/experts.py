@@ -9,7 +9,7 @@ import torch
 import torch.nn as nn
 
 from ... import ops
-from ...ops.experts import RouterRule
+from ...ops.experts import FEW_ROWS, RouterRule
 from ...ops.gemm import linear_f32
 from .context import linear, padded_rows
 
@@ -40,13 +40,18 @@ class RoutedExperts(nn.Module):
         where each is, and the shared expert's output.  fused: a few tokens take the unsorted kernels."""
         shared = (self.shared_up.weight, self.shared_down.weight) if self.shared_up is not None else (None, None)
         if fused and ops.experts_few_supported(h, self.gate_up, self.down, *shared):
-            return dict(pairs=ops.experts_few(h, self.router.weight, self.rule, self.gate_up, self.down, self.limit, *shared,
-                                              self.shared_limit), adds=[])
+            inside = h.shape[0] <= FEW_ROWS
+            gate = torch.empty(h.shape[0], dtype=torch.float32, device=h.device) if shared[0] is not None and not inside else None
+            pairs = ops.experts_few(h, self.router.weight, self.rule, self.gate_up, self.down, self.limit,
+                                    *(shared if inside else (None, None)), self.shared_limit, gate)
+            return dict(pairs=pairs, adds=[] if gate is None else [self._shared(h, gate, False)])
         logits = linear_f32(h, self.router.weight)
         r = ops.route(logits, self.rule)
         a = ops.clamped_glu(ops.expert_linear_rows(h, self.gate_up, r.offs, r.token), self.limit, r.weight)
         out: Dict[str, object] = dict(pairs=ops.expert_linear_rows(a, self.down, r.offs), inverse=r.inverse, adds=[])
         if self.shared_up is not None:
-            a = ops.clamped_glu(linear(h, self.shared_up), self.shared_limit, logits[:, self.rule.experts], sigmoid=True)
-            out["adds"] = [linear(a, self.shared_down)]
+            out["adds"] = [self._shared(h, logits[:, self.rule.experts], True)]
         return out
+
+    def _shared(self, h: torch.Tensor, gate: torch.Tensor, sigmoid: bool) -> torch.Tensor:
+        return linear(ops.clamped_glu(linear(h, self.shared_up), self.shared_limit, gate, sigmoid=sigmoid), self.shared_down)

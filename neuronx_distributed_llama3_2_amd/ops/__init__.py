@@ -9,7 +9,7 @@ from .decode import argmax_rows, decode_attention, greedy_advance_, kv_cache_wri
 from .delta_rule import DeltaSizes, delta_rule  # noqa: F401
 from .embedding import vocab_parallel_embedding  # noqa: F401
 from .experts import (RouterRule, Routing, clamped_glu, expert_linear_rows, experts_few, experts_few_supported,  # noqa: F401
-                      route)
+                      linear_few, route)
 from .group_norm import residual_norms  # noqa: F401
 from .grouped_gemm import (grouped_linear, grouped_linear_reference, moe_dispatch, moe_permutation,  # noqa: F401
                            moe_unpermute_combine)

@@ -101,8 +101,16 @@ def expert_linear_rows(x: torch.Tensor, w: torch.Tensor, offs: torch.Tensor, tok
     return y
 
 
-# tokens up to which the experts run unsorted (csrc/hybrid/expert_decode.hip)
-FEW_TOKENS = 64
+# tokens up to which the experts run unsorted, and up to which dense weights are streamed beside them
+# (csrc/hybrid/expert_decode.hip)
+FEW_TOKENS, FEW_ROWS = 64, 16
+
+
+def linear_few(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x [M, K] w^T for up to FEW_ROWS rows (GPU, bf16, K a multiple of 8): the weights are streamed once."""
+    y = torch.empty((x.shape[0], w.shape[0]), dtype=x.dtype, device=x.device)
+    hybrid_ext().linear_few(x, w, y)
+    return y
 
 
 def experts_few_supported(h: torch.Tensor, *weights: Optional[torch.Tensor]) -> bool:
@@ -112,12 +120,13 @@ def experts_few_supported(h: torch.Tensor, *weights: Optional[torch.Tensor]) -> 
 
 def experts_few(h: torch.Tensor, router: torch.Tensor, rule: RouterRule, gate_up: torch.Tensor, down: torch.Tensor, limit: float,
                 shared_up: Optional[torch.Tensor] = None, shared_down: Optional[torch.Tensor] = None,
-                shared_limit: float = 0.0) -> torch.Tensor:
+                shared_limit: float = 0.0, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """A whole routed feed-forward for a few tokens (GPU, bf16) in three launches.  router [>= E (+ 1), W]: the
     experts' rows, then the shared expert's gate.  Returns [M (top + 1), W]: for each token its experts'
-    weighted outputs and then its shared expert's; their sum is the feed-forward's output."""
+    weighted outputs and then its shared expert's; their sum is the feed-forward's output.  gate (fp32 [M],
+    instead of the shared expert's weights): receives its gate, and the rows are the experts' alone."""
     slots = rule.top + (0 if shared_up is None else 1)
     y = torch.empty((h.shape[0] * slots, h.shape[1]), dtype=h.dtype, device=h.device)
     hybrid_ext().experts_few(h, router, rule.as_list(), rule.scale, gate_up, down, float(limit), shared_up, shared_down,
-                             float(shared_limit), y)
+                             float(shared_limit), gate, y)
     return y

@@ -505,6 +505,14 @@ def test_decode_shares_keys_between_heads(B, H, G):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("M", [1, 5, 8, 16])
+@pytest.mark.parametrize("N,K", [(48, 72), (33, 8), (200, 2048), (1000, 1000), (16, 4096)])
+def test_products_of_some_rows(M, N, K):
+    w, x = (rnd(N, K) * K ** -0.5).bfloat16(), rnd(M, K, seed=1).bfloat16()
+    assert rel_err(ops.linear_few(x.cuda(), w.cuda()), x.double() @ w.double().T) < 8e-3
+
+
+@pytest.mark.gpu
 @pytest.mark.parametrize("M", [1, 3, 4])
 def test_scaled_logits_of_a_few_rows(M):
     w, x = (rnd(77, 48) * 48 ** -0.5).bfloat16(), rnd(M, 48, seed=1).bfloat16()
