@@ -378,3 +378,13 @@ def test_command_line(model_dirs, tmp_path, capsys):
          runner_cls=BezuraxRunner)
     rows = main(["generate", "--traced_path", out, "--prompt_ids", ",".join(map(str, tokens(8, 211)))], runner_cls=BezuraxRunner)
     assert rows.shape == (1, 14) and rows[0, :8].tolist() == tokens(8, 211)
+
+
+def test_benchmark_configurations():
+    """bench.py --serve: a token uses as many feed-forward parameters as in the Llama models beside it."""
+    from neuronx_distributed_llama3_2_amd.inference.serve_bench import SIZES, bezurax_config
+
+    for size, ff, layers in zip(SIZES, (8192, 14336), (16, 8)):
+        cfg = BezuraxConfig(bezurax_config(size))
+        m = cfg.layers[0].mlp
+        assert m.top * m.ff + m.shared_ff == ff and cfg.num_hidden_layers == layers
