@@ -73,7 +73,7 @@ def test_norm_of_small_rows_needs_eps_inside_the_root(where):
 
 # ------------------------------------------------------------------ router and experts
 def router_cases():
-    return [(6, 2, 3, 2, 1.7), (8, 4, 2, 1, 2.0), (4, 1, 4, 2, 1.0), (1, 1, 1, 1, 0.5), (5, 5, 1, 1, 1.0), (128, 8, 8, 4, 2.5),
+    return [(6, 2, 3, 2, 1.7), (10, 4, 2, 1, 2.2), (4, 1, 4, 2, 1.0), (1, 1, 1, 1, 0.5), (5, 5, 1, 1, 1.0), (128, 8, 8, 4, 2.5),
             (96, 6, 1, 1, 1.0), (12, 4, 6, 3, 3.0)]
 
 
@@ -164,7 +164,7 @@ def experts_module(where, W, E, top, ff, limit, scale, groups, keep, shared_ff, 
     return mod, cfg, sd
 
 
-MOES = [(48, 6, 2, 24, 1.2, 1.7, 3, 2, 40, 0.8), (64, 8, 4, 32, 0.6, 2.0, 2, 1, 64, 1.5), (36, 5, 5, 17, 1.0, 1.0, 1, 1, 0, 0.0),
+MOES = [(48, 6, 2, 24, 1.2, 1.7, 3, 2, 40, 0.8), (64, 10, 4, 32, 0.6, 2.2, 2, 1, 64, 1.1), (36, 5, 5, 17, 1.0, 1.0, 1, 1, 0, 0.0),
         (128, 16, 3, 64, 7.0, 1.0, 4, 2, 128, 7.0), (64, 1, 1, 8, 1.0, 0.5, 1, 1, 24, 0.3)]
 
 
@@ -248,7 +248,7 @@ def stale_state(where, slots, sz, value=5.0):
     return state
 
 
-SIZES = [(1, 8, 1), (3, 20, 7), (2, 33, 70), (2, 48, 16), (1, 64, 64), (2, 72, 130), (1, 128, 32), (1, 136, 9), (1, 250, 3)]
+SIZES = [(1, 8, 1), (3, 20, 7), (2, 33, 70), (2, 56, 12), (1, 64, 64), (2, 72, 130), (1, 128, 32), (1, 136, 9), (1, 250, 3)]
 
 
 @pytest.mark.parametrize("where", WHERE)
